@@ -1,8 +1,9 @@
 """Forward passes of configuration-driven designs (models/muderax.py, models/surodra.py, models/dironex.py,
-models/murulorn.py) on the layer-mechanism kernels (ops/layers.py).  Four block styles share the runner: sandwich
-norms on a sublayer's output (Muderax, described first), pre-norm blocks around matrix-state mixers (Surodra,
-described after it), pre-norm blocks on several residual streams (Dironex) and blocks with a norm before and after
-each sublayer plus a per-layer token input (Murulorn, described last).
+models/murulorn.py, models/kagorax.py) on the layer-mechanism kernels (ops/layers.py).  Five block styles share the
+runner: sandwich norms on a sublayer's output (Muderax, described first), pre-norm blocks around matrix-state mixers
+(Surodra, described after it), pre-norm blocks on several residual streams (Dironex), blocks with a norm before and
+after each sublayer plus a per-layer token input (Murulorn) and blocks whose mixer and feed-forward read one norm side by
+side (Kagorax, described last).
 
 A step is a set of packed rows -- the B decode slots first (one row each, state on the device as in ModelRunner), then
 the rows of prompt portions -- that walk the layer list once:
@@ -80,6 +81,19 @@ The bracket-norm walk (`_bracket_layers`) also goes over layer runs:
 A decode row's token becomes its slot's previous token inside embed_pair_rows (the captured graph carries it); prompt
 portions bring each row's predecessor with them (PrefillSeq.prev_token for the first row).
 
+The joint walk (`_joint_layers`), one norm per layer:
+
+    embed_rows              stream = embed[token] * scale + the position's vector
+    add_norm_rows           between layers: stream += mixer output + the experts' slots; h = rms-norm(stream) * gain, also
+                            fp32 for the router
+    attention               ONE fused GEMM [q | k | v | g] ([q | g] in a layer that attends to another layer's keys and
+                            values) -> qkv_rows (biases, q and k divided by their rms per head, k and v into the layer's
+                            pages) -> sink_attention with a distance bias, a window that keeps the first keys and an
+                            element-wise sigmoid gate, over this layer's pages or the other layer's -> output GEMM
+    feed-forward            router GEMM in fp32 (the shared expert's gate is one more row) -> moe_route (sigmoid scores as
+                            they are) -> moe_grouped with the weights on the experts' inputs
+    head                    add_norm_rows (final norm) -> GEMM on the embedding table
+
 The residual stream, norms, scores, router and recurrence are fp32 in both element types; ``dtype=torch.float32`` runs
 the projections in true fp32 as well (the exact mode).  The cache is paged with the engine's block tables and
 allocator (LatentKVCache, PagedKVCache, both at once in MixedKVCache); recurrent layers and input convolutions keep
@@ -130,7 +144,10 @@ class LayeredRunner(RunnerBase):
         self.prenorm = getattr(cfg, "family", "") == "surodra"   # pre-norm blocks with matrix-state mixers
         self.multistream = getattr(cfg, "family", "") == "dironex"  # pre-norm blocks on several residual streams
         self.bracket = getattr(cfg, "family", "") == "murulorn"    # a norm before and after each sublayer, token inputs
-        if self.bracket:
+        self.joint = getattr(cfg, "family", "") == "kagorax"       # one norm feeds the mixer and the feed-forward
+        if self.joint:
+            self._setup_joint()
+        elif self.bracket:
             self._setup_bracket()
         elif self.multistream:
             self._setup_streams()
@@ -187,6 +204,9 @@ class LayeredRunner(RunnerBase):
         el = dict(device=dev, dtype=self.dtype)
         W = cfg.width
         d = {"resid": torch.zeros(M, W, **f32), "xb": torch.zeros(M, W, **el), "y": torch.zeros(M, W, **f32)}
+        if self.joint:
+            d.update(self._joint_buffers(M))
+            return d
         if self.bracket:
             d.update(self._bracket_buffers(M))
             return d
@@ -319,6 +339,9 @@ class LayeredRunner(RunnerBase):
         prev: (previous token per row, where decode rows store their own token, which of them do) for designs whose
         embedding reads the previous token."""
         cfg, eps = self.cfg, self.cfg.eps
+        if self.joint:
+            self._joint_layers(M, d, ids, pos, slots, groups, trace)
+            return
         if self.bracket:
             self._bracket_layers(M, d, ids, prev, pos, slots, groups, trace)
             return
@@ -348,7 +371,7 @@ class LayeredRunner(RunnerBase):
         self._head(rows, xn, logits)
 
     def _head(self, resid, xn, logits) -> None:
-        if self.bracket:
+        if self.bracket or self.joint:
             ops.add_norm_rows(None, 1, None, resid, self.w.final_norm, self.cfg.eps, xn)
             self._lin(xn, self.w.head, self.w.head_t, logits)
         elif self.multistream:  # resid holds the sum of the streams: one stream with weight 1 through the RMS norm
@@ -954,6 +977,105 @@ class LayeredRunner(RunnerBase):
         ops.moe_grouped(d["xb"], tki, tkw, None, Fw.up, Fw.down, None, None, None, d["mo_sorted"], d["mo_tile"],
                         d["mo_n"], d["mo_h"], o)
         return o, f.top
+
+    # ------------------------------------------------------------------ mixer and feed-forward side by side
+    def _setup_joint(self) -> None:
+        """Pages of the layers that have keys and values of their own (a layer that attends to another layer's has none),
+        and the position vectors of the embedding."""
+        from ..models.kagorax import position_table
+
+        cfg, dev = self.cfg, self.device
+        kv = {i: (L.mixer.kv_heads, L.mixer.dim, L.mixer.vdim) for i, L in enumerate(cfg.layers) if cfg.kv_layer(i) == i}
+        flash = [i for i, (_, dm, v) in kv.items() if ops.sink_flash_ok(self.dtype, dm, v)]
+        self.kv = PagedKVCache(kv, self.num_blocks, dev, self.dtype, transposed=flash)
+        self.state = MatrixStateCache({}, self.max_batch, dev)  # no layer keeps state beside its pages
+        self._pos_table = position_table(self.max_model_len + 1, cfg.width, dev)
+
+    def _joint_buffers(self, M: int) -> dict:
+        """Scratch of a step of M rows, each sized for the widest layer: `big` the fused projection's fp32 output, `qa`
+        the normed queries, `ao` the gated heads in the element type, `hn` the fp32 normed row the router reads, and the
+        experts' lists (slots = top + 1 with a shared expert)."""
+        cfg, dev = self.cfg, self.device
+        f32 = dict(device=dev, dtype=torch.float32)
+        el = dict(device=dev, dtype=self.dtype)
+        i32 = dict(device=dev, dtype=torch.int32)
+        W = cfg.width
+        big = max(Lw.mix.n_big for Lw in self.w.layers)
+        qa = max(L.mixer.heads * L.mixer.dim for L in cfg.layers)
+        ao = max(L.mixer.heads * L.mixer.vdim for L in cfg.layers)
+        moe = [L.mlp for L in cfg.layers if L.mlp is not None]
+        d = {"big": torch.zeros(M * big, **f32), "qa": torch.zeros(M * qa, **f32), "ao": torch.zeros(M * ao, **el),
+             "hn": torch.zeros(M, W, **f32) if moe else None}
+        if moe:
+            slots = max(f.top + (1 if f.shared_ff else 0) for f in moe)
+            experts = max(f.experts for f in moe)
+            tiles = -(-M * slots // 64) + experts + 2
+            ldh = -(-max(max(f.ff, f.shared_ff) for f in moe) // 8) * 8
+            d.update({"tki": torch.zeros(M * slots, **i32), "tkw": torch.zeros(M * slots, **f32),
+                      "mo_z": torch.zeros(M * (experts + 1), **f32), "mo_sorted": torch.zeros(tiles * 64, **i32),
+                      "mo_tile": torch.zeros(tiles, **i32), "mo_n": torch.zeros(1, **i32),
+                      "mo_h": torch.zeros(M * slots, ldh, **el), "mo_o": torch.zeros(M * slots * W, **f32)})
+        return d
+
+    def _joint_layers(self, M: int, d: dict, ids, pos, slots, groups: list, trace: list | None) -> None:
+        """Every layer over M packed rows.  Between layers ONE add_norm_rows adds both sublayers' outputs to the stream and
+        norms it for the next layer; the last outputs are added before the head's norm."""
+        cfg, w, eps = self.cfg, self.w, self.cfg.eps
+        ops.embed_rows(ids, w.embed, d["resid"], None, cfg.embed_scale, pos, self._pos_table)
+        pending = (None, 1, None)  # sublayer outputs that are not in the stream yet: (rows, parts per row, second rows)
+        for i, (L, Lw) in enumerate(zip(cfg.layers, w.layers)):
+            y, nsum, y2 = pending
+            ops.add_norm_rows(y, nsum, None, d["resid"], Lw.norm1, eps, d["xb"], d["hn"] if L.mlp is not None else None, y2)
+            self._attention_joint(i, L.mixer, Lw.mix, M, d, slots, groups)
+            pending = (d["y"], 1, None) if L.mlp is None else self._input_weighted_ff(L.mlp, Lw.mlp, M, d) + (d["y"],)
+            if trace is not None:
+                ops.add_norm_rows(pending[0], pending[1], None, d["resid"], None, eps, y2=pending[2])
+                pending = (None, 1, None)
+                trace.append(d["resid"].clone())
+        if pending[0] is not None:
+            ops.add_norm_rows(pending[0], pending[1], None, d["resid"], None, eps, y2=pending[2])
+
+    def _attention_joint(self, li: int, m, Lw, M: int, d: dict, slots, groups: list) -> None:
+        """Windowed attention with a distance bias over this layer's pages, or over those of the layer it takes keys and
+        values from (that layer has written this step's rows before)."""
+        H, G, D, V = m.heads, m.kv_heads, m.dim, m.vdim
+        src = self.cfg.kv_layer(li)
+        kc, vc, vt = self.kv.k[src], self.kv.v[src], self.kv.vt.get(src)
+        own = src == li
+        big = d["big"][:M * Lw.n_big].view(M, Lw.n_big)
+        self._lin(d["xb"], Lw.big, Lw.big_t, big)
+        qa = d["qa"][:M * H * D].view(M, H, D)
+        ops.qkv_rows(big, Lw.bias, H, G, D, V, self.cfg.eps, slots, qa, kc if own else None, vc if own else None,
+                     vt if own else None)
+        c0 = H * D + (G * (D + V) if own else 0)
+        gate = big[:, c0:c0 + H * V]
+        ao = d["ao"][:M * H * V].view(M, H, V)
+        for g in groups:
+            if vt is not None and g["qt"] > 1:
+                work, form = (g["hs"], g["ht"]), (SINK_ROWS_TILE, vt, False)
+            elif vt is not None and V <= ops.layers.SINK_SPLIT_MAX_V:
+                work, form = (g["ws"], g["wt"]), (SINK_ROWS_TILE, vt, True)
+            else:
+                work, form = (g["ws"], g["wt"]), (g["qt"], None, False)
+            ops.sink_attention(qa, kc, vc, g["bt"], g["qs"], g["ql"], g["ctx"], *work, None, gate, ao, m.window, m.scale,
+                               *form, rel=Lw.rel, keep_first=m.keep_first)
+        self._lin(ao.view(M, H * V), Lw.o, Lw.o_t, d["y"])
+
+    def _input_weighted_ff(self, f, Fw, M: int, d: dict):
+        """Router GEMM in true fp32 on the fp32 normed row (the shared expert's gate is its last column) -> the largest
+        sigmoid scores, used as they are -> grouped gated-SiLU experts with the weights on their inputs, the shared expert
+        as one more slot with its gate on the output; returns (per-slot outputs [M * S, W] fp32, S)."""
+        shared = f.shared_ff > 0
+        S, W, E = f.top + shared, self.cfg.width, f.experts + shared
+        tki = d["tki"][:M * f.top].view(M, f.top)
+        tkw = d["tkw"][:M * S].view(M, S)
+        o = d["mo_o"][:M * S * W].view(M * S, W)
+        z = d["mo_z"][:M * E].view(M, E)
+        ops.gemm_rm(d["hn"], Fw.router, z)
+        ops.moe_route(z, None, tki, tkw, 1, 1, 1.0, 2)
+        ops.moe_grouped(d["xb"], tki, tkw, Fw.gate, Fw.up, Fw.down, Fw.sgate, Fw.sup, Fw.sdown, d["mo_sorted"], d["mo_tile"],
+                        d["mo_n"], d["mo_h"], o, True)
+        return o, S
 
     def _remember_last(self, seqs: list, g: dict) -> None:
         """After prompt portions: every portion's last token becomes its slot's previous token."""

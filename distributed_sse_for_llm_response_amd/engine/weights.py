@@ -857,3 +857,96 @@ def load_murulorn_dir(cfg, path: str, device="cpu", dtype=torch.bfloat16) -> Lay
     for f in sorted(Path(path).glob("*.safetensors")):
         tensors.update(load_file(str(f)))
     return convert_murulorn(cfg, tensors, device=device, dtype=dtype)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Designs whose mixer and feed-forward read one norm side by side (models/kagorax.py).  Projections of the mixer that
+# read the same input are ONE weight, as for the other configuration-driven families; gains, projection biases, the
+# router (with the shared expert's gate as its last row: one fp32 GEMM makes both) and the distance biases, laid out per
+# head and distance, are fp32 in both element types.
+@dataclass
+class BiasedAttentionWeights:
+    big: torch.Tensor        # rows [q (H D) | k (G D) | v (G V) | g (H V) | zero rows] x W; no k and v rows in a layer that
+                             # attends to another layer's keys and values
+    n_big: int
+    bias: torch.Tensor       # [H D + G D + G V] (or [H D]) fp32: the biases of q | k | v
+    rel: torch.Tensor        # [H, distances] fp32: score bias per head and distance, the last entry for all larger ones
+    o: torch.Tensor          # [W, H V]
+    big_t: torch.Tensor = None
+    o_t: torch.Tensor = None
+
+
+@dataclass
+class InputWeightedMoeWeights:
+    router: torch.Tensor     # [E (+ 1: the shared expert's gate), W] fp32 in both element types
+    gate: torch.Tensor       # [E, F, W]
+    up: torch.Tensor
+    down: torch.Tensor       # [E, W, F]
+    sgate: torch.Tensor = None
+    sup: torch.Tensor = None
+    sdown: torch.Tensor = None
+
+
+@dataclass
+class SideBySideLayer:
+    norm1: torch.Tensor      # [W] fp32
+    mix: BiasedAttentionWeights
+    mlp: InputWeightedMoeWeights = None
+
+
+@torch.no_grad()
+def convert_kagorax(cfg, tensors: dict, device="cpu", dtype=torch.bfloat16) -> LayeredWeights:
+    """Checkpoint tensors {name: tensor} (models/kagorax.py tensor_shapes) -> the engine's grouped layout in `dtype`."""
+    from ..models.kagorax import ANY, bias_by_distance, tensor_shapes
+
+    for name, shape in tensor_shapes(cfg).items():
+        if name not in tensors:
+            raise KeyError(f"checkpoint lacks tensor {name!r}")
+        got = tuple(tensors[name].shape)
+        if len(got) != len(shape) or any(s != ANY and s != g for s, g in zip(shape, got)):
+            raise ValueError(f"tensor {name!r} has shape {got}, the configuration says {shape}")
+
+    def t(name):
+        return tensors[name].to(device=device, dtype=dtype).contiguous()
+
+    def f(name):
+        return tensors[name].to(device=device, dtype=torch.float32).contiguous()
+
+    layers = []
+    for i, L in enumerate(cfg.layers):
+        p, fs = f"l{i}.", L.mlp
+        qkv = ("q", "k", "v") if L.mixer.kv_from == ANY else ("q",)
+        big = torch.cat([t(f"{p}mix.{n}") for n in qkv + ("g",)], dim=0)
+        if big.shape[0] >= TILED_MIN and big.shape[0] % 128:
+            big = torch.cat([big, big.new_zeros(128 - big.shape[0] % 128, big.shape[1])], dim=0)
+        mix = BiasedAttentionWeights(big=big.contiguous(), n_big=big.shape[0],
+                                     bias=torch.cat([f(f"{p}mix.{n}.b") for n in qkv]).contiguous(),
+                                     rel=bias_by_distance(f(p + "mix.rel"), L.mixer.bias_max), o=t(p + "mix.o"))
+        _tile_fields(mix, ("big", "o"))
+        layer = SideBySideLayer(norm1=f(p + "norm1"), mix=mix)
+        if fs is not None:
+            stack = lambda leaf: torch.stack([t(f"{p}mlp.e{e}.{leaf}") for e in range(fs.experts)]).contiguous()  # noqa: E731
+            router = [f(p + "mlp.router")] + ([f(p + "mlp.shared.sg")] if fs.shared_ff else [])
+            layer.mlp = InputWeightedMoeWeights(router=torch.cat(router).contiguous(), gate=stack("gate"), up=stack("up"),
+                                                down=stack("down"))
+            if fs.shared_ff:
+                layer.mlp.sgate, layer.mlp.sup, layer.mlp.sdown = (t(f"{p}mlp.shared.{leaf}")
+                                                                   for leaf in ("gate", "up", "down"))
+        layers.append(layer)
+    embed = t("embed")
+    out = LayeredWeights(cfg=cfg, embed=embed, layers=layers, final_norm=f("final.norm"), head=embed, dtype=dtype)
+    if fits_tiled(embed):    # the head is the embedding table: the gather keeps the row-major copy
+        out.head_t, out.head = tile_weight(embed), None
+    return out
+
+
+def load_kagorax_dir(cfg, path: str, device="cpu", dtype=torch.bfloat16) -> LayeredWeights:
+    """``*.safetensors`` of a checkpoint directory -> the engine's layout (the loader executes nothing from them)."""
+    from pathlib import Path
+
+    from safetensors.torch import load_file
+
+    tensors = {}
+    for f in sorted(Path(path).glob("*.safetensors")):
+        tensors.update(load_file(str(f)))
+    return convert_kagorax(cfg, tensors, device=device, dtype=dtype)

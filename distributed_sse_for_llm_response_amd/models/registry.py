@@ -156,13 +156,37 @@ def _murulorn() -> Family:
                   (torch.bfloat16, torch.float32))
 
 
+def _kagorax() -> Family:
+    from . import kagorax as K
+
+    def random_weights(cfg, device, dtype, seed, tp_rank, tp_size):
+        from ..engine.weights import convert_kagorax
+
+        cfg.validate(tp_size)
+        return convert_kagorax(cfg, K.init_weights(cfg, seed=seed, device=device), device=device, dtype=dtype)
+
+    def load_dir(cfg, path, device, dtype, tp_rank, tp_size):
+        from ..engine.weights import load_kagorax_dir
+
+        cfg.validate(tp_size)
+        return load_kagorax_dir(cfg, path, device=device, dtype=dtype)
+
+    def runner():
+        from ..engine.layered_runner import LayeredRunner
+
+        return LayeredRunner
+
+    return Family("kagorax", ("Kagorax",), K.KagoraxConfig.from_dict, dict(K.CONFIGS), random_weights, load_dir, runner,
+                  (torch.bfloat16, torch.float32))
+
+
 _FAMILIES = None
 
 
 def families() -> dict:
     global _FAMILIES
     if _FAMILIES is None:
-        _FAMILIES = {f.name: f for f in (_mistral(), _muderax(), _surodra(), _dironex(), _murulorn())}
+        _FAMILIES = {f.name: f for f in (_mistral(), _muderax(), _surodra(), _dironex(), _murulorn(), _kagorax())}
     return _FAMILIES
 
 
@@ -206,6 +230,6 @@ def cache_blocks_for_budget(cfg, budget_bytes: int, tp_size: int = 1, elem_bytes
     """Pages of the family's cache that fit `budget_bytes`."""
     from ..engine.kv_cache import PAGE, KVCache
 
-    if getattr(cfg, "family", "mistral") in ("muderax", "surodra", "dironex", "murulorn"):
+    if getattr(cfg, "family", "mistral") in ("muderax", "surodra", "dironex", "murulorn", "kagorax"):
         return max(1, budget_bytes // max(1, cfg.cache_bytes_per_token(elem_bytes) * PAGE))
     return KVCache.blocks_for_budget(budget_bytes, cfg.num_layers, cfg.num_kv_heads // tp_size)

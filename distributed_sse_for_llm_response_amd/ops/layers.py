@@ -38,12 +38,13 @@ def scalar_norm(y, g, resid, xb, eps: float, nsum: int = 1):
         lref.scalar_norm(y, g, resid, xb, eps, nsum)
 
 
-def embed_rows(ids, embed, resid, xb):
-    """resid (fp32) = xb = embed[ids]."""
+def embed_rows(ids, embed, resid, xb=None, scale: float = 1.0, positions=None, table=None):
+    """resid (fp32) = embed[ids] * scale + table[positions] (table [P, W] fp32 given: a vector per position); xb
+    (optional, element type) receives the same rows rounded."""
     if _hip(resid):
-        torch.ops.dsse.embed_rows(ids, embed, resid, xb)
+        torch.ops.dsse.embed_rows(ids, embed, resid, xb, scale, positions, table)
     else:
-        lref.embed_rows(ids, embed, resid, xb)
+        lref.embed_rows(ids, embed, resid, xb, scale, positions, table)
 
 
 def latent_kv_write(ckr, norm_w, positions, slots, rope, cache, eps: float, vt=None):
@@ -130,16 +131,19 @@ def moe_ffn(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, out):
         lref.moe_ffn(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, out)
 
 
-def moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, sorted_ids, tile_expert, num_tiles, h, o):
+def moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, sorted_ids, tile_expert, num_tiles, h, o,
+                weight_input: bool = False):
     """Grouped form of the routed experts: rows sorted by expert, 16-row MFMA tiles of one expert each.  o [M · S, W]
     (fp32) = weight · expert output per (row, slot), S = top (+ 1: the shared expert's slot); the norm or stream step
-    that follows sums them (nsum=S).  gate None: experts without a gate, down(relu(up x)^2).  sorted_ids / tile_expert /
+    that follows sums them (nsum=S).  gate None: experts without a gate, down(relu(up x)^2).  topk_w may have a
+    column more than topk_idx: the shared expert's weight per row (1 without it).  weight_input: a routed expert's weight
+    multiplies its input instead of its output (the shared expert's always its output).  sorted_ids / tile_expert /
     num_tiles / h are scratch."""
     if _hip(x):
         torch.ops.dsse.moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, sorted_ids, tile_expert,
-                                   num_tiles, h, o)
+                                   num_tiles, h, o, weight_input)
     else:
-        lref.moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, o)
+        lref.moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, o, weight_input)
 
 
 # ---------------------------------------------------------------------------------------------------------------------
@@ -187,7 +191,8 @@ def sink_flash_ok(dtype, dim: int, vdim: int) -> bool:
 
 
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile, sink, gate, out,
-                   window: int, scale: float, qt: int, vt=None, split: bool = False, softcap: float = 0.0, out_rope=None):
+                   window: int, scale: float, qt: int, vt=None, split: bool = False, softcap: float = 0.0, out_rope=None,
+                   rel=None, keep_first: int = 0):
     """Causal softmax attention of q [T, H, D] over paged keys [pages, 32, G, D] and values [pages, 32, G, V] (grouped
     heads), scores and weights in fp32; sink [H] adds exp(sink) to each head's denominator, gate [T, H] multiplies the
     head's output by its sigmoid.  `qt` query rows per work item (work_seq, work_tile).  With vt (transposed value
@@ -196,13 +201,15 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, wor
     softcap * tanh(scale q.k / softcap).  out_rope ([positions, V / 2, 2] (cos, sin), rotate-half pairs over the whole
     value width): each head's weighted sum is turned back by the query row's own position before the gate -- with
     values that were rotated by THEIR positions when cached, a value enters the output rotated by the distance (the
-    MFMA form then needs V % 32 == 0)."""
+    MFMA form then needs V % 32 == 0).  rel [H, N] (fp32): the entry of the key's distance to the query (the last one for
+    distances from N - 1 on) is added to the score.  keep_first: the sequence's first keep_first keys stay visible when the
+    window has passed them.  A gate of H * V columns multiplies the heads element by element."""
     if _hip(q):
         torch.ops.dsse.sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile,
-                                      sink, gate, out, window, scale, qt, vt, split, softcap, out_rope)
+                                      sink, gate, out, window, scale, qt, vt, split, softcap, out_rope, rel, keep_first)
     else:
         lref.sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sink, gate, out, window, scale, vt,
-                            softcap, out_rope)
+                            softcap, out_rope, rel, keep_first)
 
 
 def gate_math(x, kind: int, p1=None, p2=None, c: float = 1.0):
@@ -331,7 +338,9 @@ def moe_route(z, correction, topk_idx, topk_w, groups: int, keep: int, scale: fl
     `groups` equal groups of neighbouring experts only the `keep` with the largest sum of their two best choice scores
     are eligible; the top experts by choice score get the weights sigmoid(z) / (their sum + 1e-20) * scale.  kind 1
     (softmax): scores softmax(z) over ALL experts (correction may be None), a group's score is its largest score, the
-    chosen experts' weights are their scores as they are, times scale."""
+    chosen experts' weights are their scores as they are, times scale.  kind 2 (sigmoid): as kind 0, but the weights are
+    the chosen scores as they are, times scale (correction may be None).  With a column more in topk_w than in topk_idx,
+    z has one more than there are experts: a shared expert's gate logit, whose sigmoid that column receives."""
     if _hip(z):
         torch.ops.dsse.moe_route(z, correction, topk_idx, topk_w, groups, keep, scale, kind)
     else:
@@ -353,16 +362,17 @@ def embed_pair_rows(ids, prev, positions, embed, pair, mul_prev: int, mul_cur: i
         lref.embed_pair_rows(ids, prev, positions, embed, pair, mul_prev, mul_cur, buckets, resid, x0, prev_out, keep)
 
 
-def add_norm_rows(y, nsum: int, g_add, resid, g_out, eps: float, out=None, out32=None):
+def add_norm_rows(y, nsum: int, g_add, resid, g_out, eps: float, out=None, out32=None, y2=None):
     """The stream's step between sublayers of a design that norms a sublayer's input AND its output, in one pass over
     the row: y given ([M * nsum, W] fp32; a row's nsum consecutive parts are summed first, the grouped experts' slots):
     resid += y / rms(y) * g_add; out given (element type or fp32; a column slice of a wider buffer is fine):
     out = resid / rms(resid) * g_out, or the stream itself when g_out is None; out32 (fp32) receives that row unrounded
-    (what a router reads).  Gains are fp32 [W]."""
+    (what a router reads).  Gains are fp32 [W].  g_add None with y given: y is added as it is (no norm), and y2 [M, W] (a
+    second sublayer that read the same norm) with it."""
     if _hip(resid):
-        torch.ops.dsse.add_norm_rows(y, nsum, g_add, resid, g_out, eps, out, out32)
+        torch.ops.dsse.add_norm_rows(y, nsum, g_add, resid, g_out, eps, out, out32, y2)
     else:
-        lref.add_norm_rows(y, nsum, g_add, resid, g_out, eps, out, out32)
+        lref.add_norm_rows(y, nsum, g_add, resid, g_out, eps, out, out32, y2)
 
 
 def token_gate_rows(x, ids, table, col0: int, out):
@@ -395,3 +405,18 @@ def token_side_rows(y, nsum: int, g_add, resid, ids, table, col0: int, gate_w, p
                                        out32)
     else:
         lref.token_side_rows(y, nsum, g_add, resid, ids, table, col0, gate_w, proj_w, side_norm, g_out, eps, out, out32)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Designs whose mixer and feed-forward read one norm side by side.
+def qkv_rows(x, bias, heads: int, kv_heads: int, dim: int, vdim: int, eps: float, slots, q, kcache=None, vcache=None,
+             vt=None):
+    """The fused projection's rows x [T, ..] (fp32, columns [q | k | v | anything]) into the attention's operands in one
+    launch: bias (fp32, optional) added; q [T, H, D] (fp32) = the query heads, each divided by its root mean square; with
+    kcache / vcache given, the key heads (normed the same way) and the value heads go to rows slots[t] of their pages
+    (negative: skipped), the values once more to the transposed pages vt when given.  Without kcache only the query
+    columns are read."""
+    if _hip(x):
+        torch.ops.dsse.qkv_rows(x, bias, heads, kv_heads, dim, vdim, eps, slots, q, kcache, vcache, vt)
+    else:
+        lref.qkv_rows(x, bias, heads, kv_heads, dim, vdim, eps, slots, q, kcache, vcache, vt)

@@ -38,13 +38,17 @@ def scalar_norm(y, g, resid, xb, eps, nsum=1):
         xb.copy_(resid.to(xb.dtype))
 
 
-def embed_rows(ids, embed, resid, xb):
+def embed_rows(ids, embed, resid, xb, scale=1.0, positions=None, table=None):
+    """resid (fp32) = embed[ids] * scale + table[positions] (table given); xb (optional) the same rows rounded."""
     M = resid.shape[0]
     idx = ids[:M].long()
     idx = torch.where((idx >= 0) & (idx < embed.shape[0]), idx, torch.zeros_like(idx))
-    rows = embed[idx]
-    resid.copy_(rows.float())
-    xb.copy_(rows)
+    rows = embed[idx].float() * scale
+    if table is not None:
+        rows = rows + table[positions[:M].long().clamp(0, table.shape[0] - 1)]
+    resid.copy_(rows)
+    if xb is not None:
+        xb.copy_(rows.to(xb.dtype))
 
 
 def _rotate(v, cs):
@@ -193,25 +197,28 @@ def moe_ffn(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, out):
     out.copy_(acc)
 
 
-def moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, o):
-    """o [M * S, W]: slot k < top of row r = weight * expert output, slot `top` = the shared expert.  gate None: the
-    experts are down(relu(up x)^2), without a gate."""
+def moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, o, weight_input=False):
+    """o [M * S, W]: slot k < top of row r = weight * expert output, slot `top` = the shared expert (times topk_w[:, top]
+    when topk_w has that column).  gate None: the experts are down(relu(up x)^2), without a gate.  weight_input: a routed
+    expert's weight multiplies its input instead of its output."""
     xf = x.float()
     M, top = topk_idx.shape
     S = top + (1 if sgate is not None else 0)
     ov = o.view(M, S, -1)
 
-    def ffn(h, g, u, d):
+    def ffn(h, g, u, d, c=1.0):
         if g is None:
-            return torch.relu(h @ u.float().t()).pow(2).to(x.dtype).float() @ d.float().t()
-        return (torch.nn.functional.silu(h @ g.float().t()) * (h @ u.float().t())) @ d.float().t()
+            return torch.relu(c * (h @ u.float().t())).pow(2).to(x.dtype).float() @ d.float().t()
+        return (torch.nn.functional.silu(c * (h @ g.float().t())) * (c * (h @ u.float().t()))) @ d.float().t()
 
     for e in range(up.shape[0]):
         rows, ks = torch.nonzero(topk_idx == e, as_tuple=True)
         if rows.numel():
-            ov[rows, ks] = ffn(xf[rows], None if gate is None else gate[e], up[e], down[e]) * topk_w[rows, ks].unsqueeze(-1)
+            w = topk_w[rows, ks].unsqueeze(-1)
+            g = None if gate is None else gate[e]
+            ov[rows, ks] = ffn(xf[rows], g, up[e], down[e], w) if weight_input else ffn(xf[rows], g, up[e], down[e]) * w
     if sgate is not None:
-        ov[:, top] = ffn(xf, sgate, sup, sdown)
+        ov[:, top] = ffn(xf, sgate, sup, sdown) * (topk_w[:, top:] if topk_w.shape[1] > top else 1.0)
 
 
 # ---------------------------------------------------------------------------------------------------------------------
@@ -284,12 +291,14 @@ def norm_rope_rows(x, norm_w, positions, rope, out, out_rows, norm_kind, eps, sc
 
 
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sink, gate, out, window, scale, vt=None,
-                   softcap=0.0, out_rope=None):
+                   softcap=0.0, out_rope=None, rel=None, keep_first=0):
     """Softmax attention over paged keys [pages, PAGE, G, D] and values [pages, PAGE, G, V] with grouped heads; the
     denominator also holds exp(sink[h]) when sink is given; the head's output is multiplied by sigmoid(gate[row, h])
     when gate is given.  With vt the values come from the transposed pages [pages, G, V, PAGE].  softcap > 0: scores
     softcap * tanh(. / softcap).  out_rope [positions, V / 2, 2]: the head's output is turned BACK by the query's
-    position (rotate-half pairs), undoing the rotation of a value rotated by that same position."""
+    position (rotate-half pairs), undoing the rotation of a value rotated by that same position.  rel [H, N]: the entry of
+    the key's distance (the last one for distances from N - 1 on) is added to the score.  keep_first: that many first keys
+    of the sequence stay visible outside the window.  A gate of H * V columns is applied element by element."""
     H = q.shape[1]
     G = kcache.shape[2]
     kf = kcache.view(-1, G, kcache.shape[3]).float()
@@ -303,7 +312,8 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sin
         bt = block_tables[s].long()
         for i in range(ql):
             pos = p0 + i
-            j = torch.arange(max(0, pos - window + 1), pos + 1)
+            lo = max(0, pos - window + 1)
+            j = torch.cat([torch.arange(min(lo, keep_first)), torch.arange(lo, pos + 1)])
             rows = bt[j // PAGE] * PAGE + j % PAGE
             k, v = kf[rows][:, grp], vf[rows][:, grp]                       # [keys, H, D], [keys, H, V]
             if vt is not None:  # the same numbers from the transposed pages, so a wrong place shows
@@ -311,6 +321,8 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sin
             sc = torch.einsum("hd,jhd->hj", q[r0 + i].float(), k) * scale
             if softcap > 0:
                 sc = softcap * torch.tanh(sc / softcap)
+            if rel is not None:
+                sc = sc + rel.float()[:, (pos - j).clamp(max=rel.shape[1] - 1)]
             mx = sc.max(-1, keepdim=True).values
             if sink is not None:
                 mx = torch.maximum(mx, sink.float()[:, None])
@@ -324,7 +336,7 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sin
                 cs[:, 1] = -cs[:, 1]
                 o = rotate_half_rows(o[None], cs[None], 2 * out_rope.shape[1])[0]
             if gate is not None:
-                o = o * torch.sigmoid(gate[r0 + i].float())[:, None]
+                o = o * torch.sigmoid(gate[r0 + i].float()).view(H, -1)
             out[r0 + i] = o.to(out.dtype)
 
 
@@ -432,9 +444,14 @@ def moe_route(z, correction, topk_idx, topk_w, groups, keep, scale, kind=0):
     """kind 1: scores softmax(z) over all experts, a group's score is its largest score, the weights are the chosen
     scores as they are (times scale).  kind 0: router logits z [M, E] fp32 -> the `top` experts with the largest sigmoid(z) + correction among the experts of
     the `keep` best of `groups` equal groups of neighbours (a group's score: the sum of its two largest such values);
-    weights: the chosen sigmoid(z) over their sum (+ 1e-20), times scale.  Ties go to the lower index."""
-    M, E = z.shape
+    weights: the chosen sigmoid(z) over their sum (+ 1e-20), times scale.  Ties go to the lower index.  kind 2: sigmoid
+    scores, groups as for kind 0, the weights are the chosen scores as they are (times scale).  topk_w may have a column
+    more than topk_idx and z then one more than there are experts: the shared expert's gate logit, whose sigmoid it gets."""
     top = topk_idx.shape[1]
+    if topk_w.shape[1] > top:
+        topk_w[:, top] = torch.sigmoid(torch.nan_to_num(z[:, -1].float(), nan=0.0))
+        z, topk_w = z[:, :-1], topk_w[:, :top]
+    M, E = z.shape
     zz = torch.nan_to_num(z.float(), nan=0.0)
     s = torch.softmax(zz, dim=-1) if kind == 1 else torch.sigmoid(zz)
     choice = s + correction.float() if correction is not None else s.clone()
@@ -447,7 +464,7 @@ def moe_route(z, correction, topk_idx, topk_w, groups, keep, scale, kind=0):
     idx = torch.argsort(choice, dim=-1, descending=True, stable=True)[:, :top]
     w = s.gather(1, idx)
     topk_idx.copy_(idx.to(torch.int32))
-    topk_w.copy_(w * scale if kind == 1 else w / (w.sum(-1, keepdim=True) + 1e-20) * scale)
+    topk_w.copy_(w * scale if kind >= 1 else w / (w.sum(-1, keepdim=True) + 1e-20) * scale)
 
 
 # ---------------------------------------------------------------------------------------------------------------------
@@ -475,12 +492,15 @@ def embed_pair_rows(ids, prev, positions, embed, pair, mul_prev, mul_cur, bucket
         x0.copy_(rows.to(x0.dtype))
 
 
-def add_norm_rows(y, nsum, g_add, resid, g_out, eps, out, out32):
+def add_norm_rows(y, nsum, g_add, resid, g_out, eps, out, out32, y2=None):
     """The residual stream's step of a design with a norm before AND after each sublayer.  y given ([M * nsum, W] fp32,
     a row's nsum consecutive parts are summed first): resid += y / rms(y) * g_add.  out given (element type or fp32, may
     be a column slice): out = resid / rms(resid) * g_out, or resid itself without g_out; out32 (optional, fp32) receives
-    the same row unrounded."""
-    if y is not None:
+    the same row unrounded.  g_add None: y is added as it is, and so is y2 (a second sublayer's output) when given."""
+    if y is not None and g_add is None:
+        v = y.float().view(resid.shape[0], nsum, -1).sum(1)
+        resid.add_(v if y2 is None else v + y2.float())
+    elif y is not None:
         v = y.float().view(resid.shape[0], nsum, -1).sum(1)
         resid.add_(v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps) * g_add.float())
     if out is not None or out32 is not None:
@@ -511,3 +531,24 @@ def token_side_rows(y, nsum, g_add, resid, ids, table, col0, gate_w, proj_w, sid
     sh = torch.empty(resid.shape[0], F, dtype=gate_w.dtype)
     token_gate_rows(sg, ids, table, col0, sh)
     add_norm_rows(sh.float() @ proj_w.float().t(), 1, side_norm, resid, g_out, eps, out, out32)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Designs whose mixer and feed-forward read one norm side by side (models/kagorax.py)
+def qkv_rows(x, bias, H, G, D, V, eps, slots, q, kcache, vcache, vt):
+    """x [T, >= H D (+ G D + G V)] fp32, columns [q | k | v]; bias (optional, fp32) is added first.  q [T, H, D] = the
+    query heads, each divided by its root mean square; with kcache, rows slots[t] of the pages receive the key heads
+    (normed the same way) and the value heads as they are, the latter also in transposed pages vt when given."""
+    n = H * D + (G * (D + V) if kcache is not None else 0)
+    y = x[:, :n].float()
+    if bias is not None:
+        y = y + bias.float()[:n]
+    T = y.shape[0]
+
+    def rms_heads(v):
+        return v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+
+    q.copy_(rms_heads(y[:, :H * D].reshape(T, H, D)).to(q.dtype))
+    if kcache is not None:
+        norm_rope_rows(rms_heads(y[:, H * D:(H + G) * D].reshape(T, G, D)), None, None, None, kcache, slots, 0, 0.0, 1.0)
+        norm_rope_rows(y[:, (H + G) * D:].reshape(T, G, V), None, None, None, vcache, slots, 0, 0.0, 1.0, vt)

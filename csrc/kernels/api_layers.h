@@ -141,7 +141,9 @@ struct MoeFfnParams {
 struct MoeGroupedParams {
   const void* x;         // [M, W]
   const int* topk_idx;   // [M, top]
-  const float* topk_w;   // [M, top]
+  const float* topk_w;   // [M, ldw]
+  int ldw;               // top, or top + 1: the last column is the shared expert's weight (1 otherwise)
+  int weight_in;         // 1: a routed expert's weight multiplies its input (gate and up outputs), not its output
   const void* gate;      // [E, F, W], or null: experts without a gate, h = relu(up x)^2
   const void* up;
   const void* down;      // [E, W, F]
@@ -164,8 +166,9 @@ struct MoeGroupedParams {
 extern "C" {
 hipError_t dsse_gemm_rm(const dsse::GemmRmParams* p, hipStream_t st);
 hipError_t dsse_scalar_norm(const dsse::ScalarNormParams* p, hipStream_t st);
-hipError_t dsse_embed_rows(int M, int W, int vocab, const int* ids, const void* embed, float* resid, void* xb, int f32,
-                           hipStream_t st);
+// resid = embed[ids] * scale + table[positions] (table fp32 [table_len, W] or null); xb (or null) the same rounded
+hipError_t dsse_embed_rows(int M, int W, int vocab, const int* ids, const void* embed, float* resid, void* xb, float scale,
+                           const int* positions, const float* table, int table_len, int f32, hipStream_t st);
 hipError_t dsse_latent_kv_write(const dsse::LatentKvWriteParams* p, void* vt, hipStream_t st);  // vt: see below, or null
 hipError_t dsse_latent_attention(int num_work, const dsse::LatentAttnParams* p, hipStream_t st);
 // transposed latent pages vt [pages, rk, kBS] (keys permuted inside a page) for the MFMA form, and that form itself

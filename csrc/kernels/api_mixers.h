@@ -63,6 +63,24 @@ struct SinkAttnParams {
   float softcap;         // > 0: score = softcap * tanh(scale q.k / softcap)
   const float2* out_rope;  // [out_rope_len, V / 2] (cos, sin) or null: each head's sum is turned back by the row's own
   int out_rope_len;        // position, rotate-half pairs (m, m + V / 2), before the gate
+  const float* rel;      // [H, rel_len] or null: the entry of the key's distance (the last one beyond) joins the score
+  int rel_len;
+  int keep_first;        // the sequence's first keys that stay visible outside the window
+  int gate_wide;         // 1: the gate has H * V columns, one per element of the output
+};
+
+// The fused projection's q | k | v columns into the attention's operands.
+struct QkvRowsParams {
+  const float* x;        // rows ldx apart: [q (H D) | k (G D) | v (G V) | ..] (only q when k is null)
+  const float* bias;     // same columns, or null
+  const int* slots;      // [T] cache row, negative = skip
+  float* q;              // [T, H, D]
+  void* k;               // [pages * kBS, G, D] element type, or null: the row has no keys and values
+  void* v;               // [pages * kBS, G, V]
+  void* vt;              // transposed value pages [pages, G, V, kBS], or null
+  int T, H, G, D, V, ldx, num_slots;
+  float eps;
+  int f32;
 };
 
 struct MatrixScanParams {
@@ -151,7 +169,8 @@ struct EmbedPairParams {
 struct AddNormParams {
   const float* y;        // [M * nsum, W] or null: resid += rms-norm(sum of the row's parts) * g_add
   int nsum;
-  const float* g_add;    // [W]
+  const float* g_add;    // [W] or null: the parts' sum is added as it is
+  const float* y2;       // [M, W] or null: added too (with g_add null)
   float* resid;          // [M, W] fp32
   const float* g_out;    // [W] or null: out = resid itself
   void* out;             // rows ldo apart (fp32 when out_f32, else bf16) or null
@@ -184,6 +203,7 @@ struct TokenSideParams {
 }  // namespace dsse
 
 extern "C" {
+hipError_t dsse_qkv_rows(const dsse::QkvRowsParams* p, hipStream_t st);
 hipError_t dsse_token_side_rows(const dsse::TokenSideParams* p, hipStream_t st);
 hipError_t dsse_embed_pair_rows(const dsse::EmbedPairParams* p, hipStream_t st);
 hipError_t dsse_add_norm_rows(const dsse::AddNormParams* p, hipStream_t st);
@@ -195,9 +215,11 @@ hipError_t dsse_stream_mix(const dsse::StreamMixParams* p, hipStream_t st);
 hipError_t dsse_act_rows(const float* x, int ldx, void* out, int M, int F, int kind, const float* params,
                          const float* gate, int ldg, int f32, hipStream_t st);
 // group-limited routing from fp32 logits [M, E] (E <= 256); kind 0: sigmoid scores + correction, groups by the sum of
-// their two best, weights renormalised; kind 1: softmax scores (corr may be null), groups by their best, weights as is
-hipError_t dsse_moe_route(const float* z, const float* corr, int M, int E, int top, int groups, int keep, float scale,
-                          int kind, int* topk_idx, float* topk_w, hipStream_t st);
+// their two best, weights renormalised; kind 1: softmax scores (corr may be null), groups by their best, weights as is;
+// kind 2: kind 0's choice (corr may be null), weights as is.  Rows of z are ldz apart and rows of topk_w ldw; ldw > top:
+// column E of z is a shared expert's gate logit and column top of topk_w receives its sigmoid
+hipError_t dsse_moe_route(const float* z, int ldz, const float* corr, int M, int E, int top, int groups, int keep,
+                          float scale, int kind, int* topk_idx, float* topk_w, int ldw, hipStream_t st);
 hipError_t dsse_stream_step(const dsse::StreamStepParams* p, hipStream_t st);
 hipError_t dsse_gated_act(const float* gu, int ldg, void* h, int M, int F, int kind, int f32, hipStream_t st);
 hipError_t dsse_norm_rope_rows(const dsse::NormRopeParams* p, hipStream_t st);

@@ -118,16 +118,37 @@ void scalar_norm(const OptTensor& y, const Tensor& g, Tensor& resid, Tensor& xb,
   DSSE_CHECK_HIP(dsse_scalar_norm(&p, cur_stream()));
 }
 
-void embed_rows(const Tensor& ids, const Tensor& embed, Tensor& resid, Tensor& xb) {
+void embed_rows(const Tensor& ids, const Tensor& embed, Tensor& resid, const OptTensor& xb, double scale,
+                const OptTensor& positions, const OptTensor& table) {
   i32(ids, "ids");
   gpu(embed, "embed");
   f32t(resid, "resid");
-  gpu(xb, "xb");
-  same(embed, xb, "xb");
   const int M = (int)resid.size(0), W = (int)resid.size(1);
-  TORCH_CHECK(embed.dim() == 2 && embed.size(1) == W && ids.numel() >= M && xb.sizes() == resid.sizes(), "embed shapes");
+  TORCH_CHECK(embed.dim() == 2 && embed.size(1) == W && ids.numel() >= M, "embed shapes");
+  void* xbp = nullptr;
+  if (xb.has_value()) {
+    gpu(*xb, "xb");
+    same(embed, *xb, "xb");
+    TORCH_CHECK(xb->sizes() == resid.sizes(), "xb must match resid");
+    xbp = xb->data_ptr();
+  }
+  const int* pos = nullptr;
+  const float* tab = nullptr;
+  int len = 0;
+  if (table.has_value()) {
+    f32t(*table, "table");
+    TORCH_CHECK(positions.has_value() && table->dim() == 2 && table->size(1) == W && table->size(0) >= 1 &&
+                    table->size(0) < INT_MAX,
+                "table must be [positions, W]");
+    i32(*positions, "positions");
+    TORCH_CHECK(positions->numel() >= M, "positions too short");
+    pos = positions->data_ptr<int>();
+    tab = table->data_ptr<float>();
+    len = (int)table->size(0);
+  }
   DSSE_CHECK_HIP(dsse_embed_rows(M, W, (int)embed.size(0), ids.data_ptr<int>(), embed.data_ptr(),
-                                 resid.data_ptr<float>(), xb.data_ptr(), elem(xb, "xb"), cur_stream()));
+                                 resid.data_ptr<float>(), xbp, (float)scale, pos, tab, len, elem(embed, "embed"),
+                                 cur_stream()));
 }
 
 void latent_kv_write(const Tensor& ckr, const Tensor& norm_w, const Tensor& positions, const Tensor& slots,
@@ -431,7 +452,7 @@ void moe_ffn(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, cons
 // tile_expert [tiles], num_tiles [1] (int32), h [M * S, ldh] (element type), tiles >= ceil(M S / 64) + experts + 1.
 void moe_grouped(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, const OptTensor& gate, const Tensor& up,
                  const Tensor& down, const OptTensor& sgate, const OptTensor& sup, const OptTensor& sdown, Tensor& sorted,
-                 Tensor& tile_expert, Tensor& num_tiles, Tensor& h, Tensor& o) {
+                 Tensor& tile_expert, Tensor& num_tiles, Tensor& h, Tensor& o, bool weight_input) {
   gpu(x, "x");
   i32(topk_idx, "topk_idx");
   f32t(topk_w, "topk_w");
@@ -457,7 +478,11 @@ void moe_grouped(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, 
   }
   p.E = (int)up.size(0), p.F = (int)up.size(1), p.top = (int)topk_idx.size(1);
   TORCH_CHECK(down.dim() == 3 && down.size(0) == p.E && down.size(1) == p.W && down.size(2) == p.F, "down must be [E, W, F]");
-  TORCH_CHECK(topk_idx.dim() == 2 && topk_idx.size(0) == p.M && topk_w.sizes() == topk_idx.sizes(), "routing shapes");
+  TORCH_CHECK(topk_idx.dim() == 2 && topk_idx.size(0) == p.M && topk_w.dim() == 2 && topk_w.size(0) == p.M &&
+                  (topk_w.size(1) == p.top || (sgate.has_value() && topk_w.size(1) == p.top + 1)),
+              "routing shapes");
+  p.ldw = (int)topk_w.size(1);
+  p.weight_in = weight_input ? 1 : 0;
   p.S = p.top;
   if (sgate.has_value()) {
     TORCH_CHECK(sup.has_value() && sdown.has_value(), "the shared expert needs gate, up and down");
@@ -522,8 +547,9 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
   m.def("scalar_norm(Tensor? y, Tensor g, Tensor(a!) resid, Tensor(b!) xb, float eps, int nsum=1) -> ()");
   m.def("moe_grouped(Tensor x, Tensor topk_idx, Tensor topk_w, Tensor? gate, Tensor up, Tensor down, Tensor? sgate, "
         "Tensor? sup, Tensor? sdown, Tensor(a!) sorted, Tensor(b!) tile_expert, Tensor(c!) num_tiles, Tensor(d!) h, "
-        "Tensor(e!) o) -> ()");
-  m.def("embed_rows(Tensor ids, Tensor embed, Tensor(a!) resid, Tensor(b!) xb) -> ()");
+        "Tensor(e!) o, bool weight_input=False) -> ()");
+  m.def("embed_rows(Tensor ids, Tensor embed, Tensor(a!) resid, Tensor(b!)? xb, float scale=1.0, Tensor? positions=None, "
+        "Tensor? table=None) -> ()");
   m.def("latent_kv_write(Tensor ckr, Tensor norm_w, Tensor positions, Tensor slots, Tensor rope, Tensor(a!) cache, "
         "float eps, Tensor(b!)? vt=None) -> ()");
   m.def("latent_attention(Tensor q, Tensor q_abs, Tensor cache, Tensor block_tables, Tensor q_start, Tensor q_len, "

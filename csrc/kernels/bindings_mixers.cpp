@@ -176,7 +176,8 @@ void norm_rope_rows(const Tensor& x, const OptTensor& norm_w, const Tensor& posi
 void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache, const Tensor& block_tables,
                     const Tensor& q_start, const Tensor& q_len, const Tensor& ctx_len, const Tensor& work_seq,
                     const Tensor& work_tile, const OptTensor& sink, const OptTensor& gate, Tensor& out, int64_t window,
-                    double scale, int64_t qt, const OptTensor& vt, bool split, double softcap, const OptTensor& out_rope) {
+                    double scale, int64_t qt, const OptTensor& vt, bool split, double softcap, const OptTensor& out_rope,
+                    const OptTensor& rel, int64_t keep_first) {
   f32t(q, "q");
   gpu(kcache, "kcache");
   gpu(vcache, "vcache");
@@ -214,7 +215,9 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
   p.sink = opt_f32(sink, "sink", p.H);
   if (gate.has_value()) {
     col_view(*gate, "gate");
-    TORCH_CHECK(gate->size(0) == T && gate->size(1) == p.H, "gate must be [T, H]");
+    TORCH_CHECK(gate->size(0) == T && (gate->size(1) == p.H || gate->size(1) == (int64_t)p.H * p.V),
+                "gate must be [T, H] or [T, H * V]");
+    p.gate_wide = p.V > 1 && gate->size(1) == (int64_t)p.H * p.V ? 1 : 0;
     p.gate = gate->data_ptr<float>();
     p.ldg = (int)gate->stride(0);
   }
@@ -224,6 +227,14 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
   p.f32 = elem(kcache, "kcache");
   TORCH_CHECK(softcap >= 0, "softcap >= 0");
   p.softcap = (float)softcap;
+  TORCH_CHECK(keep_first >= 0, "keep_first >= 0");
+  p.keep_first = (int)std::min<int64_t>(keep_first, INT_MAX);
+  if (rel.has_value()) {
+    f32t(*rel, "rel");
+    TORCH_CHECK(rel->dim() == 2 && rel->size(0) == p.H && rel->size(1) >= 1 && rel->size(1) < INT_MAX, "rel must be [H, N]");
+    p.rel = rel->data_ptr<float>();
+    p.rel_len = (int)rel->size(1);
+  }
   if (out_rope.has_value()) {
     f32t(*out_rope, "out_rope");
     TORCH_CHECK(out_rope->dim() == 3 && out_rope->size(2) == 2 && 2 * out_rope->size(1) == p.V && out_rope->size(0) >= 1,
@@ -523,19 +534,23 @@ void act_rows(const Tensor& x, Tensor& out, int64_t kind, const OptTensor& param
 void moe_route(const Tensor& z, const OptTensor& correction, Tensor& topk_idx, Tensor& topk_w, int64_t groups,
                int64_t keep, double scale, int64_t kind) {
   f32t(z, "z");
-  TORCH_CHECK(kind == 0 || kind == 1, "kind: 0 sigmoid scores, 1 softmax scores");
-  TORCH_CHECK(kind == 1 || correction.has_value(), "sigmoid routing needs its correction");
+  TORCH_CHECK(kind >= 0 && kind <= 2, "kind: 0 sigmoid scores, 1 softmax scores, 2 sigmoid scores as they are");
+  TORCH_CHECK(kind >= 1 || correction.has_value(), "sigmoid routing needs its correction");
   i32(topk_idx, "topk_idx");
   f32t(topk_w, "topk_w");
   TORCH_CHECK(z.dim() == 2 && topk_idx.dim() == 2, "z must be [M, E], topk_idx [M, top]");
-  const int M = (int)z.size(0), E = (int)z.size(1), top = (int)topk_idx.size(1);
-  TORCH_CHECK(topk_idx.size(0) == M && topk_w.sizes() == topk_idx.sizes(), "routing shapes");
+  // one more column in topk_w than in topk_idx: z's last column is a shared expert's gate logit
+  const int M = (int)z.size(0), top = (int)topk_idx.size(1);
+  const int shared = topk_w.dim() == 2 && topk_w.size(1) == top + 1 ? 1 : 0, E = (int)z.size(1) - shared;
+  TORCH_CHECK(topk_idx.size(0) == M && topk_w.dim() == 2 && topk_w.size(0) == M && topk_w.size(1) == top + shared,
+              "routing shapes");
   const float* corr = opt_f32(correction, "correction", E);
   TORCH_CHECK(E >= 1 && E <= 256 && groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top >= 1 &&
                   top <= keep * (E / groups),
               "routing: E <= 256, equal groups, 1 <= keep <= groups, top <= experts of the kept groups");
-  DSSE_CHECK_HIP(dsse_moe_route(z.data_ptr<float>(), corr, M, E, top, (int)groups, (int)keep, (float)scale, (int)kind,
-                                topk_idx.data_ptr<int>(), topk_w.data_ptr<float>(), cur_stream()));
+  DSSE_CHECK_HIP(dsse_moe_route(z.data_ptr<float>(), E + shared, corr, M, E, top, (int)groups, (int)keep, (float)scale,
+                                (int)kind, topk_idx.data_ptr<int>(), topk_w.data_ptr<float>(), top + shared,
+                                cur_stream()));
 }
 
 void embed_pair_rows(const Tensor& ids, const OptTensor& prev, const Tensor& positions, const Tensor& embed,
@@ -589,7 +604,7 @@ void embed_pair_rows(const Tensor& ids, const OptTensor& prev, const Tensor& pos
 }
 
 void add_norm_rows(const OptTensor& y, int64_t nsum, const OptTensor& g_add, Tensor& resid, const OptTensor& g_out,
-                   double eps, const OptTensor& out, const OptTensor& out32) {
+                   double eps, const OptTensor& out, const OptTensor& out32, const OptTensor& y2) {
   f32t(resid, "resid");
   TORCH_CHECK(resid.dim() == 2 && nsum >= 1, "resid [M, W], nsum >= 1");
   dsse::AddNormParams p{};
@@ -599,9 +614,12 @@ void add_norm_rows(const OptTensor& y, int64_t nsum, const OptTensor& g_add, Ten
   if (y.has_value()) {
     f32t(*y, "y");
     TORCH_CHECK(y->numel() == (int64_t)p.M * nsum * p.W, "y must hold M * nsum rows of W");
-    TORCH_CHECK(g_add.has_value(), "y needs its norm's gain");
     p.y = y->data_ptr<float>();
     p.g_add = opt_f32(g_add, "g_add", p.W);
+  }
+  if (y2.has_value()) {
+    TORCH_CHECK(p.y && !p.g_add, "y2 is added beside a y that has no norm");
+    p.y2 = opt_f32(y2, "y2", (int64_t)p.M * p.W);
   }
   p.g_out = opt_f32(g_out, "g_out", p.W);
   if (out.has_value()) {
@@ -688,7 +706,57 @@ void token_side_rows(const OptTensor& y, int64_t nsum, const OptTensor& g_add, T
   DSSE_CHECK_HIP(dsse_token_side_rows(&p, cur_stream()));
 }
 
+void qkv_rows(const Tensor& x, const OptTensor& bias, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, double eps,
+              const Tensor& slots, Tensor& q, const OptTensor& kcache, const OptTensor& vcache, const OptTensor& vt) {
+  col_view(x, "x");
+  f32t(q, "q");
+  dsse::QkvRowsParams p{};
+  p.T = (int)x.size(0), p.H = (int)heads, p.G = (int)kv_heads, p.D = (int)dim, p.V = (int)vdim;
+  TORCH_CHECK(heads >= 1 && kv_heads >= 1 && dim >= 1 && vdim >= 1 && dim <= 512 && vdim <= 512, "head counts and widths");
+  TORCH_CHECK(q.dim() == 3 && q.size(0) == p.T && q.size(1) == p.H && q.size(2) == p.D, "q must be [T, H, D]");
+  const bool own = kcache.has_value();
+  TORCH_CHECK(own == vcache.has_value() && (own || !vt.has_value()), "keys and values come together");
+  const int64_t n = heads * dim + (own ? kv_heads * (dim + vdim) : 0);
+  TORCH_CHECK(x.size(1) >= n, "x must hold the q | k | v columns");
+  p.x = x.data_ptr<float>();
+  p.ldx = (int)x.stride(0);
+  if (bias.has_value()) {
+    f32t(*bias, "bias");
+    TORCH_CHECK(bias->numel() >= n, "bias must cover the q | k | v columns");
+    p.bias = bias->data_ptr<float>();
+  }
+  p.q = q.data_ptr<float>();
+  p.eps = (float)eps;
+  if (own) {
+    i32(slots, "slots");
+    gpu(*kcache, "kcache");
+    gpu(*vcache, "vcache");
+    TORCH_CHECK(kcache->dim() == 4 && vcache->dim() == 4 && kcache->scalar_type() == vcache->scalar_type() &&
+                    kcache->size(1) == dsse::kBS && vcache->size(1) == dsse::kBS && kcache->size(2) == p.G &&
+                    vcache->size(2) == p.G && kcache->size(3) == p.D && vcache->size(3) == p.V &&
+                    kcache->size(0) == vcache->size(0) && kcache->size(0) * dsse::kBS < INT_MAX,
+                "caches must be [pages, 32, G, D] and [pages, 32, G, V]");
+    TORCH_CHECK(slots.numel() >= p.T, "slots too short");
+    p.slots = slots.data_ptr<int>();
+    p.k = kcache->data_ptr();
+    p.v = vcache->data_ptr();
+    p.num_slots = (int)(kcache->size(0) * dsse::kBS);
+    p.f32 = elem(*kcache, "kcache");
+    if (vt.has_value()) {
+      gpu(*vt, "vt");
+      TORCH_CHECK(vt->scalar_type() == vcache->scalar_type() && vt->dim() == 4 && vt->size(0) == vcache->size(0) &&
+                      vt->size(1) == p.G && vt->size(2) == p.V && vt->size(3) == dsse::kBS,
+                  "vt must be [pages, G, V, 32]");
+      p.vt = vt->data_ptr();
+    }
+  }
+  TORCH_CHECK((heads + 2 * kv_heads + 3) / 4 <= 65535, "too many heads");
+  DSSE_CHECK_HIP(dsse_qkv_rows(&p, cur_stream()));
+}
+
 TORCH_LIBRARY_FRAGMENT(dsse, m) {
+  m.def("qkv_rows(Tensor x, Tensor? bias, int heads, int kv_heads, int dim, int vdim, float eps, Tensor slots, "
+        "Tensor(a!) q, Tensor(b!)? kcache=None, Tensor(c!)? vcache=None, Tensor(d!)? vt=None) -> ()");
   m.def("token_side_rows(Tensor? y, int nsum, Tensor? g_add, Tensor(a!) resid, Tensor ids, Tensor table, int col0, "
         "Tensor gate_w, Tensor proj_w, Tensor side_norm, Tensor? g_out, float eps, Tensor(b!)? out, Tensor(c!)? out32) -> ()");
   m.def("stream_mix(Tensor? y, int nsum, float mult, Tensor(a!) streams, Tensor? ids, Tensor? embed, float embed_scale, "
@@ -699,7 +767,7 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
   m.def("embed_pair_rows(Tensor ids, Tensor? prev, Tensor positions, Tensor embed, Tensor? pair, int mul_prev, "
         "int mul_cur, int buckets, Tensor(a!) resid, Tensor(b!)? x0, Tensor(c!)? prev_out, Tensor? keep) -> ()");
   m.def("add_norm_rows(Tensor? y, int nsum, Tensor? g_add, Tensor(a!) resid, Tensor? g_out, float eps, "
-        "Tensor(b!)? out, Tensor(c!)? out32) -> ()");
+        "Tensor(b!)? out, Tensor(c!)? out32, Tensor? y2=None) -> ()");
   m.def("token_gate_rows(Tensor x, Tensor ids, Tensor table, int col0, Tensor(a!) out) -> ()");
   m.def("stream_step(Tensor? y, float mult, Tensor(a!) resid, Tensor? ids, Tensor? embed, Tensor? vec, Tensor? alpha, "
         "Tensor? w, Tensor? b, Tensor(b!)? xb) -> ()");
@@ -708,7 +776,8 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
         "int kind, float eps, float scale=1.0, Tensor(b!)? out_t=None) -> ()");
   m.def("sink_attention(Tensor q, Tensor kcache, Tensor vcache, Tensor block_tables, Tensor q_start, Tensor q_len, "
         "Tensor ctx_len, Tensor work_seq, Tensor work_tile, Tensor? sink, Tensor? gate, Tensor(a!) out, int window, "
-        "float scale, int qt, Tensor? vt=None, bool split=False, float softcap=0.0, Tensor? out_rope=None) -> ()");
+        "float scale, int qt, Tensor? vt=None, bool split=False, float softcap=0.0, Tensor? out_rope=None, "
+        "Tensor? rel=None, int keep_first=0) -> ()");
   m.def("gate_math(Tensor(a!) x, int kind, Tensor? p1=None, Tensor? p2=None, float c=1.0) -> ()");
   m.def("matrix_scan(Tensor q, Tensor k, Tensor v, Tensor? decay, Tensor? beta, Tensor(a!) state, Tensor q_start, "
         "Tensor q_len, Tensor ctx_len, Tensor state_slot, Tensor(b!) out, float q_scale=1.0) -> ()");
@@ -721,6 +790,7 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
 }
 
 TORCH_LIBRARY_IMPL(dsse, CUDA, m) {
+  m.impl("qkv_rows", &qkv_rows);
   m.impl("stream_mix", &stream_mix);
   m.impl("act_rows", &act_rows);
   m.impl("moe_route", &moe_route);

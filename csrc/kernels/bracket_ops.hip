@@ -4,7 +4,8 @@
 //   embed_pair_rows  resid = embed[id] + pair[(prev * a + id * b) mod n]  (row n at position 0); the same row once more
 //                    in the element type where the projection that opens a loop pass reads it; decode slots store their
 //                    token as the next token's predecessor
-//   add_norm_rows    resid += y / rms(y) * g_add  (y summed over the experts' slots first), then
+//   add_norm_rows    resid += y / rms(y) * g_add  (y summed over the experts' slots first; without g_add: resid += y + y2,
+//                    the outputs of two sublayers that read the same norm, as they are), then
 //                    out = resid / rms(resid) * g_out (or resid itself): the add of one sublayer and the norm of the next
 //                    in one pass over the row, the row held in registers between its two statistics
 //   token_gate_rows  out = gelu_tanh(x) * table[id, col0 : col0 + F]
@@ -118,7 +119,25 @@ __global__ __launch_bounds__(256) void add_norm_rows_kernel(AddNormParams p) {
     return v;
   };
   float ss = 0.f;
-  if (y) {
+  if (y && !p.g_add) {  // sublayers whose outputs are added as they are
+    const float* y2 = p.y2 ? p.y2 + row * W : nullptr;
+    each([&](int i, int d) {
+      FVec<VEC> v = parts(d);
+      if (y2) {
+        const FVec<VEC> t = ld_f<VEC>(y2 + d);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) v.v[e] += t.v[e];
+      }
+      FVec<VEC> r = ld_f<VEC>(resid + d);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        r.v[e] += v.v[e];
+        ss += r.v[e] * r.v[e];
+      }
+      st_f<VEC>(resid + d, r);
+      if (REG) vals[i] = r;
+    });
+  } else if (y) {
     float sy = 0.f;
     each([&](int i, int d) {
       const FVec<VEC> v = parts(d);
@@ -327,7 +346,7 @@ template <typename OutT>
 void launch_add_norm(const AddNormParams& p, hipStream_t st) {
   const dim3 g(p.M), b(256);
   auto al = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
-  const bool vec = p.W % 4 == 0 && p.ldo % 4 == 0 && al(p.y) && al(p.resid) && al(p.g_add) && al(p.g_out) && al(p.out) &&
+  const bool vec = p.W % 4 == 0 && p.ldo % 4 == 0 && al(p.y) && al(p.y2) && al(p.resid) && al(p.g_add) && al(p.g_out) && al(p.out) &&
                    al(p.out32);
   if (vec && p.W <= 256 * kNormRegs * 4) hipLaunchKernelGGL((add_norm_rows_kernel<OutT, 4, true>), g, b, 0, st, p);
   else if (p.W <= 256 * kNormRegs) hipLaunchKernelGGL((add_norm_rows_kernel<OutT, 1, true>), g, b, 0, st, p);
@@ -347,7 +366,7 @@ extern "C" hipError_t dsse_embed_pair_rows(const dsse::EmbedPairParams* p, hipSt
 
 extern "C" hipError_t dsse_add_norm_rows(const dsse::AddNormParams* p, hipStream_t st) {
   if (p->M <= 0) return hipSuccess;
-  if (p->nsum < 1 || (p->y && !p->g_add)) return hipErrorInvalidValue;
+  if (p->nsum < 1 || (p->y2 && (!p->y || p->g_add))) return hipErrorInvalidValue;
   if (p->out_f32) dsse::launch_add_norm<float>(*p, st);
   else dsse::launch_add_norm<bf16>(*p, st);
   return hipGetLastError();

@@ -152,6 +152,22 @@ __global__ __launch_bounds__(256) void moe_ffn_kernel(MoeFfnParams p) {
 //   moe_down      o[id, :] = weight(id) * down_e . h[id]                          (fp32)
 // The residual norm that follows sums a row's S slots (scalar_norm nsum).
 
+// Weights: by default a routed expert's weight multiplies its output (moe_down).  weight_in moves it to the expert's
+// input; the gate and up products are linear in it, so it multiplies their fp32 sums (moe_gate_up).  The shared expert's
+// weight, when topk_w has a column for it, always multiplies its output.
+
+DEV float slot_weight(const MoeGroupedParams& p, int row, int k) {
+  return k < p.ldw ? p.topk_w[(int64_t)row * p.ldw + k] : 1.0f;
+}
+DEV float out_weight(const MoeGroupedParams& p, int row, int k) {
+  return p.weight_in && k < p.top ? 1.0f : slot_weight(p, row, k);
+}
+DEV float in_weight(const MoeGroupedParams& p, int id) {
+  if (!p.weight_in) return 1.0f;
+  const int row = id / p.S, k = id - row * p.S;
+  return k < p.top ? slot_weight(p, row, k) : 1.0f;
+}
+
 constexpr int kMoeRows = 64;  // rows of one expert per workgroup tile: four 16-row MFMA tiles share every weight fragment
 
 __global__ __launch_bounds__(256) void moe_align_kernel(MoeGroupedParams p) {
@@ -267,7 +283,8 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(MoeGroupedParams p) {
   for (int j = 0; j < 4; ++j) {
     const int id2 = ids[16 * wave + 4 * g + j];
     if (id2 < 0) continue;
-    const float gv = ag[0][j], uv = au[0][j];
+    const float wi = in_weight(p, id2);
+    const float gv = ag[0][j] * wi, uv = au[0][j] * wi;
     reinterpret_cast<T*>(p.h)[(int64_t)id2 * p.ldh + f] =
         (T)(gated ? gv / (1.0f + expf(-gv)) * uv : (uv > 0.0f ? uv * uv : 0.0f));
   }
@@ -317,7 +334,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeGroupedParams p) {
     const int id2 = ids[16 * wave + 4 * g + j];
     if (id2 < 0) continue;
     const int row = id2 / p.S, k = id2 % p.S;
-    const float wgt = k < p.top ? p.topk_w[row * p.top + k] : 1.0f;
+    const float wgt = out_weight(p, row, k);
     p.o[(int64_t)id2 * p.W + d] = wgt * acc[0][j];
   }
 }
@@ -438,18 +455,19 @@ __global__ __launch_bounds__(256) void moe_tile_lds_kernel(MoeGroupedParams p) {
       if (MODE == 0) {
         const int f = n0 + 16 * wave + r;
         if (f >= N) continue;
-        const float gv = acc[i][0][j];
-        reinterpret_cast<bf16*>(p.h)[(int64_t)id * p.ldh + f] = (bf16)(gv / (1.0f + expf(-gv)) * acc[i][1][j]);
+        const float wi = in_weight(p, id);
+        const float gv = acc[i][0][j] * wi;
+        reinterpret_cast<bf16*>(p.h)[(int64_t)id * p.ldh + f] = (bf16)(gv / (1.0f + expf(-gv)) * (acc[i][1][j] * wi));
       } else if (MODE == 2) {
 #pragma unroll
         for (int q = 0; q < 2; ++q) {
           const int f = n0 + 32 * wave + 16 * q + r;
-          const float uv = acc[i][q][j];
+          const float uv = acc[i][q][j] * in_weight(p, id);
           if (f < N) reinterpret_cast<bf16*>(p.h)[(int64_t)id * p.ldh + f] = (bf16)(uv > 0.0f ? uv * uv : 0.0f);
         }
       } else {
         const int row = id / p.S, k = id % p.S;
-        const float wgt = k < p.top ? p.topk_w[row * p.top + k] : 1.0f;
+        const float wgt = out_weight(p, row, k);
 #pragma unroll
         for (int q = 0; q < 2; ++q) {
           const int d = n0 + 32 * wave + 16 * q + r;

@@ -188,12 +188,14 @@ __global__ __launch_bounds__(256) void act_rows_kernel(const float* x, int ldx, 
 // ranks, and every pick is a wave-wide argmax (ties go to the lower index, as in the reference).
 constexpr int kMaxRouteExperts = 256;
 
-__global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ corr, int M,
-                                                       int E, int top, int groups, int keep, float scale, int kind,
-                                                       int* topk_idx, float* topk_w) {
+__global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, int ldz,
+                                                       const float* __restrict__ corr, int M, int E, int top, int groups,
+                                                       int keep, float scale, int kind, int* topk_idx, float* topk_w,
+                                                       int ldw) {
   __shared__ float choice[kMaxRouteExperts], score[kMaxRouteExperts], gs[kMaxRouteExperts];
   const int row = blockIdx.x, lane = threadIdx.x;
-  const float* zr = z + (int64_t)row * E;
+  const float* zr = z + (int64_t)row * ldz;
+  float* wr = topk_w + (int64_t)row * ldw;
   const float ninf = -__builtin_inff();
   float zmax = ninf, zsum = 0.f;
   if (kind == 1) {  // softmax over all experts: the row's maximum and the sum of exponentials, wave-wide
@@ -225,7 +227,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
         if (c > a) b = a, a = c;
         else if (c > b) b = c;
       }
-      gs[o] = per > 1 && kind == 0 ? a + b : a;
+      gs[o] = per > 1 && kind != 1 ? a + b : a;
     }
     __syncthreads();
     // rank of a group = groups with a larger score (or the same score and a lower index); eligible when rank < keep
@@ -259,13 +261,17 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
     if (lane == 0) {
       choice[best] = __builtin_nanf("");  // taken: out of every later pick
       topk_idx[(int64_t)row * top + k] = best;
-      topk_w[(int64_t)row * top + k] = sg;
+      wr[k] = sg;
     }
     __syncthreads();
   }
-  const float inv = kind == 1 ? scale : scale / (sum + 1e-20f);
+  const float inv = kind >= 1 ? scale : scale / (sum + 1e-20f);
   __syncthreads();
-  for (int k = lane; k < top; k += 64) topk_w[(int64_t)row * top + k] *= inv;
+  for (int k = lane; k < top; k += 64) wr[k] *= inv;
+  if (ldw > top && lane == 0) {  // a shared expert's gate rides as one more logit
+    const float v = zr[E];
+    wr[top] = 1.0f / (1.0f + expf(-(v == v ? v : 0.0f)));
+  }
 }
 
 inline int flat_blocks(int64_t n) {
@@ -328,12 +334,14 @@ extern "C" hipError_t dsse_act_rows(const float* x, int ldx, void* out, int M, i
   return hipGetLastError();
 }
 
-extern "C" hipError_t dsse_moe_route(const float* z, const float* corr, int M, int E, int top, int groups, int keep,
-                                     float scale, int kind, int* topk_idx, float* topk_w, hipStream_t st) {
+extern "C" hipError_t dsse_moe_route(const float* z, int ldz, const float* corr, int M, int E, int top, int groups,
+                                     int keep, float scale, int kind, int* topk_idx, float* topk_w, int ldw,
+                                     hipStream_t st) {
   if (M <= 0) return hipSuccess;
   if (E > dsse::kMaxRouteExperts || groups < 1 || E % groups || top > E) return hipErrorInvalidValue;
-  if ((kind != 0 && kind != 1) || (kind == 0 && !corr)) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(dsse::moe_route_kernel, dim3(M), dim3(64), 0, st, z, corr, M, E, top, groups, keep, scale, kind,
-                     topk_idx, topk_w);
+  if (kind < 0 || kind > 2 || (kind == 0 && !corr)) return hipErrorInvalidValue;
+  if (ldw < top || ldz < E + (ldw > top ? 1 : 0)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(dsse::moe_route_kernel, dim3(M), dim3(64), 0, st, z, ldz, corr, M, E, top, groups, keep, scale, kind,
+                     topk_idx, topk_w, ldw);
   return hipGetLastError();
 }

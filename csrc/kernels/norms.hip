@@ -49,15 +49,23 @@ __global__ __launch_bounds__(256) void scalar_norm_kernel(ScalarNormParams p) {
 
 template <typename T>
 __global__ __launch_bounds__(256) void embed_rows_kernel(int W, int vocab, const int* ids, const T* embed, float* resid,
-                                                         T* xb) {
+                                                         T* xb, float scale, const int* positions, const float* table,
+                                                         int table_len) {
   const int row = blockIdx.x;
   int id = ids[row];
   id = (unsigned)id < (unsigned)vocab ? id : 0;  // padded / inactive rows carry any id
   const T* e = embed + (int64_t)id * W;
+  const float* t = nullptr;
+  if (table) {  // a vector per position (padded rows carry any position)
+    int pos = positions[row];
+    pos = pos < 0 ? 0 : (pos < table_len ? pos : table_len - 1);
+    t = table + (int64_t)pos * W;
+  }
   for (int d = threadIdx.x; d < W; d += blockDim.x) {
-    const T v = e[d];
-    resid[(int64_t)row * W + d] = (float)v;
-    xb[(int64_t)row * W + d] = v;
+    float v = (float)e[d] * scale;
+    if (t) v += t[d];
+    resid[(int64_t)row * W + d] = v;
+    if (xb) xb[(int64_t)row * W + d] = (T)v;
   }
 }
 
@@ -72,13 +80,17 @@ extern "C" hipError_t dsse_scalar_norm(const dsse::ScalarNormParams* p, hipStrea
 }
 
 extern "C" hipError_t dsse_embed_rows(int M, int W, int vocab, const int* ids, const void* embed, float* resid, void* xb,
-                                      int f32, hipStream_t st) {
+                                      float scale, const int* positions, const float* table, int table_len, int f32,
+                                      hipStream_t st) {
   if (M <= 0) return hipSuccess;
+  if (table && (!positions || table_len < 1)) return hipErrorInvalidValue;
   if (f32)
     hipLaunchKernelGGL(dsse::embed_rows_kernel<float>, dim3(M), dim3(256), 0, st, W, vocab, ids,
-                       reinterpret_cast<const float*>(embed), resid, reinterpret_cast<float*>(xb));
+                       reinterpret_cast<const float*>(embed), resid, reinterpret_cast<float*>(xb), scale, positions, table,
+                       table_len);
   else
     hipLaunchKernelGGL(dsse::embed_rows_kernel<bf16>, dim3(M), dim3(256), 0, st, W, vocab, ids,
-                       reinterpret_cast<const bf16*>(embed), resid, reinterpret_cast<bf16*>(xb));
+                       reinterpret_cast<const bf16*>(embed), resid, reinterpret_cast<bf16*>(xb), scale, positions, table,
+                       table_len);
   return hipGetLastError();
 }

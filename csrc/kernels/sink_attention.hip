@@ -9,6 +9,10 @@
 // pairs (m, m + V / 2), angles from a (cos, sin) table), before the gate: with values that were rotated by THEIR
 // positions when they were cached, a value then enters the output rotated by its distance to the query.
 //
+// A gate may also have one column per element of the output instead of one per head.  Distance bias and kept keys: an
+// entry rel[h][min(pos - j, rel_len - 1)] joins the score (after the scale), and the sequence's first keep_first keys stay
+// visible when the window has passed them: the kernels then walk the kept keys first and jump to the window.
+//
 // The sink is a learned logit with no key and no value: it only enlarges the denominator, so a head can attend to
 // "nothing".  Scores, the running maximum, the weights and the output sums are fp32 in both element types; queries
 // arrive in fp32 (normed and rotated), keys and values are read from their pages in the cache's element type.
@@ -74,7 +78,10 @@ __global__ __launch_bounds__(256) void sink_attention_kernel(SinkAttnParams p) {
     const int row = p.q_start[seq] + off;
     const int pos = p.ctx_len[seq] - ql + off;
     const int lo = pos - p.window + 1 > 0 ? pos - p.window + 1 : 0;
-    const int nkeys = pos - lo + 1;
+    const int kept = p.keep_first < lo ? p.keep_first : lo;  // keys 0 .. kept - 1 are walked ahead of the window's
+    const int nkeys = kept + pos - lo + 1;
+    const int last_rel = p.rel_len - 1;
+    const float* rel = p.rel ? p.rel + (int64_t)h * p.rel_len : nullptr;
     __syncthreads();  // the previous row's merge has read qs / acc_s
     for (int d = threadIdx.x; d < D; d += blockDim.x) qs[d] = p.q[((int64_t)row * p.H + h) * D + d];
     __syncthreads();
@@ -85,13 +92,15 @@ __global__ __launch_bounds__(256) void sink_attention_kernel(SinkAttnParams p) {
     for (int c = wave; c * 64 < nkeys; c += 4) {
       const int jj = c * 64 + lane;
       const bool on = jj < nkeys;
-      const int j = lo + (on ? jj : 0);
+      const int j0 = on ? jj : 0;
+      const int j = j0 < kept ? j0 : lo + j0 - kept;
       int page = bt[j / kBS];
       page = (unsigned)page < (unsigned)p.num_blocks ? page : 0;
       const int krow = (page * kBS + j % kBS) * p.G + g;
       const float s_dot = dot_row(qs, kc + (int64_t)krow * D, D);
       float s = s_dot * p.scale;
       if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
+      if (rel) s += rel[pos - j < last_rel ? pos - j : last_rel];
       s = on ? s : -INFINITY;
       const float m_new = fmaxf(m, wave_max(s));  // finite: the chunk holds at least one key
       const float w = on ? expf(s - m_new) : 0.f;
@@ -126,7 +135,8 @@ __global__ __launch_bounds__(256) void sink_attention_kernel(SinkAttnParams p) {
       fw[w] = m_s[w] == -INFINITY ? 0.f : expf(m_s[w] - mm);
       den += l_s[w] * fw[w];
     }
-    const float gate = p.gate ? 1.0f / (1.0f + expf(-p.gate[(int64_t)row * p.ldg + h])) : 1.0f;
+    const float* gp = p.gate ? p.gate + (int64_t)row * p.ldg + (p.gate_wide ? h * p.V : h) : nullptr;
+    const float gate = gp && !p.gate_wide ? 1.0f / (1.0f + expf(-gp[0])) : 1.0f;
     T* out = reinterpret_cast<T*>(p.out) + ((int64_t)row * p.H + h) * V;
     const int half = V >> 1;
     const float2* orp = p.out_rope ? p.out_rope + (int64_t)(pos < p.out_rope_len ? pos : p.out_rope_len - 1) * half : nullptr;
@@ -141,7 +151,9 @@ __global__ __launch_bounds__(256) void sink_attention_kernel(SinkAttnParams p) {
         const float2 c = orp[lo_half ? d : dp];
         o = lo_half ? o * c.x + op * c.y : o * c.x - op * c.y;
       }
-      out[d] = (T)(o / den * gate);
+      o = o / den * gate;
+      if (p.gate_wide) o *= 1.0f / (1.0f + expf(-gp[d]));
+      out[d] = (T)o;
     }
   }
 }
@@ -173,8 +185,11 @@ DEV float tanh_fast(float x) {
   return (e - 1.0f) / (e + 1.0f);
 }
 
-template <int NT, bool SPLIT>  // V / 16 value tiles
-__global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const bf16* __restrict__ vt, int head_tiles) {
+// NT: V / 16 value tiles.  EXT: the kept first keys and the distance bias (its first rel_lds entries per head in LDS, the
+// rest read from memory; pages whose keys are all so far away that they share the last entry look nothing up).
+template <int NT, bool SPLIT, bool EXT>
+__global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const bf16* __restrict__ vt, int head_tiles,
+                                                         int rel_lds) {
   extern __shared__ __align__(16) unsigned char smem_raw[];
   const int D = p.D, V = p.V;
   const int ldq = D + 8;  // bf16 elements per LDS row (16 B of padding)
@@ -204,6 +219,16 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
       *reinterpret_cast<bf16x8*>(qs + r * ldq + d) = v;
     }
   }
+  // the heads' bias entries behind the query tiles (SPLIT: one head; otherwise one strip per wave)
+  float* rels = reinterpret_cast<float*>(smem_raw + (blockDim.x >> 6) * 16 * ldq * sizeof(bf16));
+  const float* relg = nullptr;
+  float rel_far = 0.f;
+  if (EXT && p.rel) {
+    relg = p.rel + (int64_t)hh * p.rel_len;
+    rel_far = relg[p.rel_len - 1];
+    if (!SPLIT) rels += wave * rel_lds;
+    for (int i = SPLIT ? (int)threadIdx.x : lane; i < rel_lds; i += SPLIT ? (int)blockDim.x : 64) rels[i] = relg[i];
+  }
   __syncthreads();
   if (!SPLIT && !h_ok) return;
   const int last_off = tile * 16 + 15 < ql ? tile * 16 + 15 : ql - 1;
@@ -218,7 +243,15 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
   float m = -INFINITY, l = 0.f;
   const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f;
   const int nks = D / 32;
-  for (int pg = lo / kBS + (SPLIT ? wave : 0); pg <= hi / kBS; pg += SPLIT ? 4 : 1) {
+  const int pg_lo = lo / kBS;
+  int kept_pages = 0;  // whole pages of kept keys before the window's first page
+  if (EXT && p.keep_first > 0) {
+    kept_pages = (p.keep_first + kBS - 1) / kBS;
+    kept_pages = kept_pages < pg_lo ? kept_pages : pg_lo;
+  }
+  const int walk = kept_pages + hi / kBS - pg_lo + 1;
+  for (int pi = SPLIT ? wave : 0; pi < walk; pi += SPLIT ? 4 : 1) {
+    const int pg = pi < kept_pages ? pi : pg_lo + pi - kept_pages;
     int blk = bt[pg];
     blk = (unsigned)blk < (unsigned)p.num_blocks ? blk : 0;
     const bf16* krow0 = kc + (((int64_t)blk * kBS + r) * p.G + kvh) * D + 8 * g;  // key r of the page's first half
@@ -247,12 +280,23 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
     }
     float sv[8];
     float mx = -INFINITY;
+    // uniform: every (row, key) pair of this tile and page is at least rel_len - 1 apart
+    const bool far = EXT && p.rel && pos0 + tile * 16 - (pg * kBS + kBS - 1) >= p.rel_len - 1;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
-      const bool seen = c_ok && key <= c_pos && c_pos - key < p.window;
+      const bool seen = c_ok && key <= c_pos && (c_pos - key < p.window || (EXT && key < p.keep_first));
       float sc = (i < 4 ? s0[i] : s1[i - 4]) * p.scale;
       if (p.softcap > 0.f) sc = p.softcap * tanh_fast(sc * cap_inv);
+      if (EXT && p.rel) {
+        if (far) {
+          sc += rel_far;
+        } else {
+          int n = c_pos - key;
+          n = n < 0 ? 0 : (n < p.rel_len ? n : p.rel_len - 1);
+          sc += n < rel_lds ? rels[n] : relg[n];
+        }
+      }
       sv[i] = seen ? sc : -INFINITY;
       mx = fmaxf(mx, sv[i]);
     }
@@ -279,7 +323,7 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
   }
   if (SPLIT) {
     // merge the four waves' partial results: [wave][16 columns][V + 2] floats, after every wave has read its queries
-    float* mg = reinterpret_cast<float*>(smem_raw) + 4 * 16 * ((ldq + 1) / 2);
+    float* mg = reinterpret_cast<float*>(smem_raw) + 4 * 16 * ((ldq + 1) / 2) + rel_lds;
     const int ldm = V + 2;
     float* mine = mg + (wave * 16 + r) * ldm;
 #pragma unroll
@@ -314,7 +358,7 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
         num = lo_half ? num * c.x + nump * c.y : num * c.x - nump * c.y;
       }
       float o = den > 0.f ? num / den : 0.f;
-      if (p.gate) o *= 1.0f / (1.0f + expf(-p.gate[row * p.ldg + h]));
+      if (p.gate) o *= 1.0f / (1.0f + expf(-p.gate[row * p.ldg + (p.gate_wide ? h * V + d : h)]));
       reinterpret_cast<bf16*>(p.out)[(row * p.H + h) * V + d] = (bf16)o;
     }
     return;
@@ -328,7 +372,7 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
       den = l * f + expf(sk - mm);
     }
     float inv = den > 0.f ? f / den : 0.0f;
-    if (p.gate) inv *= 1.0f / (1.0f + expf(-p.gate[c_row * p.ldg + h]));
+    if (p.gate && !p.gate_wide) inv *= 1.0f / (1.0f + expf(-p.gate[c_row * p.ldg + h]));
     if (p.out_rope) {  // NT is even (the host checks V % 32 == 0): dimension m = 16 n + 4 g + i pairs with tile n + NT / 2
       const float2* orp = p.out_rope + (int64_t)(c_pos < p.out_rope_len ? c_pos : p.out_rope_len - 1) * (V >> 1);
 #pragma unroll
@@ -342,27 +386,50 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
         }
     }
     bf16* out = reinterpret_cast<bf16*>(p.out) + (c_row * p.H + h) * V;
+    const float* gw = p.gate_wide ? p.gate + c_row * p.ldg + h * V + 4 * g : nullptr;
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       bf16x4 v;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) v[i] = (bf16)(O[n][i] * inv);
+      for (int i = 0; i < 4; ++i) {
+        float o = O[n][i] * inv;
+        if (gw) o *= 1.0f / (1.0f + expf(-gw[16 * n + i]));
+        v[i] = (bf16)o;
+      }
       *reinterpret_cast<bf16x4*>(out + 16 * n + 4 * g) = v;
     }
   }
 }
 
-template <int NT>
-void launch_flash(int num_work, const SinkAttnParams& p, const bf16* vt, int split, hipStream_t st) {
+constexpr size_t kFlashLds = 64 * 1024;
+
+template <int NT, bool EXT>
+void launch_flash_ext(int num_work, const SinkAttnParams& p, const bf16* vt, int split, hipStream_t st) {
   const size_t qbytes = 16 * (size_t)(p.D + 8) * sizeof(bf16);
-  if (split) {  // one head per workgroup, its four waves share the keys; LDS: 4 query tiles + the merge area
-    const size_t lds = 4 * 16 * (size_t)((p.D + 8 + 1) / 2) * sizeof(float) + 4 * 16 * (size_t)(p.V + 2) * sizeof(float);
-    hipLaunchKernelGGL((sink_flash_kernel<NT, true>), dim3(num_work, p.H), dim3(256), lds, st, p, vt, p.H);
+  auto strip = [&](size_t used, int strips) {  // bias entries per head that fit beside the rest, at most 1024
+    if (!EXT || !p.rel || used >= kFlashLds) return 0;
+    const size_t room = (kFlashLds - used) / (strips * sizeof(float));
+    const size_t want = p.rel_len < 1024 ? (size_t)p.rel_len : 1024;
+    return (int)(want < room ? want : room);
+  };
+  if (split) {  // one head per workgroup, its four waves share the keys; LDS: 4 query tiles + bias + the merge area
+    size_t lds = 4 * 16 * (size_t)((p.D + 8 + 1) / 2) * sizeof(float) + 4 * 16 * (size_t)(p.V + 2) * sizeof(float);
+    const int rel_lds = strip(lds, 1);
+    lds += rel_lds * sizeof(float);
+    hipLaunchKernelGGL((sink_flash_kernel<NT, true, EXT>), dim3(num_work, p.H), dim3(256), lds, st, p, vt, p.H, rel_lds);
     return;
   }
   const int wy = p.H < 4 ? p.H : 4;
+  const int rel_lds = strip(wy * qbytes, wy);
   dim3 grid(num_work, (p.H + wy - 1) / wy), block(64 * wy);
-  hipLaunchKernelGGL((sink_flash_kernel<NT, false>), grid, block, wy * qbytes, st, p, vt, p.H);
+  hipLaunchKernelGGL((sink_flash_kernel<NT, false, EXT>), grid, block, wy * (qbytes + rel_lds * sizeof(float)), st, p, vt,
+                     p.H, rel_lds);
+}
+
+template <int NT>
+void launch_flash(int num_work, const SinkAttnParams& p, const bf16* vt, int split, hipStream_t st) {
+  if (p.rel || p.keep_first > 0) launch_flash_ext<NT, true>(num_work, p, vt, split, st);
+  else launch_flash_ext<NT, false>(num_work, p, vt, split, st);
 }
 
 }  // namespace

@@ -124,6 +124,9 @@ FLASH_ROWS_TILE = 4   # query rows per work item of the MFMA attention form, x 4
                       # read once for four heads (16 rows x 1 head re-read it per head: 2-3x the time at 16 heads)
 
 
+LDS_BYTES = 64 * 1024  # what an attention launch may ask for
+
+
 class LayeredRunner(RunnerBase):
     def __init__(self, w: LayeredWeights, num_blocks: int, max_batch: int = 64, max_model_len: int = 4096,
                  max_prefill_tokens: int = 8192, device="cuda", comm: TPComm | None = None, use_graphs=None):
@@ -986,7 +989,8 @@ class LayeredRunner(RunnerBase):
 
         cfg, dev = self.cfg, self.device
         kv = {i: (L.mixer.kv_heads, L.mixer.dim, L.mixer.vdim) for i, L in enumerate(cfg.layers) if cfg.kv_layer(i) == i}
-        flash = [i for i, (_, dm, v) in kv.items() if ops.sink_flash_ok(self.dtype, dm, v)]
+        flash = [i for i, (_, dm, v) in kv.items() if ops.sink_flash_ok(self.dtype, dm, v) and
+                 ops.sink_flash_lds(dm) <= LDS_BYTES]
         self.kv = PagedKVCache(kv, self.num_blocks, dev, self.dtype, transposed=flash)
         self.state = MatrixStateCache({}, self.max_batch, dev)  # no layer keeps state beside its pages
         self._pos_table = position_table(self.max_model_len + 1, cfg.width, dev)
@@ -1053,7 +1057,7 @@ class LayeredRunner(RunnerBase):
         for g in groups:
             if vt is not None and g["qt"] > 1:
                 work, form = (g["hs"], g["ht"]), (SINK_ROWS_TILE, vt, False)
-            elif vt is not None and V <= ops.layers.SINK_SPLIT_MAX_V:
+            elif vt is not None and V <= ops.layers.SINK_SPLIT_MAX_V and ops.sink_flash_lds(D, V, True) <= LDS_BYTES:
                 work, form = (g["ws"], g["wt"]), (SINK_ROWS_TILE, vt, True)
             else:
                 work, form = (g["ws"], g["wt"]), (g["qt"], None, False)

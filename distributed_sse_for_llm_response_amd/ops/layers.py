@@ -190,6 +190,11 @@ def sink_flash_ok(dtype, dim: int, vdim: int) -> bool:
     return dtype == torch.bfloat16 and dim % 32 == 0 and dim <= 512 and vdim % 16 == 0 and vdim // 16 in SINK_FLASH_TILES
 
 
+def sink_flash_lds(dim: int, vdim: int = 0, split: bool = False) -> int:
+    """LDS bytes of the MFMA form before a distance bias: four waves' query tiles, and the key split's merge area."""
+    return 4 * 16 * ((dim + 8) * 2 + ((vdim + 2) * 4 if split else 0))
+
+
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile, sink, gate, out,
                    window: int, scale: float, qt: int, vt=None, split: bool = False, softcap: float = 0.0, out_rope=None,
                    rel=None, keep_first: int = 0):

@@ -157,8 +157,23 @@ struct MoeGroupedParams {
   float* o;              // [M * S, W]
   int M, W, F, Fs, E, top, S, ldh, max_tiles;
   int vec_w, vec_h;      // 16-byte fragment loads allowed on rows W wide / on rows of h
+  int aligned;           // 1: sorted / tile_expert / num_tiles are already made (moe_route_rows)
   int lds_tiles;         // 1: enough rows for the LDS-staged tiles (prompt portions); 0: the register-direct kernels
   int f32;
+};
+
+// Router, choice and work list of a decode-sized step in one launch.
+struct MoeRouteRowsParams {
+  const float* x;        // [M, W]
+  const float* w;        // [E (+ 1: a shared expert's gate), W]
+  int* topk_idx;         // [M, top]
+  float* topk_w;         // [M, S]: sigmoid scores as they are times scale; column top: the shared expert's gate
+  int* sorted;           // as in MoeGroupedParams
+  int* tile_expert;
+  int* num_tiles;        // [2]: tiles | arrivals (0 before the first launch, left at 0)
+  int M, W, E, top, S, max_tiles;
+  int vec;               // 16-byte loads allowed
+  float scale;
 };
 
 }  // namespace dsse
@@ -180,5 +195,6 @@ hipError_t dsse_lru_scan(const dsse::LruScanParams* p, hipStream_t st);
 hipError_t dsse_moe_router(const dsse::MoeRouterParams* p, hipStream_t st);
 hipError_t dsse_moe_ffn(const dsse::MoeFfnParams* p, hipStream_t st);
 hipError_t dsse_moe_grouped(const dsse::MoeGroupedParams* p, hipStream_t st);
+hipError_t dsse_moe_route_rows(const dsse::MoeRouteRowsParams* p, hipStream_t st);
 hipError_t dsse_moe_topk(const float* z, int M, int E, int top, int* topk_idx, float* topk_w, hipStream_t st);
 }

@@ -228,6 +228,8 @@ hipError_t dsse_sink_attention(int num_work, const dsse::SinkAttnParams* p, hipS
 // transposed pages vt [pages, G, V, kBS] (keys permuted inside a page as the MFMA's k axis wants them)
 // split (V <= 128): the four waves of a workgroup share one (tile, head) and split its pages -- decode steps
 hipError_t dsse_sink_flash(int num_work, const dsse::SinkAttnParams* p, const void* vt, int split, hipStream_t st);
+// decode form over the same pages: one row per item, the heads of a key/value group side by side, pages split over waves
+hipError_t dsse_sink_decode(int num_work, const dsse::SinkAttnParams* p, const void* vt, hipStream_t st);
 // p1 / p2 hold N / rep1 and N / rep2 numbers: entry j serves columns [j rep, (j + 1) rep)
 hipError_t dsse_gate_math(float* x, int ld, int M, int N, int kind, const float* p1, int rep1, const float* p2, int rep2,
                           float c, hipStream_t st);

@@ -452,7 +452,8 @@ void moe_ffn(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, cons
 // tile_expert [tiles], num_tiles [1] (int32), h [M * S, ldh] (element type), tiles >= ceil(M S / 64) + experts + 1.
 void moe_grouped(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, const OptTensor& gate, const Tensor& up,
                  const Tensor& down, const OptTensor& sgate, const OptTensor& sup, const OptTensor& sdown, Tensor& sorted,
-                 Tensor& tile_expert, Tensor& num_tiles, Tensor& h, Tensor& o, bool weight_input) {
+                 Tensor& tile_expert, Tensor& num_tiles, Tensor& h, Tensor& o, bool weight_input,
+                 bool aligned) {
   gpu(x, "x");
   i32(topk_idx, "topk_idx");
   f32t(topk_w, "topk_w");
@@ -483,6 +484,7 @@ void moe_grouped(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, 
               "routing shapes");
   p.ldw = (int)topk_w.size(1);
   p.weight_in = weight_input ? 1 : 0;
+  p.aligned = aligned ? 1 : 0;
   p.S = p.top;
   if (sgate.has_value()) {
     TORCH_CHECK(sup.has_value() && sdown.has_value(), "the shared expert needs gate, up and down");
@@ -528,6 +530,41 @@ void moe_grouped(const Tensor& x, const Tensor& topk_idx, const Tensor& topk_w, 
   DSSE_CHECK_HIP(dsse_moe_grouped(&p, cur_stream()));
 }
 
+// Router GEMM (fp32), choice by sigmoid scores and the work list of moe_grouped in one launch: w holds one row per expert,
+// and one more for a shared expert's gate when topk_w has a column for it.
+void moe_route_rows(const Tensor& x, const Tensor& w, Tensor& topk_idx, Tensor& topk_w, double scale, Tensor& sorted,
+                    Tensor& tile_expert, Tensor& num_tiles) {
+  f32t(x, "x");
+  f32t(w, "w");
+  i32(topk_idx, "topk_idx");
+  f32t(topk_w, "topk_w");
+  i32(sorted, "sorted");
+  i32(tile_expert, "tile_expert");
+  i32(num_tiles, "num_tiles");
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1) && topk_idx.dim() == 2 && topk_w.dim() == 2,
+              "x [M, W], w [experts, W]");
+  dsse::MoeRouteRowsParams p{};
+  p.M = (int)x.size(0), p.W = (int)x.size(1), p.top = (int)topk_idx.size(1), p.S = (int)topk_w.size(1);
+  p.E = (int)w.size(0) - (p.S - p.top);
+  TORCH_CHECK(topk_idx.size(0) == p.M && topk_w.size(0) == p.M && (p.S == p.top || p.S == p.top + 1) && p.top >= 1 &&
+                  p.top <= p.E && p.E <= 256,
+              "routing shapes: 1 <= top <= experts <= 256");
+  const int64_t ids = (int64_t)p.M * p.S;
+  p.max_tiles = (int)tile_expert.numel();
+  TORCH_CHECK(p.max_tiles >= (ids + 63) / 64 + p.E + 1 && sorted.numel() >= (int64_t)p.max_tiles * 64 && num_tiles.numel() >= 2,
+              "moe_route_rows: scratch too small for ", ids, " ids");
+  p.x = x.data_ptr<float>();
+  p.w = w.data_ptr<float>();
+  p.topk_idx = topk_idx.data_ptr<int>();
+  p.topk_w = topk_w.data_ptr<float>();
+  p.sorted = sorted.data_ptr<int>();
+  p.tile_expert = tile_expert.data_ptr<int>();
+  p.num_tiles = num_tiles.data_ptr<int>();
+  p.vec = p.W % 4 == 0 && reinterpret_cast<uintptr_t>(p.x) % 16 == 0 && reinterpret_cast<uintptr_t>(p.w) % 16 == 0;
+  p.scale = (float)scale;
+  DSSE_CHECK_HIP(dsse_moe_route_rows(&p, cur_stream()));
+}
+
 void moe_topk(const Tensor& logits, Tensor& topk_idx, Tensor& topk_w) {
   f32t(logits, "logits");
   i32(topk_idx, "topk_idx");
@@ -547,7 +584,9 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
   m.def("scalar_norm(Tensor? y, Tensor g, Tensor(a!) resid, Tensor(b!) xb, float eps, int nsum=1) -> ()");
   m.def("moe_grouped(Tensor x, Tensor topk_idx, Tensor topk_w, Tensor? gate, Tensor up, Tensor down, Tensor? sgate, "
         "Tensor? sup, Tensor? sdown, Tensor(a!) sorted, Tensor(b!) tile_expert, Tensor(c!) num_tiles, Tensor(d!) h, "
-        "Tensor(e!) o, bool weight_input=False) -> ()");
+        "Tensor(e!) o, bool weight_input=False, bool aligned=False) -> ()");
+  m.def("moe_route_rows(Tensor x, Tensor w, Tensor(a!) topk_idx, Tensor(b!) topk_w, float scale, Tensor(c!) sorted, "
+        "Tensor(d!) tile_expert, Tensor(e!) num_tiles) -> ()");
   m.def("embed_rows(Tensor ids, Tensor embed, Tensor(a!) resid, Tensor(b!)? xb, float scale=1.0, Tensor? positions=None, "
         "Tensor? table=None) -> ()");
   m.def("latent_kv_write(Tensor ckr, Tensor norm_w, Tensor positions, Tensor slots, Tensor rope, Tensor(a!) cache, "
@@ -579,4 +618,5 @@ TORCH_LIBRARY_IMPL(dsse, CUDA, m) {
   m.impl("moe_topk", &moe_topk);
   m.impl("moe_ffn", &moe_ffn);
   m.impl("moe_grouped", &moe_grouped);
+  m.impl("moe_route_rows", &moe_route_rows);
 }

@@ -239,7 +239,7 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
     f32t(*out_rope, "out_rope");
     TORCH_CHECK(out_rope->dim() == 3 && out_rope->size(2) == 2 && 2 * out_rope->size(1) == p.V && out_rope->size(0) >= 1,
                 "out_rope must be [P, V / 2, 2]");
-    TORCH_CHECK(!vt.has_value() || p.V % 32 == 0, "the MFMA form turns outputs back only for V % 32 == 0");
+    TORCH_CHECK(!vt.has_value() || qt == 1 || p.V % 32 == 0, "the MFMA form turns outputs back only for V % 32 == 0");
     p.out_rope = reinterpret_cast<const float2*>(out_rope->data_ptr<float>());
     p.out_rope_len = (int)out_rope->size(0);
   }
@@ -249,6 +249,12 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
     TORCH_CHECK(vt->dim() == 4 && vt->size(0) == vcache.size(0) && vt->size(1) == p.G && vt->size(2) == p.V &&
                     vt->size(3) == dsse::kBS,
                 "vt must be [pages, G, V, 32]");
+    if (qt == 1) {  // decode form: one row per item
+      TORCH_CHECK(p.D % 32 == 0 && p.V % 16 == 0 && !split, "the decode form needs D % 32 == 0, V % 16 == 0, no split");
+      TORCH_CHECK(p.G <= 65535 && p.H / p.G <= 16 * 65535, "too many heads");
+      DSSE_CHECK_HIP(dsse_sink_decode((int)work_seq.numel(), &p, vt->data_ptr(), cur_stream()));
+      return;
+    }
     TORCH_CHECK(qt == 16 && p.D % 32 == 0 && p.V % 16 == 0, "the MFMA form needs qt = 16, D % 32 == 0, V % 16 == 0");
     TORCH_CHECK(!split || p.V <= 128, "the key split of the MFMA form needs V <= 128");
     DSSE_CHECK_HIP(dsse_sink_flash((int)work_seq.numel(), &p, vt->data_ptr(), split ? 1 : 0, cur_stream()));

@@ -170,87 +170,267 @@ DEV float in_weight(const MoeGroupedParams& p, int id) {
 
 constexpr int kMoeRows = 64;  // rows of one expert per workgroup tile: four 16-row MFMA tiles share every weight fragment
 
-__global__ __launch_bounds__(256) void moe_align_kernel(MoeGroupedParams p) {
-  extern __shared__ int sm[];
-  const int NE = p.E + (p.S > p.top ? 1 : 0);
+// The work list from the choices, by one workgroup; sm holds 3 NE + 1 ints.  The choices are read with agent scope: in the
+// one-launch form below other workgroups of the same launch have just written them.
+DEV void align_ids(int M, int S, int top, int E, const int* topk_idx, int* sorted, int* tile_expert, int* num_tiles,
+                   int max_tiles, int* sm) {
+  const int NE = E + (S > top ? 1 : 0);
   int* cnt = sm;            // [NE]
   int* off = sm + NE;       // [NE + 1] first sorted position of each expert (multiples of kMoeRows)
   int* fill = off + NE + 1; // [NE]
-  const int n = p.M * p.S;
+  const int n = M * S;
+  auto expert_of = [&](int id) {
+    const int row = id / S, k = id % S;
+    const int e = k < top ? __hip_atomic_load(topk_idx + row * top + k, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) : E;
+    return (unsigned)e < (unsigned)NE ? e : 0;
+  };
+  const int mine = (int)threadIdx.x < n ? expert_of(threadIdx.x) : 0;  // a thread's first id: read once
   for (int e = threadIdx.x; e < NE; e += blockDim.x) cnt[e] = 0, fill[e] = 0;
   __syncthreads();
-  for (int id = threadIdx.x; id < n; id += blockDim.x) {
-    const int row = id / p.S, k = id % p.S;
-    int e = k < p.top ? p.topk_idx[row * p.top + k] : p.E;
-    e = (unsigned)e < (unsigned)NE ? e : 0;
-    atomicAdd(&cnt[e], 1);
-  }
+  for (int id = threadIdx.x; id < n; id += blockDim.x) atomicAdd(&cnt[id == (int)threadIdx.x ? mine : expert_of(id)], 1);
   __syncthreads();
-  if (threadIdx.x == 0) {
+  if (threadIdx.x < 64) {  // offsets: a wave's prefix sums over the padded counts, 64 experts at a time
+    const int lane = threadIdx.x;
     int at = 0;
-    for (int e = 0; e < NE; ++e) {
-      off[e] = at;
-      at += (cnt[e] + kMoeRows - 1) / kMoeRows * kMoeRows;
+    for (int e0 = 0; e0 < NE; e0 += 64) {
+      const int pad = e0 + lane < NE ? (cnt[e0 + lane] + kMoeRows - 1) / kMoeRows * kMoeRows : 0;
+      int sum = pad;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int v = __shfl_up(sum, o);
+        if (lane >= o) sum += v;
+      }
+      if (e0 + lane < NE) off[e0 + lane] = at + sum - pad;
+      at += __shfl(sum, 63);
     }
-    off[NE] = at;
-    *p.num_tiles = at / kMoeRows;
+    if (lane == 0) {
+      off[NE] = at;
+      *num_tiles = at / kMoeRows;
+    }
   }
   __syncthreads();
   const int total = off[NE];
-  for (int i = threadIdx.x; i < total; i += blockDim.x) p.sorted[i] = -1;
+  for (int i = threadIdx.x; i < total; i += blockDim.x) sorted[i] = -1;
   for (int e = threadIdx.x; e < NE; e += blockDim.x)
-    for (int t = off[e] / kMoeRows; t < off[e + 1] / kMoeRows; ++t) p.tile_expert[t] = e;
+    for (int t = off[e] / kMoeRows; t < off[e + 1] / kMoeRows; ++t) tile_expert[t] = e;
+  for (int t = total / kMoeRows + threadIdx.x; t < max_tiles; t += blockDim.x) tile_expert[t] = -1;
   __syncthreads();
   for (int id = threadIdx.x; id < n; id += blockDim.x) {
-    const int row = id / p.S, k = id % p.S;
-    int e = k < p.top ? p.topk_idx[row * p.top + k] : p.E;
-    e = (unsigned)e < (unsigned)NE ? e : 0;
-    p.sorted[off[e] + atomicAdd(&fill[e], 1)] = id;
+    const int e = id == (int)threadIdx.x ? mine : expert_of(id);
+    sorted[off[e] + atomicAdd(&fill[e], 1)] = id;
   }
 }
 
-// Both expert GEMMs: a workgroup owns 16 output columns of one 64-row tile; its four waves split the K axis (k-steps
-// w, w + 4, ...) and meet in LDS, where wave i finishes the tile's i-th 16-row sub-tile.  Sixteen columns per workgroup
-// give a decode step (17 tiles or so) thousands of workgroups to hide the weight stream's latency with.
-DEV void reduce4(f32x4 (&acc)[4], float* red, int wave, int lane) {
-  // red [wave][sub][reg][lane]; afterwards acc[wave] of every wave holds the sum over the four waves of sub-tile `wave`
+__global__ __launch_bounds__(256) void moe_align_kernel(MoeGroupedParams p) {
+  extern __shared__ int sm[];
+  align_ids(p.M, p.S, p.top, p.E, p.topk_idx, p.sorted, p.tile_expert, p.num_tiles, p.max_tiles, sm);
+}
+
+// Router, choice and work list of a decode-sized step in ONE launch (three latency-sized ones otherwise): a workgroup of
+// sixteen waves per row.  A wave makes the fp32 logits of up to four experts per pass over the row (the lanes split the
+// width, 16-byte loads), wave 0 picks the `top` largest sigmoid scores (ties to the lower index) and the shared expert's
+// gate, and the workgroup that finishes last -- a counter, nobody waits -- builds the list.
+constexpr int kRouteThreads = 1024;
+constexpr int kRouteLanes = 4;  // experts per lane in the choice: up to 256
+
+// s[u] += x . w[u] over this lane's share of the row, eight 16-byte loads of every operand in flight
+template <int NU>
+DEV void route_dots(const float* x, const float* const (&w)[4], int W, int lane, float (&s)[4]) {
+  int d = lane * 4;
+  for (; d + 7 * 256 < W; d += 8 * 256) {
+    f32x4 xv[8], wv[NU][8];
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < 8; ++i) {
+      xv[i] = ld_global<f32x4>(x + d + 256 * i);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) red[((wave * 4 + i) * 4 + j) * 64 + lane] = acc[i][j];
+      for (int u = 0; u < NU; ++u) wv[u][i] = ld_global<f32x4>(w[u] + d + 256 * i);
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+#pragma unroll
+      for (int u = 0; u < NU; ++u)
+#pragma unroll
+        for (int c = 0; c < 4; ++c) s[u] += xv[i][c] * wv[u][i][c];
+  }
+  for (; d < W; d += 256) {
+    const f32x4 xv = ld_global<f32x4>(x + d);
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      const f32x4 wv = ld_global<f32x4>(w[u] + d);
+#pragma unroll
+      for (int c = 0; c < 4; ++c) s[u] += xv[c] * wv[c];
+    }
+  }
+}
+
+__global__ __launch_bounds__(kRouteThreads) void moe_route_rows_kernel(MoeRouteRowsParams p) {
+  extern __shared__ int sm[];
+  __shared__ int last;
+  const int NE = p.E + (p.S > p.top ? 1 : 0);
+  float* z = reinterpret_cast<float*>(sm + 3 * NE + 1);  // [NE] logits
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  constexpr int kWaves = kRouteThreads / 64;
+  const int64_t row = blockIdx.x;
+  const float* x = p.x + row * p.W;
+  for (int e0 = wave; e0 < NE; e0 += 4 * kWaves) {
+    const float* w[4];
+    float s[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int u = 0; u < 4; ++u) w[u] = p.w + (int64_t)(e0 + u * kWaves < NE ? e0 + u * kWaves : e0) * p.W;
+    const int nu = e0 + kWaves >= NE ? 1 : (e0 + 2 * kWaves >= NE ? 2 : 4);  // uniform: experts of this pass (rounded up)
+    if (p.vec) {
+      if (nu == 1) route_dots<1>(x, w, p.W, lane, s);
+      else if (nu == 2) route_dots<2>(x, w, p.W, lane, s);
+      else route_dots<4>(x, w, p.W, lane, s);
+    } else {
+      for (int d = lane; d < p.W; d += 64)
+#pragma unroll
+        for (int u = 0; u < 4; ++u) s[u] += x[d] * w[u][d];
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (u >= nu) continue;
+      const float v = wave_sum(s[u]);
+      if (lane == 0 && e0 + u * kWaves < NE) z[e0 + u * kWaves] = v;
+    }
+  }
+  __syncthreads();
+  if (wave == 0) {
+    const float ninf = -__builtin_inff();
+    auto sigmoid = [](float v) { return 1.0f / (1.0f + expf(-(v == v ? v : 0.0f))); };
+    float sc[kRouteLanes];
+#pragma unroll
+    for (int i = 0; i < kRouteLanes; ++i) sc[i] = i * 64 + lane < p.E ? sigmoid(z[i * 64 + lane]) : ninf;
+    for (int k = 0; k < p.top; ++k) {
+      float bv = ninf;
+      int best = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < kRouteLanes; ++i)
+        if (sc[i] > bv) bv = sc[i], best = i * 64 + lane;
+#pragma unroll
+      for (int o = 32; o >= 1; o >>= 1) {
+        const float ov = __shfl_xor(bv, o);
+        const int oi = __shfl_xor(best, o);
+        if (ov > bv || (ov == bv && oi < best)) bv = ov, best = oi;
+      }
+#pragma unroll
+      for (int i = 0; i < kRouteLanes; ++i)
+        if (i * 64 + lane == best) sc[i] = ninf;  // taken
+      if (lane == 0) {
+        __hip_atomic_store(p.topk_idx + row * p.top + k, best, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        p.topk_w[row * p.S + k] = bv * p.scale;
+      }
+    }
+    if (lane == 0) {
+      if (p.S > p.top) p.topk_w[row * p.S + p.top] = sigmoid(z[p.E]);
+      // the choices before the count: they are agent-scope stores, so it is enough that they have been performed
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      const int n = __hip_atomic_fetch_add(p.num_tiles + 1, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      last = n == p.M - 1;
+      if (last) __hip_atomic_store(p.num_tiles + 1, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // for the next launch
+    }
+  }
+  __syncthreads();
+  if (!last) return;  // uniform for the workgroup; align_ids reads the choices with agent scope
+  align_ids(p.M, p.S, p.top, p.E, p.topk_idx, p.sorted, p.tile_expert, p.num_tiles, p.max_tiles, sm);
+}
+
+// Both expert GEMMs: a workgroup owns 16 output columns of one 64-row tile; its four waves split the K axis and meet in
+// LDS.  Sixteen columns per workgroup give a decode step (17 tiles or so) thousands of workgroups to hide the weight
+// stream's latency with.  SUBS: 16-row sub-tiles that can hold rows -- a row chooses an expert at most once, so a step of
+// up to 16 (32) rows needs one (two) of a tile's four, and the kernel fewer registers and more waves.
+//
+// reduce_waves: red [wave][sub][reg][lane]; afterwards wave w holds the four-wave sums of the SUBS accumulator registers
+// w SUBS .. w SUBS + SUBS - 1 (register t of a tile: sub-tile t / 4, row 4 g + t % 4), one per entry of out.
+template <int SUBS>
+DEV void reduce_waves(const f32x4 (&acc)[SUBS], float (&out)[SUBS], float* red, int wave, int lane) {
+#pragma unroll
+  for (int i = 0; i < SUBS; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) red[((wave * SUBS + i) * 4 + j) * 64 + lane] = acc[i][j];
   __syncthreads();
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
+  for (int s = 0; s < SUBS; ++s) {
     float v = 0.f;
 #pragma unroll
-    for (int w = 0; w < 4; ++w) v += red[((w * 4 + wave) * 4 + j) * 64 + lane];
-    acc[0][j] = v;
+    for (int w = 0; w < 4; ++w) v += red[(w * SUBS * 4 + wave * SUBS + s) * 64 + lane];
+    out[s] = v;
   }
   __syncthreads();
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void moe_gate_up_kernel(MoeGroupedParams p) {
+// One wave's share of a workgroup's products over the K axis: au += X . up^T and, with a gate, ag += X . gate^T for the
+// live sub-tiles.  Aligned rows take blocks of 4 AHEAD k-steps, AHEAD per wave in neighbouring pairs (a pair is a whole
+// 128-byte line of every bf16 weight row), and request all of a block's weights before the first product waits for one:
+// a decode step has one live sub-tile, so the weight stream's latency is what these loops are made of.  Rows and columns
+// that do not exist point at valid memory and are dropped by the caller.
+template <typename T, int SUBS, int AHEAD, bool GATED>
+DEV void expert_products(const T* const (&xr)[SUBS], const bool (&xv)[SUBS], const bool (&live)[SUBS], bool vecx,
+                         const T* ur, const T* gr, bool fv, bool vecw, int K, int wave, int g, f32x4 (&ag)[SUBS],
+                         f32x4 (&au)[SUBS]) {
   using F = Frag<T>;
-  __shared__ float red[4 * 4 * 4 * 64];
+  const int steps = vecx && vecw ? K / F::KS : 0;  // whole k-steps on the aligned path
+  for (int s0 = 0; s0 < steps; s0 += 4 * AHEAD) {
+    typename F::V bu[AHEAD], bg[AHEAD];
+    int at[AHEAD];
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      const int st = s0 + (u >> 1) * 8 + 2 * wave + (u & 1);
+      at[u] = st < steps ? st * F::KS + F::PER * g : -1;  // uniform sign over the wave
+      if (at[u] >= 0) {
+        bu[u] = ld_global<typename F::V>(ur + at[u]);
+        if (GATED) bg[u] = ld_global<typename F::V>(gr + at[u]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < SUBS; ++i) {
+      if (!live[i]) continue;  // uniform over the workgroup
+      typename F::V a[AHEAD];
+#pragma unroll
+      for (int u = 0; u < AHEAD; ++u)
+        if (at[u] >= 0) a[u] = ld_global<typename F::V>(xr[i] + at[u]);
+#pragma unroll
+      for (int u = 0; u < AHEAD; ++u)
+        if (at[u] >= 0) {
+          if (GATED) ag[i] = mma(a[u], bg[u], ag[i]);
+          au[i] = mma(a[u], bu[u], au[i]);
+        }
+    }
+  }
+  for (int k0 = (steps + wave) * F::KS; k0 < K; k0 += 4 * F::KS) {  // unaligned rows, or the rest of the K axis
+    const int k = k0 + F::PER * g;
+    const typename F::V bu = load_frag<T>(ur, k, K, fv, vecw);
+    const typename F::V bg = GATED ? load_frag<T>(gr, k, K, fv, vecw) : bu;
+#pragma unroll
+    for (int i = 0; i < SUBS; ++i) {
+      if (!live[i]) continue;
+      const typename F::V a = load_frag<T>(xr[i], k, K, xv[i], vecx);
+      if (GATED) ag[i] = mma(a, bg, ag[i]);
+      au[i] = mma(a, bu, au[i]);
+    }
+  }
+}
+
+template <typename T, int SUBS, bool GATED>
+__global__ __launch_bounds__(256) void moe_gate_up_kernel(MoeGroupedParams p) {
+  __shared__ float red[4 * SUBS * 4 * 64];
   const int t = blockIdx.y;
-  if (t >= *p.num_tiles) return;
   const int e = p.tile_expert[t];
+  if (e < 0) return;  // past the last tile
   const bool sh = e >= p.E;
   const int Fe = sh ? p.Fs : p.F;
   if ((int)blockIdx.x * 16 >= Fe) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
-  const bool gated = p.gate != nullptr;  // uniform: experts without a gate are down(relu(up x)^2)
   const T* up = sh ? reinterpret_cast<const T*>(p.sup) : reinterpret_cast<const T*>(p.up) + (int64_t)e * p.F * p.W;
-  const T* gate = !gated ? up
+  const T* gate = !GATED ? up  // experts without a gate are down(relu(up x)^2)
                          : (sh ? reinterpret_cast<const T*>(p.sgate)
                                : reinterpret_cast<const T*>(p.gate) + (int64_t)e * p.F * p.W);
   const int* ids = p.sorted + t * kMoeRows;
   // an expert's ids fill its tiles from the front: a 16-row sub-tile is empty when its first id is a pad
-  const T* xr[4];
-  bool xv[4], live[4];
+  const T* xr[SUBS];
+  bool xv[SUBS], live[SUBS];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < SUBS; ++i) {
     const int id = ids[16 * i + r];
     live[i] = ids[16 * i] >= 0;
     xv[i] = id >= 0;
@@ -261,51 +441,42 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(MoeGroupedParams p) {
   const T* gr = gate + (int64_t)(fv ? f : 0) * p.W;
   const T* ur = up + (int64_t)(fv ? f : 0) * p.W;
   const bool vec = p.vec_w != 0;
-  f32x4 ag[4], au[4];
+  f32x4 ag[SUBS], au[SUBS];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) ag[i] = au[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = wave * F::KS; k0 < p.W; k0 += 4 * F::KS) {
-    const int k = k0 + F::PER * g;
-    const typename F::V bu = load_frag<T>(ur, k, p.W, fv, vec);
-    const typename F::V bg = gated ? load_frag<T>(gr, k, p.W, fv, vec) : bu;
+  for (int i = 0; i < SUBS; ++i) ag[i] = au[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  expert_products<T, SUBS, 4, GATED>(xr, xv, live, vec, ur, gr, fv, vec, p.W, wave, g, ag, au);
+  float sg[SUBS], su[SUBS];
+  if (GATED) reduce_waves<SUBS>(ag, sg, red, wave, lane);
+  reduce_waves<SUBS>(au, su, red, wave, lane);
+  if (!fv) return;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      if (!live[i]) continue;  // uniform over the workgroup
-      const typename F::V a = load_frag<T>(xr[i], k, p.W, xv[i], vec);
-      if (gated) ag[i] = mma(a, bg, ag[i]);
-      au[i] = mma(a, bu, au[i]);
-    }
-  }
-  if (gated) reduce4(ag, red, wave, lane);
-  reduce4(au, red, wave, lane);
-  if (!fv || !live[wave]) return;
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int id2 = ids[16 * wave + 4 * g + j];
+  for (int s = 0; s < SUBS; ++s) {
+    const int reg = wave * SUBS + s;
+    const int id2 = ids[16 * (reg >> 2) + 4 * g + (reg & 3)];
     if (id2 < 0) continue;
     const float wi = in_weight(p, id2);
-    const float gv = ag[0][j] * wi, uv = au[0][j] * wi;
+    const float gv = GATED ? sg[s] * wi : 0.f, uv = su[s] * wi;
     reinterpret_cast<T*>(p.h)[(int64_t)id2 * p.ldh + f] =
-        (T)(gated ? gv / (1.0f + expf(-gv)) * uv : (uv > 0.0f ? uv * uv : 0.0f));
+        (T)(GATED ? gv / (1.0f + expf(-gv)) * uv : (uv > 0.0f ? uv * uv : 0.0f));
   }
 }
 
-template <typename T>
+template <typename T, int SUBS>
 __global__ __launch_bounds__(256) void moe_down_kernel(MoeGroupedParams p) {
   using F = Frag<T>;
-  __shared__ float red[4 * 4 * 4 * 64];
+  __shared__ float red[4 * SUBS * 4 * 64];
   const int t = blockIdx.y;
-  if (t >= *p.num_tiles) return;
   const int e = p.tile_expert[t];
+  if (e < 0) return;
   const bool sh = e >= p.E;
   const int Fe = sh ? p.Fs : p.F;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
   const T* down = sh ? reinterpret_cast<const T*>(p.sdown) : reinterpret_cast<const T*>(p.down) + (int64_t)e * p.W * p.F;
   const int* ids = p.sorted + t * kMoeRows;
-  const T* hr[4];
-  bool hv[4], live[4];
+  const T* hr[SUBS];
+  bool hv[SUBS], live[SUBS];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < SUBS; ++i) {
     const int id = ids[16 * i + r];
     live[i] = ids[16 * i] >= 0;
     hv[i] = id >= 0;
@@ -315,28 +486,28 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeGroupedParams p) {
   const bool dv = d < p.W;
   const T* dr = down + (int64_t)(dv ? d : 0) * Fe;
   const bool vech = p.vec_h != 0, vecd = p.vec_h != 0 && Fe % F::PER == 0;
-  f32x4 acc[4];
+  f32x4 acc[SUBS];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = wave * F::KS; k0 < Fe; k0 += 4 * F::KS) {
-    const int k = k0 + F::PER * g;
-    const typename F::V b = load_frag<T>(dr, k, Fe, dv, vecd);
+  for (int i = 0; i < SUBS; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  expert_products<T, SUBS, SUBS == 1 ? 8 : 4, false>(hr, hv, live, vech, dr, dr, dv, vecd, Fe, wave, g, acc, acc);
+  float sum[SUBS];
+  reduce_waves<SUBS>(acc, sum, red, wave, lane);
+  if (!dv) return;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      if (!live[i]) continue;
-      acc[i] = mma(load_frag<T>(hr[i], k, Fe, hv[i], vech), b, acc[i]);
-    }
-  }
-  reduce4(acc, red, wave, lane);
-  if (!dv || !live[wave]) return;
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int id2 = ids[16 * wave + 4 * g + j];
+  for (int s = 0; s < SUBS; ++s) {
+    const int reg = wave * SUBS + s;
+    const int id2 = ids[16 * (reg >> 2) + 4 * g + (reg & 3)];
     if (id2 < 0) continue;
     const int row = id2 / p.S, k = id2 % p.S;
-    const float wgt = out_weight(p, row, k);
-    p.o[(int64_t)id2 * p.W + d] = wgt * acc[0][j];
+    p.o[(int64_t)id2 * p.W + d] = out_weight(p, row, k) * sum[s];
   }
+}
+
+template <typename T, int SUBS>
+void launch_expert_gemms(const MoeGroupedParams& p, dim3 g1, dim3 g2, hipStream_t st) {
+  if (p.gate) hipLaunchKernelGGL((moe_gate_up_kernel<T, SUBS, true>), g1, dim3(256), 0, st, p);
+  else hipLaunchKernelGGL((moe_gate_up_kernel<T, SUBS, false>), g1, dim3(256), 0, st, p);
+  hipLaunchKernelGGL((moe_down_kernel<T, SUBS>), g2, dim3(256), 0, st, p);
 }
 
 // Prompt-sized row counts (bf16, widths multiples of 8): the same two GEMMs with both operands staged through LDS.
@@ -501,7 +672,8 @@ extern "C" hipError_t dsse_moe_ffn(const dsse::MoeFfnParams* p, hipStream_t st) 
 extern "C" hipError_t dsse_moe_grouped(const dsse::MoeGroupedParams* p, hipStream_t st) {
   if (p->M <= 0) return hipSuccess;
   const int NE = p->E + (p->S > p->top ? 1 : 0);
-  hipLaunchKernelGGL(dsse::moe_align_kernel, dim3(1), dim3(256), sizeof(int) * (3 * NE + 1), st, *p);
+  if (!p->aligned)
+    hipLaunchKernelGGL(dsse::moe_align_kernel, dim3(1), dim3(256), sizeof(int) * (3 * NE + 1), st, *p);
   const int fmax = p->F > p->Fs ? p->F : p->Fs;
   dim3 g1((fmax + 15) / 16, p->max_tiles), g2((p->W + 15) / 16, p->max_tiles);
   // prompt-sized steps in bf16 with 16-byte-aligned rows: operands staged through LDS
@@ -512,18 +684,31 @@ extern "C" hipError_t dsse_moe_grouped(const dsse::MoeGroupedParams* p, hipStrea
     hipLaunchKernelGGL(dsse::moe_tile_lds_kernel<1>, l2, dim3(256), 0, st, *p);
     return hipGetLastError();
   }
+  const int subs = p->M <= 16 ? 1 : (p->M <= 32 ? 2 : 4);  // rows of one expert: at most M (the shared one has all M)
+#define DSSE_EXPERT_CASE(T)                                                    \
+  if (subs == 1) dsse::launch_expert_gemms<T, 1>(*p, g1, g2, st);              \
+  else if (subs == 2) dsse::launch_expert_gemms<T, 2>(*p, g1, g2, st);         \
+  else dsse::launch_expert_gemms<T, 4>(*p, g1, g2, st);
   if (p->f32) {
-    hipLaunchKernelGGL(dsse::moe_gate_up_kernel<float>, g1, dim3(256), 0, st, *p);
-    hipLaunchKernelGGL(dsse::moe_down_kernel<float>, g2, dim3(256), 0, st, *p);
+    DSSE_EXPERT_CASE(float)
   } else {
-    hipLaunchKernelGGL(dsse::moe_gate_up_kernel<bf16>, g1, dim3(256), 0, st, *p);
-    hipLaunchKernelGGL(dsse::moe_down_kernel<bf16>, g2, dim3(256), 0, st, *p);
+    DSSE_EXPERT_CASE(bf16)
   }
+#undef DSSE_EXPERT_CASE
   return hipGetLastError();
 }
 
 extern "C" hipError_t dsse_moe_topk(const float* z, int M, int E, int top, int* topk_idx, float* topk_w, hipStream_t st) {
   if (M <= 0) return hipSuccess;
   hipLaunchKernelGGL(dsse::moe_topk_kernel, dim3((M + 255) / 256), dim3(256), 0, st, z, M, E, top, topk_idx, topk_w);
+  return hipGetLastError();
+}
+
+extern "C" hipError_t dsse_moe_route_rows(const dsse::MoeRouteRowsParams* p, hipStream_t st) {
+  if (p->M <= 0) return hipSuccess;
+  const int NE = p->E + (p->S > p->top ? 1 : 0);
+  if (p->E > 64 * dsse::kRouteLanes || p->top < 1 || p->top > p->E || p->S < p->top || p->S > p->top + 1)
+    return hipErrorInvalidValue;
+  hipLaunchKernelGGL(dsse::moe_route_rows_kernel, dim3(p->M), dim3(dsse::kRouteThreads), sizeof(int) * (4 * NE + 1), st, *p);
   return hipGetLastError();
 }

@@ -401,7 +401,238 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
   }
 }
 
+// ---------------------------------------------------------------------------------------------------------------------
+// Decode form of the MFMA kernel: one query row per work item, and the heads of ONE key/value group side by side as the
+// 16 columns, so a page of keys and values is read once per group instead of once per head.  The NW waves of a workgroup
+// split the pages (wave, wave + NW, ...) and are merged through LDS.  A decode step has few workgroups and short walks,
+// so the walk is written against latency: a wave reads the ids of its next 64 pages in one load, requests the next
+// page's keys before it needs them (heads up to 128 wide: KB k-steps of both 16-key halves stay in registers), and the
+// values of a page while its scores are being made.  Same key order, masks, bias and epilogue as above.
+template <int NT, int KB, int NW, bool EXT>
+__global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, const bf16* __restrict__ vt, int rel_lds) {
+  extern __shared__ __align__(16) unsigned char smem_raw[];
+  const int D = p.D, V = p.V;
+  const int ldq = D + 8;
+  const int rep = p.H / p.G;
+  const int kvh = blockIdx.y;
+  const int h0 = kvh * rep + blockIdx.z * 16;                       // first head of this column tile
+  const int cols = rep - (int)blockIdx.z * 16 < 16 ? rep - (int)blockIdx.z * 16 : 16;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
+  const int seq = p.work_seq[blockIdx.x], off = p.work_tile[blockIdx.x];
+  const int ql = p.q_len[seq];
+  if (off >= ql) return;  // uniform for the workgroup
+  const int64_t row = p.q_start[seq] + off;
+  const int pos = p.ctx_len[seq] - ql + off;
+  int lo = pos - p.window + 1;
+  lo = lo > 0 ? lo : 0;
+  const int pg_lo = lo / kBS;
+  int kept_pages = 0;
+  if (EXT && p.keep_first > 0) {
+    kept_pages = (p.keep_first + kBS - 1) / kBS;
+    kept_pages = kept_pages < pg_lo ? kept_pages : pg_lo;
+  }
+  const int walk = kept_pages + pos / kBS - pg_lo + 1;
+  const int mine = walk > wave ? (walk - wave + NW - 1) / NW : 0;   // pages of this wave
+  const int* bt = p.block_tables + (int64_t)seq * p.max_blocks;
+  auto page_at = [&](int it) {  // logical page of this wave's it-th step
+    const int pi = wave + it * NW;
+    return pi < kept_pages ? pi : pg_lo + pi - kept_pages;
+  };
+  auto ids_from = [&](int it0) {  // the physical pages of this wave's steps it0 .. it0 + 63, one per lane
+    int b = it0 + lane < mine ? bt[page_at(it0 + lane)] : 0;
+    return (unsigned)b < (unsigned)p.num_blocks ? b : 0;
+  };
+  int blks = ids_from(0);
+  bf16* qs = reinterpret_cast<bf16*>(smem_raw);
+  float* rels = reinterpret_cast<float*>(smem_raw + 16 * ldq * sizeof(bf16));   // [cols][rel_lds]
+  float* mg = rels + cols * rel_lds;                                            // [NW][cols][V + 2]
+  for (int i = threadIdx.x; i < 16 * (D / 4); i += NW * 64) {
+    const int col = i / (D / 4), d = (i - col * (D / 4)) * 4;
+    const f32x4 q4 = col < cols ? *reinterpret_cast<const f32x4*>(p.q + (row * p.H + h0 + col) * D + d)
+                                : f32x4{0.f, 0.f, 0.f, 0.f};
+    bf16x4 v;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = (bf16)q4[j];
+    *reinterpret_cast<bf16x4*>(qs + col * ldq + d) = v;
+  }
+  const bool c_ok = r < cols;
+  const float* relg = nullptr;
+  float rel_far = 0.f;
+  if (EXT && p.rel) {
+    for (int i = threadIdx.x; i < cols * rel_lds; i += NW * 64) {
+      const int col = i / rel_lds;
+      rels[i] = p.rel[(int64_t)(h0 + col) * p.rel_len + i - col * rel_lds];
+    }
+    relg = p.rel + (int64_t)(h0 + (c_ok ? r : 0)) * p.rel_len;
+    rel_far = relg[p.rel_len - 1];
+  }
+  const float* relc = rels + (c_ok ? r : 0) * rel_lds;
+  const bf16* kc = reinterpret_cast<const bf16*>(p.k);
+  const int nks = D / 32;
+  auto key_row = [&](int blk) { return kc + (((int64_t)blk * kBS + r) * p.G + kvh) * D + 8 * g; };
+  bf16x8 ka[KB], kb[KB];  // the current page's keys (k-steps 0 .. KB - 1)
+  auto load_keys = [&](int blk) {
+    const bf16* k0 = key_row(blk);
+    const bf16* k1 = k0 + (int64_t)16 * p.G * D;
+#pragma unroll
+    for (int u = 0; u < KB; ++u)
+      if (u < nks) {
+        ka[u] = ld_global<bf16x8>(k0 + 32 * u);
+        kb[u] = ld_global<bf16x8>(k1 + 32 * u);
+      }
+  };
+  f32x4 O[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n) O[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f;
+  if (mine > 0) load_keys(__builtin_amdgcn_readlane(blks, 0));
+  __syncthreads();
+  for (int it = 0; it < mine; ++it) {
+    const int pg = page_at(it);
+    const int blk = __builtin_amdgcn_readlane(blks, it & 63);
+    const bf16* vrow = vt + (((int64_t)blk * p.G + kvh) * V + r) * kBS + 8 * g;
+    bf16x8 vf[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) vf[n] = ld_global<bf16x8>(vrow + (int64_t)n * 16 * kBS);
+    f32x4 s0 = f32x4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+    for (int u = 0; u < KB; ++u)
+      if (u < nks) {
+        const bf16x8 q8 = *reinterpret_cast<const bf16x8*>(qs + r * ldq + 32 * u + 8 * g);
+        s0 = mfma16x16x32(ka[u], q8, s0);
+        s1 = mfma16x16x32(kb[u], q8, s1);
+      }
+    if (nks > KB) {  // wider heads: the rest of the row, no prefetch
+      const bf16* k0 = key_row(blk);
+      const bf16* k1 = k0 + (int64_t)16 * p.G * D;
+      for (int s = KB; s < nks; ++s) {
+        const bf16x8 q8 = *reinterpret_cast<const bf16x8*>(qs + r * ldq + 32 * s + 8 * g);
+        s0 = mfma16x16x32(ld_global<bf16x8>(k0 + 32 * s), q8, s0);
+        s1 = mfma16x16x32(ld_global<bf16x8>(k1 + 32 * s), q8, s1);
+      }
+    }
+    if (it + 1 < mine) {
+      if (((it + 1) & 63) == 0) blks = ids_from(it + 1);
+      load_keys(__builtin_amdgcn_readlane(blks, (it + 1) & 63));
+    }
+    float sv[8];
+    float mx = -INFINITY;
+    const bool far = EXT && p.rel && pos - (pg * kBS + kBS - 1) >= p.rel_len - 1;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
+      const bool seen = c_ok && key <= pos && (pos - key < p.window || (EXT && key < p.keep_first));
+      float sc = (i < 4 ? s0[i] : s1[i - 4]) * p.scale;
+      if (p.softcap > 0.f) sc = p.softcap * tanh_fast(sc * cap_inv);
+      if (EXT && p.rel) {
+        if (far) {
+          sc += rel_far;
+        } else {
+          int n = pos - key;
+          n = n < 0 ? 0 : (n < p.rel_len ? n : p.rel_len - 1);
+          sc += n < rel_lds ? relc[n] : relg[n];
+        }
+      }
+      sv[i] = seen ? sc : -INFINITY;
+      mx = fmaxf(mx, sv[i]);
+    }
+    mx = rows4_max(mx);
+    const float mn = fmaxf(m, mx);
+    const float corr = mn == -INFINITY ? 1.0f : expf(m - mn);
+    bf16x8 pf;
+    float ps = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const float e = sv[i] == -INFINITY ? 0.0f : expf(sv[i] - mn);
+      ps += e;
+      pf[i] = (bf16)e;
+    }
+    l = l * corr + rows4_sum(ps);
+    m = mn;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      f32x4 o = O[n];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o[i] *= corr;
+      O[n] = mfma16x16x32(vf[n], pf, o);
+    }
+  }
+  const int ldm = V + 2;
+  if (c_ok) {
+    float* my = mg + (wave * cols + r) * ldm;
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) my[16 * n + 4 * g + i] = O[n][i];
+    if (g == 0) {
+      my[V] = m;
+      my[V + 1] = l;
+    }
+  }
+  __syncthreads();
+  const int half = V >> 1;
+  const float2* orp = p.out_rope ? p.out_rope + (int64_t)(pos < p.out_rope_len ? pos : p.out_rope_len - 1) * half : nullptr;
+  for (int idx = threadIdx.x; idx < cols * V; idx += NW * 64) {
+    const int col = idx / V, d = idx - col * V, h = h0 + col;
+    float mm = p.sink ? p.sink[h] : -INFINITY;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) mm = fmaxf(mm, mg[(w * cols + col) * ldm + V]);
+    float den = p.sink ? expf(p.sink[h] - mm) : 0.f, num = 0.f, nump = 0.f;
+    const bool lo_half = d < half;
+    const int dp = orp ? (lo_half ? d + half : d - half) : d;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) {
+      const float* src = mg + (w * cols + col) * ldm;
+      const float f = src[V] == -INFINITY ? 0.f : expf(src[V] - mm);
+      den += src[V + 1] * f;
+      num += src[d] * f;
+      nump += src[dp] * f;
+    }
+    if (orp) {  // back by the row's position
+      const float2 cs = orp[lo_half ? d : dp];
+      num = lo_half ? num * cs.x + nump * cs.y : num * cs.x - nump * cs.y;
+    }
+    float o = den > 0.f ? num / den : 0.f;
+    if (p.gate) o *= 1.0f / (1.0f + expf(-p.gate[row * p.ldg + (p.gate_wide ? h * V + d : h)]));
+    reinterpret_cast<bf16*>(p.out)[(row * p.H + h) * V + d] = (bf16)o;
+  }
+}
+
 constexpr size_t kFlashLds = 64 * 1024;
+
+// LDS of the decode form with nw waves, before the bias entries
+inline size_t decode_lds(const SinkAttnParams& p, int nw) {
+  const int rep = p.H / p.G, cols = rep < 16 ? rep : 16;
+  return 16 * (size_t)(p.D + 8) * sizeof(bf16) + (size_t)nw * cols * (p.V + 2) * sizeof(float);
+}
+
+template <int NT, int NW, bool EXT>
+void launch_decode_waves(int num_work, const SinkAttnParams& p, const bf16* vt, hipStream_t st) {
+  const int rep = p.H / p.G, cols = rep < 16 ? rep : 16;
+  size_t lds = decode_lds(p, NW);
+  int rel_lds = 0;
+  if (EXT && p.rel) {
+    const size_t room = (kFlashLds - lds) / (cols * sizeof(float));
+    const size_t want = p.rel_len < 1024 ? (size_t)p.rel_len : 1024;
+    rel_lds = (int)(want < room ? want : room);
+    lds += cols * rel_lds * sizeof(float);
+  }
+  hipLaunchKernelGGL((sink_decode_kernel<NT, 4, NW, EXT>), dim3(num_work, p.G, (rep + 15) / 16), dim3(NW * 64), lds, st, p,
+                     vt, rel_lds);
+}
+
+template <int NT>
+void launch_decode(int num_work, const SinkAttnParams& p, const bf16* vt, hipStream_t st) {
+  const bool ext = p.rel || p.keep_first > 0;
+  if (decode_lds(p, 8) <= kFlashLds) {
+    if (ext) launch_decode_waves<NT, 8, true>(num_work, p, vt, st);
+    else launch_decode_waves<NT, 8, false>(num_work, p, vt, st);
+  } else {
+    if (ext) launch_decode_waves<NT, 4, true>(num_work, p, vt, st);
+    else launch_decode_waves<NT, 4, false>(num_work, p, vt, st);
+  }
+}
 
 template <int NT, bool EXT>
 void launch_flash_ext(int num_work, const SinkAttnParams& p, const bf16* vt, int split, hipStream_t st) {
@@ -449,6 +680,23 @@ extern "C" hipError_t dsse_sink_flash(int num_work, const dsse::SinkAttnParams* 
     DSSE_FLASH_CASE(7) DSSE_FLASH_CASE(8) DSSE_FLASH_CASE(10) DSSE_FLASH_CASE(12) DSSE_FLASH_CASE(16)
     DSSE_FLASH_CASE(20) DSSE_FLASH_CASE(24) DSSE_FLASH_CASE(32)
 #undef DSSE_FLASH_CASE
+    default: return hipErrorInvalidValue;
+  }
+  return hipGetLastError();
+}
+
+// decode form: work_tile counts single rows; V / 16 as above, LDS for at least four waves
+extern "C" hipError_t dsse_sink_decode(int num_work, const dsse::SinkAttnParams* p, const void* vt, hipStream_t st) {
+  if (num_work <= 0 || p->H <= 0) return hipSuccess;
+  if (p->f32 || p->D % 32 || p->V % 16 || p->V > 512 || p->D > 512 || p->H % p->G) return hipErrorInvalidValue;
+  if (dsse::decode_lds(*p, 4) > dsse::kFlashLds) return hipErrorInvalidValue;
+  const bf16* v = reinterpret_cast<const bf16*>(vt);
+  switch (p->V / 16) {
+#define DSSE_DECODE_CASE(n) case n: dsse::launch_decode<n>(num_work, *p, v, st); break;
+    DSSE_DECODE_CASE(1) DSSE_DECODE_CASE(2) DSSE_DECODE_CASE(3) DSSE_DECODE_CASE(4) DSSE_DECODE_CASE(5)
+    DSSE_DECODE_CASE(6) DSSE_DECODE_CASE(7) DSSE_DECODE_CASE(8) DSSE_DECODE_CASE(10) DSSE_DECODE_CASE(12)
+    DSSE_DECODE_CASE(16) DSSE_DECODE_CASE(20) DSSE_DECODE_CASE(24) DSSE_DECODE_CASE(32)
+#undef DSSE_DECODE_CASE
     default: return hipErrorInvalidValue;
   }
   return hipGetLastError();

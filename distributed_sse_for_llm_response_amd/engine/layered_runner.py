@@ -994,6 +994,9 @@ class LayeredRunner(RunnerBase):
         self.kv = PagedKVCache(kv, self.num_blocks, dev, self.dtype, transposed=flash)
         self.state = MatrixStateCache({}, self.max_batch, dev)  # no layer keeps state beside its pages
         self._pos_table = position_table(self.max_model_len + 1, cfg.width, dev)
+        # mixer and feed-forward read the same rows and write different ones: on a GPU the feed-forward runs on a stream of
+        # its own between the norm and the next add (a fork and a join in the captured graph)
+        self._side_stream = torch.cuda.Stream(dev) if dev.type == "cuda" else None
 
     def _joint_buffers(self, M: int) -> dict:
         """Scratch of a step of M rows, each sized for the widest layer: `big` the fused projection's fp32 output, `qa`
@@ -1017,21 +1020,33 @@ class LayeredRunner(RunnerBase):
             ldh = -(-max(max(f.ff, f.shared_ff) for f in moe) // 8) * 8
             d.update({"tki": torch.zeros(M * slots, **i32), "tkw": torch.zeros(M * slots, **f32),
                       "mo_z": torch.zeros(M * (experts + 1), **f32), "mo_sorted": torch.zeros(tiles * 64, **i32),
-                      "mo_tile": torch.zeros(tiles, **i32), "mo_n": torch.zeros(1, **i32),
+                      "mo_tile": torch.zeros(tiles, **i32), "mo_n": torch.zeros(2, **i32),
                       "mo_h": torch.zeros(M * slots, ldh, **el), "mo_o": torch.zeros(M * slots * W, **f32)})
         return d
 
     def _joint_layers(self, M: int, d: dict, ids, pos, slots, groups: list, trace: list | None) -> None:
         """Every layer over M packed rows.  Between layers ONE add_norm_rows adds both sublayers' outputs to the stream and
-        norms it for the next layer; the last outputs are added before the head's norm."""
+        norms it for the next layer; the last outputs are added before the head's norm.  Both sublayers of a layer run at
+        the same time: the mixer's launches are latency-sized, the experts' stream weights."""
         cfg, w, eps = self.cfg, self.w, self.cfg.eps
         ops.embed_rows(ids, w.embed, d["resid"], None, cfg.embed_scale, pos, self._pos_table)
         pending = (None, 1, None)  # sublayer outputs that are not in the stream yet: (rows, parts per row, second rows)
         for i, (L, Lw) in enumerate(zip(cfg.layers, w.layers)):
             y, nsum, y2 = pending
             ops.add_norm_rows(y, nsum, None, d["resid"], Lw.norm1, eps, d["xb"], d["hn"] if L.mlp is not None else None, y2)
-            self._attention_joint(i, L.mixer, Lw.mix, M, d, slots, groups)
-            pending = (d["y"], 1, None) if L.mlp is None else self._input_weighted_ff(L.mlp, Lw.mlp, M, d) + (d["y"],)
+            pending = (d["y"], 1, None)
+            if L.mlp is None:
+                self._attention_joint(i, L.mixer, Lw.mix, M, d, slots, groups)
+            elif self._side_stream is None:
+                self._attention_joint(i, L.mixer, Lw.mix, M, d, slots, groups)
+                pending = self._input_weighted_ff(L.mlp, Lw.mlp, M, d) + (d["y"],)
+            else:
+                main = torch.cuda.current_stream(self.device)
+                self._side_stream.wait_stream(main)
+                with torch.cuda.stream(self._side_stream):
+                    pending = self._input_weighted_ff(L.mlp, Lw.mlp, M, d) + (d["y"],)
+                self._attention_joint(i, L.mixer, Lw.mix, M, d, slots, groups)
+                main.wait_stream(self._side_stream)
             if trace is not None:
                 ops.add_norm_rows(pending[0], pending[1], None, d["resid"], None, eps, y2=pending[2])
                 pending = (None, 1, None)
@@ -1057,8 +1072,8 @@ class LayeredRunner(RunnerBase):
         for g in groups:
             if vt is not None and g["qt"] > 1:
                 work, form = (g["hs"], g["ht"]), (SINK_ROWS_TILE, vt, False)
-            elif vt is not None and V <= ops.layers.SINK_SPLIT_MAX_V and ops.sink_flash_lds(D, V, True) <= LDS_BYTES:
-                work, form = (g["ws"], g["wt"]), (SINK_ROWS_TILE, vt, True)
+            elif vt is not None and ops.sink_decode_ok(self.dtype, H, G, D, V):
+                work, form = (g["ws"], g["wt"]), (1, vt, False)
             else:
                 work, form = (g["ws"], g["wt"]), (g["qt"], None, False)
             ops.sink_attention(qa, kc, vc, g["bt"], g["qs"], g["ql"], g["ctx"], *work, None, gate, ao, m.window, m.scale,
@@ -1067,18 +1082,23 @@ class LayeredRunner(RunnerBase):
 
     def _input_weighted_ff(self, f, Fw, M: int, d: dict):
         """Router GEMM in true fp32 on the fp32 normed row (the shared expert's gate is its last column) -> the largest
-        sigmoid scores, used as they are -> grouped gated-SiLU experts with the weights on their inputs, the shared expert
+        sigmoid scores, used as they are (decode-sized steps: one launch that also lists the work) -> grouped gated-SiLU experts with the weights on their inputs, the shared expert
         as one more slot with its gate on the output; returns (per-slot outputs [M * S, W] fp32, S)."""
         shared = f.shared_ff > 0
         S, W, E = f.top + shared, self.cfg.width, f.experts + shared
         tki = d["tki"][:M * f.top].view(M, f.top)
         tkw = d["tkw"][:M * S].view(M, S)
         o = d["mo_o"][:M * S * W].view(M * S, W)
-        z = d["mo_z"][:M * E].view(M, E)
-        ops.gemm_rm(d["hn"], Fw.router, z)
-        ops.moe_route(z, None, tki, tkw, 1, 1, 1.0, 2)
-        ops.moe_grouped(d["xb"], tki, tkw, Fw.gate, Fw.up, Fw.down, Fw.sgate, Fw.sup, Fw.sdown, d["mo_sorted"], d["mo_tile"],
-                        d["mo_n"], d["mo_h"], o, True)
+        lists = (d["mo_sorted"], d["mo_tile"], d["mo_n"])
+        one_launch = M <= ops.layers.ROUTE_ROWS_MAX
+        if one_launch:
+            ops.moe_route_rows(d["hn"], Fw.router, tki, tkw, 1.0, *lists)
+        else:
+            z = d["mo_z"][:M * E].view(M, E)
+            ops.gemm_rm(d["hn"], Fw.router, z)
+            ops.moe_route(z, None, tki, tkw, 1, 1, 1.0, 2)
+        ops.moe_grouped(d["xb"], tki, tkw, Fw.gate, Fw.up, Fw.down, Fw.sgate, Fw.sup, Fw.sdown, *lists, d["mo_h"], o, True,
+                        one_launch)
         return o, S
 
     def _remember_last(self, seqs: list, g: dict) -> None:

@@ -132,18 +132,31 @@ def moe_ffn(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, out):
 
 
 def moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, sorted_ids, tile_expert, num_tiles, h, o,
-                weight_input: bool = False):
+                weight_input: bool = False, aligned: bool = False):
     """Grouped form of the routed experts: rows sorted by expert, 16-row MFMA tiles of one expert each.  o [M · S, W]
     (fp32) = weight · expert output per (row, slot), S = top (+ 1: the shared expert's slot); the norm or stream step
     that follows sums them (nsum=S).  gate None: experts without a gate, down(relu(up x)^2).  topk_w may have a
     column more than topk_idx: the shared expert's weight per row (1 without it).  weight_input: a routed expert's weight
-    multiplies its input instead of its output (the shared expert's always its output).  sorted_ids / tile_expert /
-    num_tiles / h are scratch."""
+    multiplies its input instead of its output (the shared expert's always its output).  A row's chosen experts are
+    distinct.  sorted_ids / tile_expert / num_tiles / h are scratch; aligned: the first three are moe_route_rows'."""
     if _hip(x):
         torch.ops.dsse.moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, sorted_ids, tile_expert,
-                                   num_tiles, h, o, weight_input)
+                                   num_tiles, h, o, weight_input, aligned)
     else:
         lref.moe_grouped(x, topk_idx, topk_w, gate, up, down, sgate, sup, sdown, o, weight_input)
+
+
+ROUTE_ROWS_MAX = 64  # steps of up to this many rows make router, choice and work list in one launch
+
+
+def moe_route_rows(x, w, topk_idx, topk_w, scale: float, sorted_ids, tile_expert, num_tiles):
+    """The fp32 router GEMM z = w x, moe_route (kind 2, no groups; topk_w [M, S] with a shared expert's gate as the last
+    row of w and the last column) and moe_grouped's work list in ONE launch, for decode-sized steps.  num_tiles holds two
+    numbers, zeros before the first call."""
+    if _hip(x):
+        torch.ops.dsse.moe_route_rows(x, w, topk_idx, topk_w, scale, sorted_ids, tile_expert, num_tiles)
+    else:
+        lref.moe_route(x.float() @ w.float().t(), None, topk_idx, topk_w, 1, 1, scale, 2)
 
 
 # ---------------------------------------------------------------------------------------------------------------------
@@ -190,9 +203,15 @@ def sink_flash_ok(dtype, dim: int, vdim: int) -> bool:
     return dtype == torch.bfloat16 and dim % 32 == 0 and dim <= 512 and vdim % 16 == 0 and vdim // 16 in SINK_FLASH_TILES
 
 
-def sink_flash_lds(dim: int, vdim: int = 0, split: bool = False) -> int:
-    """LDS bytes of the MFMA form before a distance bias: four waves' query tiles, and the key split's merge area."""
-    return 4 * 16 * ((dim + 8) * 2 + ((vdim + 2) * 4 if split else 0))
+def sink_decode_ok(dtype, heads: int, kv_heads: int, dim: int, vdim: int) -> bool:
+    """Shapes the decode form of sink_attention covers: the MFMA form's, with room in LDS for four waves' sums."""
+    return sink_flash_ok(dtype, dim, vdim) and \
+        16 * (dim + 8) * 2 + 4 * min(16, heads // kv_heads) * (vdim + 2) * 4 <= 64 * 1024
+
+
+def sink_flash_lds(dim: int) -> int:
+    """LDS bytes of the MFMA form before a distance bias: four waves' query tiles."""
+    return 4 * 16 * (dim + 8) * 2
 
 
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile, sink, gate, out,
@@ -202,7 +221,9 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, wor
     heads), scores and weights in fp32; sink [H] adds exp(sink) to each head's denominator, gate [T, H] multiplies the
     head's output by its sigmoid.  `qt` query rows per work item (work_seq, work_tile).  With vt (transposed value
     pages [pages, G, V, 32], sink_flash_ok shapes, qt = 16): the MFMA form; split (V <= 128) lets the four waves of a
-    workgroup share one (tile, head) and split its pages, for decode steps.  softcap > 0: scores
+    workgroup share one (tile, head) and split its pages, for decode steps.  With vt and qt = 1: the decode form
+    (sink_decode_ok shapes), one row per item, the heads of a key/value group side by side, pages split over the waves of
+    a workgroup.  softcap > 0: scores
     softcap * tanh(scale q.k / softcap).  out_rope ([positions, V / 2, 2] (cos, sin), rotate-half pairs over the whole
     value width): each head's weighted sum is turned back by the query row's own position before the gate -- with
     values that were rotated by THEIR positions when cached, a value enters the output rotated by the distance (the

@@ -8,6 +8,7 @@ import pytest
 import torch
 
 from distributed_sse_for_llm_response_amd import ops
+from distributed_sse_for_llm_response_amd.models.surodra import HalfRotarySpec
 from distributed_sse_for_llm_response_amd.ops import layers_reference as lref
 
 pytestmark = pytest.mark.gpu
@@ -162,6 +163,39 @@ def test_attention_mfma_form_with_bias_and_kept_keys(H, G, D, V):
             close(o, o_ref, 2e-2)
 
 
+@pytest.mark.parametrize("H,G,D,V", [(4, 2, 64, 64), (6, 1, 32, 32), (5, 5, 128, 96), (8, 2, 96, 320), (16, 1, 64, 128),
+                                     (40, 2, 160, 16), (2, 1, 512, 128)])
+def test_attention_decode_form(H, G, D, V):
+    """One row per item (also two rows of one sequence), the heads of a group side by side in up to two column tiles, with
+    and without bias, kept keys, sink, cap, output rotation, per-head and per-element gates; a long walk (more than 64
+    pages per wave in the widest case)."""
+    g = torch.Generator().manual_seed(7)
+    ctx, ql = [300, 1, 33, 45, 0, 2400], [1, 1, 1, 2, 0, 1]
+    if H == 6:
+        ctx[5] = 18000
+    bt, pages = _pages(ctx, g)
+    T = sum(ql)
+    q = torch.randn(T, H, D, generator=g)
+    kc = torch.randn(pages, PAGE, G, D, generator=g).bfloat16()
+    vc = torch.randn(pages, PAGE, G, V, generator=g).bfloat16()
+    vt = _transposed(vc)
+    wide = torch.randn(T, H * V + 3, generator=g)
+    sink = torch.randn(H, generator=g)
+    rope = HalfRotarySpec(dims=V, base=50.0).table(310)
+    qs, ws, wt = i32([0, 1, 2, 3, 5, 5]), i32([5, 0, 1, 2, 3, 3, 4]), i32([0, 0, 0, 0, 0, 1, 0])
+    for window, keep, dist, gate, sk, cap, turn in (
+            (10 ** 9, 0, 30, wide[:, 1:1 + H * V], None, 0.0, None), (37, 5, 60, wide[:, :H], sink, 0.0, None),
+            (33, 40, 1, None, None, 3.0, None), (20, 3, 5000, wide[:, 1:1 + H * V], None, 0.0, rope), (1, 1, 2, None, sink, 0.0, None),
+            (64, 0, 0, wide[:, :H], sink, 2.0, rope), (10 ** 9, 0, 0, None, None, 0.0, None)):
+        rel = torch.randn(H, dist, generator=g) * 2 if dist else None
+        o_ref = torch.zeros(T, H, V, dtype=torch.bfloat16)
+        lref.sink_attention(q, kc, vc, bt, qs, i32(ql), i32(ctx), sk, gate, o_ref, window, 0.2, vt, cap, turn, rel, keep)
+        o = torch.zeros(T, H, V, dtype=torch.bfloat16, device=dev())
+        ops.sink_attention(c(q), c(kc), c(vc), c(bt), c(qs), c(i32(ql)), c(i32(ctx)), c(ws), c(wt), c(sk), c(gate), o, window,
+                           0.2, 1, c(vt), False, cap, c(turn), c(rel), keep)
+        close(o, o_ref, 2e-2)
+
+
 @pytest.mark.parametrize("E,top", [(1, 1), (6, 2), (16, 1), (64, 8), (256, 5)])
 def test_sigmoid_routing_with_a_shared_gate(E, top):
     g = torch.Generator().manual_seed(5)
@@ -175,8 +209,41 @@ def test_sigmoid_routing_with_a_shared_gate(E, top):
         close(w, w_ref, 1e-6)
 
 
+@pytest.mark.parametrize("M,W,E,top,shared", [(1, 1, 1, 1, 0), (16, 2048, 16, 2, 1), (64, 333, 70, 4, 1), (5, 1024, 256, 8, 0),
+                                             (33, 64, 3, 3, 1)])
+def test_route_rows_in_one_launch(M, W, E, top, shared):
+    """The one-launch router against the reference's choice, and its work list: every (row, slot) once, under its expert,
+    tiles beyond the last marked; several launches on the same scratch."""
+    g = torch.Generator().manual_seed(8)
+    S, tiles = top + shared, -(-M * (top + shared) // 64) + E + 2
+    w = torch.randn(E + shared, W, generator=g) / math.sqrt(W) * 2
+    srt, til, num = (torch.zeros(n, dtype=torch.int32, device=dev()) for n in (tiles * 64, tiles, 2))
+    for _ in range(3):
+        x = torch.randn(M, W, generator=g)
+        i_ref, w_ref = torch.zeros(M, top, dtype=torch.int32), torch.zeros(M, S)
+        z = x @ w.t()
+        lref.moe_route(z, None, i_ref, w_ref, 1, 1, 1.25, 2)
+        i, wt = torch.zeros(M, top, dtype=torch.int32, device=dev()), torch.zeros(M, S, device=dev())
+        ops.moe_route_rows(c(x), c(w), i, wt, 1.25, srt, til, num)
+        i, wt = i.cpu(), wt.cpu()
+        # rows whose scores come close are decided by rounding: judge the scores, and the indices elsewhere
+        close(wt, w_ref, 1e-5)
+        sc = torch.sigmoid(z[:, :E]).sort(-1, descending=True).values
+        clear = (sc[:, :-1] - sc[:, 1:])[:, :top].amin(-1) > 1e-5 if E > 1 else torch.ones(M, dtype=torch.bool)
+        assert torch.equal(i[clear], i_ref[clear])
+        n = int(num[0])
+        assert int(num[1]) == 0 and bool((til[n:] == -1).all())
+        seen = []
+        for t in range(n):
+            for v in srt[t * 64:(t + 1) * 64].tolist():
+                if v >= 0:
+                    seen.append(v)
+                    assert int(til[t]) == (E if v % S == top else int(i[v // S, v % S]))
+        assert sorted(seen) == list(range(M * S))
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("M,W,F,Fs,E,top", [(3, 48, 24, 40, 5, 2), (19, 33, 7, 0, 4, 1), (300, 128, 72, 136, 6, 2), (200, 64, 64, 32, 3, 3)])
+@pytest.mark.parametrize("M,W,F,Fs,E,top", [(16, 520, 136, 72, 5, 2), (32, 64, 96, 0, 4, 2), (3, 48, 24, 40, 5, 2), (19, 33, 7, 0, 4, 1), (300, 128, 72, 136, 6, 2), (200, 64, 64, 32, 3, 3)])
 def test_expert_weights_on_the_input(dtype, M, W, F, Fs, E, top):
     """Register-direct and LDS-staged expert GEMMs, with and without a shared expert."""
     g = torch.Generator().manual_seed(6)

@@ -185,6 +185,30 @@ DEV float tanh_fast(float x) {
   return (e - 1.0f) / (e + 1.0f);
 }
 
+// The distance biases of a lane's eight keys of a page: keys 0 .. 3 and 16 .. 19 from its first one, which is n0 away from
+// the query.  The branches are uniform: far pages share the last entry, a table that fits its LDS strip needs no memory.
+DEV void bias_entries(float (&bv)[8], bool far, float rel_far, const float* strip, const float* table, int strip_len,
+                      int rel_len, int n0) {
+  if (far) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) bv[i] = rel_far;
+    return;
+  }
+  int at[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int n = n0 - (i < 4 ? i : 12 + i);
+    at[i] = n < 0 ? 0 : (n < rel_len ? n : rel_len - 1);  // negative: a key behind the query, masked by the caller
+  }
+  if (strip_len >= rel_len) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) bv[i] = strip[at[i]];
+  } else {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) bv[i] = at[i] < strip_len ? strip[at[i]] : ld_global<float>(table + at[i]);
+  }
+}
+
 // NT: V / 16 value tiles.  EXT: the kept first keys and the distance bias (its first rel_lds entries per head in LDS, the
 // rest read from memory; pages whose keys are all so far away that they share the last entry look nothing up).
 template <int NT, bool SPLIT, bool EXT>
@@ -250,53 +274,92 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
     kept_pages = kept_pages < pg_lo ? kept_pages : pg_lo;
   }
   const int walk = kept_pages + hi / kBS - pg_lo + 1;
-  for (int pi = SPLIT ? wave : 0; pi < walk; pi += SPLIT ? 4 : 1) {
-    const int pg = pi < kept_pages ? pi : pg_lo + pi - kept_pages;
-    int blk = bt[pg];
-    blk = (unsigned)blk < (unsigned)p.num_blocks ? blk : 0;
-    const bf16* krow0 = kc + (((int64_t)blk * kBS + r) * p.G + kvh) * D + 8 * g;  // key r of the page's first half
-    const bf16* krow1 = krow0 + (int64_t)16 * p.G * D;                              // key 16 + r
-    const bf16* vrow = vt + (((int64_t)blk * p.G + kvh) * V + r) * kBS + 8 * g;   // dim r of value tile 0
-    bf16x8 vf[NT];
+  // Loads run a page ahead: the ids of the wave's next 64 pages come in one load, a page's keys (the first four k-steps)
+  // and -- for values up to 128 wide -- its values are requested while the page before it is in the softmax.
+  constexpr int KB = 4, STEP = SPLIT ? 4 : 1;
+  constexpr bool AHEAD_V = NT <= 8;
+  const int first = SPLIT ? wave : 0;
+  const int mine = walk > first ? (walk - first + STEP - 1) / STEP : 0;
+  auto page_at = [&](int it) {
+    const int pi = first + it * STEP;
+    return pi < kept_pages ? pi : pg_lo + pi - kept_pages;
+  };
+  auto ids_from = [&](int it0) {
+    const int b = it0 + lane < mine ? bt[page_at(it0 + lane)] : 0;
+    return (unsigned)b < (unsigned)p.num_blocks ? b : 0;
+  };
+  auto key_row = [&](int blk) { return kc + (((int64_t)blk * kBS + r) * p.G + kvh) * D + 8 * g; };  // key r, then 16 + r
+  bf16x8 ka[KB], kb[KB], vf[NT];
+  auto load_keys = [&](int blk) {
+    const bf16* k0 = key_row(blk);
+    const bf16* k1 = k0 + (int64_t)16 * p.G * D;
 #pragma unroll
-    for (int n = 0; n < NT; ++n) vf[n] = ld_global<bf16x8>(vrow + (int64_t)n * 16 * kBS);
+    for (int u = 0; u < KB; ++u)
+      if (u < nks) {
+        ka[u] = ld_global<bf16x8>(k0 + 32 * u);
+        kb[u] = ld_global<bf16x8>(k1 + 32 * u);
+      }
+  };
+  auto load_values = [&](int blk, bf16x8(&v)[NT]) {
+    const bf16* vrow = vt + (((int64_t)blk * p.G + kvh) * V + r) * kBS + 8 * g;   // dim r of value tile 0
+#pragma unroll
+    for (int n = 0; n < NT; ++n) v[n] = ld_global<bf16x8>(vrow + (int64_t)n * 16 * kBS);
+  };
+  int blks = ids_from(0);
+  if (mine > 0) {
+    load_keys(__builtin_amdgcn_readlane(blks, 0));
+    if (AHEAD_V) load_values(__builtin_amdgcn_readlane(blks, 0), vf);
+  }
+  for (int it = 0; it < mine; ++it) {
+    const int pg = page_at(it);
+    const int blk = __builtin_amdgcn_readlane(blks, it & 63);
+    if (!AHEAD_V) load_values(blk, vf);
     f32x4 s0 = f32x4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
-    for (int sb = 0; sb < nks; sb += 4) {  // four k-steps of key loads are requested before the first MFMA needs one
-      bf16x8 ka[4], kb[4], qb[4];
+#pragma unroll
+    for (int u = 0; u < KB; ++u)
+      if (u < nks) {
+        const bf16x8 q8 = *reinterpret_cast<const bf16x8*>(qs + r * ldq + 32 * u + 8 * g);
+        s0 = mfma16x16x32(ka[u], q8, s0);
+        s1 = mfma16x16x32(kb[u], q8, s1);
+      }
+    for (int sb = KB; sb < nks; sb += 4) {  // wider heads: four k-steps at a time
+      const bf16* k0 = key_row(blk);
+      const bf16* k1 = k0 + (int64_t)16 * p.G * D;
+      bf16x8 wa[4], wb[4];
 #pragma unroll
       for (int u = 0; u < 4; ++u) {
         const int s = sb + u < nks ? sb + u : nks - 1;
-        ka[u] = ld_global<bf16x8>(krow0 + 32 * s);
-        kb[u] = ld_global<bf16x8>(krow1 + 32 * s);
-        qb[u] = *reinterpret_cast<const bf16x8*>(qs + r * ldq + 32 * s + 8 * g);
+        wa[u] = ld_global<bf16x8>(k0 + 32 * s);
+        wb[u] = ld_global<bf16x8>(k1 + 32 * s);
       }
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
+      for (int u = 0; u < 4; ++u)
         if (sb + u < nks) {
-          s0 = mfma16x16x32(ka[u], qb[u], s0);
-          s1 = mfma16x16x32(kb[u], qb[u], s1);
+          const bf16x8 q8 = *reinterpret_cast<const bf16x8*>(qs + r * ldq + 32 * (sb + u) + 8 * g);
+          s0 = mfma16x16x32(wa[u], q8, s0);
+          s1 = mfma16x16x32(wb[u], q8, s1);
         }
-      }
+    }
+    bf16x8 vn[AHEAD_V ? NT : 1];
+    if (it + 1 < mine) {
+      if (((it + 1) & 63) == 0) blks = ids_from(it + 1);
+      const int nb = __builtin_amdgcn_readlane(blks, (it + 1) & 63);
+      load_keys(nb);
+      if constexpr (AHEAD_V) load_values(nb, vn);
     }
     float sv[8];
     float mx = -INFINITY;
     // uniform: every (row, key) pair of this tile and page is at least rel_len - 1 apart
     const bool far = EXT && p.rel && pos0 + tile * 16 - (pg * kBS + kBS - 1) >= p.rel_len - 1;
+    float bv[8];
+    if (EXT && p.rel) bias_entries(bv, far, rel_far, rels, relg, rel_lds, p.rel_len, c_pos - pg * kBS - 4 * g);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
       const bool seen = c_ok && key <= c_pos && (c_pos - key < p.window || (EXT && key < p.keep_first));
       float sc = (i < 4 ? s0[i] : s1[i - 4]) * p.scale;
       if (p.softcap > 0.f) sc = p.softcap * tanh_fast(sc * cap_inv);
-      if (EXT && p.rel) {
-        if (far) {
-          sc += rel_far;
-        } else {
-          int n = c_pos - key;
-          n = n < 0 ? 0 : (n < p.rel_len ? n : p.rel_len - 1);
-          sc += n < rel_lds ? rels[n] : relg[n];
-        }
-      }
+      if (EXT && p.rel) sc += bv[i];
       sv[i] = seen ? sc : -INFINITY;
       mx = fmaxf(mx, sv[i]);
     }
@@ -319,6 +382,10 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
 #pragma unroll
       for (int i = 0; i < 4; ++i) o[i] *= corr;
       O[n] = mfma16x16x32(vf[n], pf, o);
+    }
+    if constexpr (AHEAD_V) {
+#pragma unroll
+      for (int n = 0; n < NT; ++n) vf[n] = vn[n];
     }
   }
   if (SPLIT) {
@@ -519,21 +586,15 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
     float sv[8];
     float mx = -INFINITY;
     const bool far = EXT && p.rel && pos - (pg * kBS + kBS - 1) >= p.rel_len - 1;
+    float bv[8];
+    if (EXT && p.rel) bias_entries(bv, far, rel_far, relc, relg, rel_lds, p.rel_len, pos - pg * kBS - 4 * g);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
       const bool seen = c_ok && key <= pos && (pos - key < p.window || (EXT && key < p.keep_first));
       float sc = (i < 4 ? s0[i] : s1[i - 4]) * p.scale;
       if (p.softcap > 0.f) sc = p.softcap * tanh_fast(sc * cap_inv);
-      if (EXT && p.rel) {
-        if (far) {
-          sc += rel_far;
-        } else {
-          int n = pos - key;
-          n = n < 0 ? 0 : (n < p.rel_len ? n : p.rel_len - 1);
-          sc += n < rel_lds ? relc[n] : relg[n];
-        }
-      }
+      if (EXT && p.rel) sc += bv[i];
       sv[i] = seen ? sc : -INFINITY;
       mx = fmaxf(mx, sv[i]);
     }

@@ -119,8 +119,9 @@ DEV uint4 philox4x32(uint4 ctr, uint2 key) {
   }
   return ctr;
 }
-// Uniform in (0, 1]: never exactly 0 so -log(-log(u)) is finite.
-DEV float u01(uint32_t x) { return ((float)(x >> 8) + 1.0f) * (1.0f / 16777216.0f); }
+// Uniform inside (0, 1), the midpoints of 2^23 equal steps (each exact in fp32): neither 0 nor 1, so -log(-log(u)) is
+// finite on both sides.
+DEV float u01(uint32_t x) { return ((float)(x >> 9) + 0.5f) * (1.0f / 8388608.0f); }
 
 // ---- checked build (DSSE_KERNEL_CHECKS=1, `_build.py kernels-checked`) -----------------------------
 // Data-dependent indices the host cannot validate without a sync (block-table entries, KV slots, token

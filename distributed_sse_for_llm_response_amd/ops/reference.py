@@ -228,7 +228,7 @@ def philox4x32(c0, c1, c2, c3, k0, k1):
 def gumbel_noise(seed_lo: int, seed_hi: int, position: int, gidx: np.ndarray) -> np.ndarray:
     x, _, _, _ = philox4x32(gidx, np.full_like(gidx, position), np.full_like(gidx, 0x5353), np.zeros_like(gidx),
                             seed_lo, seed_hi)
-    u = ((x >> np.uint64(8)).astype(np.float64) + 1.0) / 16777216.0
+    u = ((x >> np.uint64(9)).astype(np.float64) + 0.5) / 8388608.0  # inside (0, 1): finite noise
     return -np.log(-np.log(u))
 
 

@@ -2,6 +2,7 @@
 import math
 import os
 
+import numpy as np
 import pytest
 import torch
 
@@ -672,6 +673,24 @@ def test_sampler_distribution(gpu):
     counts = torch.bincount(ids.cpu().long(), minlength=V).float()
     expect = torch.softmax(logits / 0.8, 0) * N
     assert ((counts - expect).abs() <= 5 * expect.sqrt() + 5).all(), (counts, expect)
+
+
+def test_sampler_noise_is_finite(gpu):
+    """Draws whose random word is all ones in its upper bits: the noise stays finite there, so a token that leads by 40
+    is picked (and not the token that such a word belongs to)."""
+    V, spots = 32768, [(60, 26594), (557, 15709), (787, 29093)]  # (position, vocabulary index) of such words, seed (0, 0)
+    for pos, i in spots:
+        assert np.isfinite(R.gumbel_noise(0, 0, pos, np.array([i], dtype=np.uint64))).all()
+    B = len(spots)
+    logits = torch.zeros(B, V)
+    logits[:, 3] = 40.0
+    for topp in (1.0, 0.999):  # the chunked path and the filtered one
+        args = (torch.ones(B), torch.zeros(B, dtype=torch.int32), torch.full((B,), topp), torch.zeros(B, 2, dtype=torch.int32),
+                torch.tensor([p for p, _ in spots], dtype=torch.int32))
+        ids, ids_r = torch.zeros(B, dtype=torch.int32, device=gpu), torch.zeros(B, dtype=torch.int32)
+        ops.sample(logits.to(gpu), *(a.to(gpu) for a in args), None, ids)
+        R.sample(logits, *args, None, ids_r)
+        assert ids.tolist() == ids_r.tolist() == [3] * B
 
 
 def test_sampler_tp_candidates(gpu):

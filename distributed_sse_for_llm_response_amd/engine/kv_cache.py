@@ -157,3 +157,22 @@ class ConvTailCache(RecurrentStateCache):
         self.state = {}
         self.tail = {k: torch.zeros(num_slots, taps - 1, c, device=device, dtype=torch.float32)
                      for k, (c, taps) in shapes.items() if taps > 1}
+
+
+class MemoryStateCache(RecurrentStateCache):
+    """Per-sequence state of matrix memories and of short convolutions in front of attention, indexed by the decode slot
+    like RecurrentStateCache, all fp32: per memory run the matrix [slots, H, D, V] and its normaliser with the running
+    maximum behind it [slots, H, D + 1]; per convolved run the last taps - 1 projected rows [slots, taps - 1, C].
+    ``memories`` maps a run's key -> (H, D, V), ``convs`` -> (C, taps)."""
+
+    def __init__(self, memories: dict, convs: dict, num_slots: int, device):
+        self.num_slots = num_slots
+        f32 = dict(device=device, dtype=torch.float32)
+        self.state = {r: torch.zeros(num_slots, h, d, v, **f32) for r, (h, d, v) in memories.items()}
+        self.norm = {r: torch.zeros(num_slots, h, d + 1, **f32) for r, (h, d, _) in memories.items()}
+        self.tail = {r: torch.zeros(num_slots, k - 1, c, **f32) for r, (c, k) in convs.items() if k > 1}
+
+    def move(self, src_idx: torch.Tensor, dst_idx: torch.Tensor) -> None:
+        super().move(src_idx, dst_idx)
+        for t in self.norm.values():
+            t.index_copy_(0, dst_idx, t.index_select(0, src_idx))

@@ -1,9 +1,9 @@
 """Forward passes of configuration-driven designs (models/muderax.py, models/surodra.py, models/dironex.py,
-models/murulorn.py, models/kagorax.py) on the layer-mechanism kernels (ops/layers.py).  Five block styles share the
+models/murulorn.py, models/kagorax.py, models/lobidra.py) on the layer-mechanism kernels (ops/layers.py).  Five block styles share the
 runner: sandwich norms on a sublayer's output (Muderax, described first), pre-norm blocks around matrix-state mixers
 (Surodra, described after it), pre-norm blocks on several residual streams (Dironex), blocks with a norm before and
-after each sublayer plus a per-layer token input (Murulorn) and blocks whose mixer and feed-forward read one norm side by
-side (Kagorax, described last).
+after each sublayer (Murulorn, with a per-layer token input, and Lobidra) and blocks whose mixer and feed-forward read
+one norm side by side (Kagorax, described last).
 
 A step is a set of packed rows -- the B decode slots first (one row each, state on the device as in ModelRunner), then
 the rows of prompt portions -- that walk the layer list once:
@@ -81,6 +81,19 @@ The bracket-norm walk (`_bracket_layers`) also goes over layer runs:
 A decode row's token becomes its slot's previous token inside embed_pair_rows (the captured graph carries it); prompt
 portions bring each row's predecessor with them (PrefillSeq.prev_token for the first row).
 
+Lobidra's layers on the same walk:
+
+    embed_rows              stream = embed[token] * scale
+    moe_table_lists         every table-routed layer's choices and work list in one launch: they depend on the token alone
+    convolved attention     ONE fused GEMM [q | k | g] -> conv_qkv_rows (convolution from the slot's tail, interleaved
+                            rotation, keys and unrotated keys as values into this run's pages) -> sink_attention (sink of
+                            score 0, gate per head) -> output GEMM
+    twin layer              ONE fused GEMM for both halves -> attention: conv_qkv_rows (queries times their position's
+                            factor) -> sink_attention (learned sink, element-wise gate); memory: matrix_memory (gates,
+                            state, read-out, head norm and gate in one launch for decode rows; chunks of 32 tokens on
+                            MFMA for prompt portions); their gated, scaled heads lie side by side -> ONE output GEMM
+    feed-forward            up GEMM -> act_rows (gelu) -> down GEMM; or moe_grouped on the ready work list
+
 The joint walk (`_joint_layers`), one norm per layer:
 
     embed_rows              stream = embed[token] * scale + the position's vector
@@ -97,7 +110,7 @@ The joint walk (`_joint_layers`), one norm per layer:
 The residual stream, norms, scores, router and recurrence are fp32 in both element types; ``dtype=torch.float32`` runs
 the projections in true fp32 as well (the exact mode).  The cache is paged with the engine's block tables and
 allocator (LatentKVCache, PagedKVCache, both at once in MixedKVCache); recurrent layers and input convolutions keep
-their state in the sequence's decode slot (RecurrentStateCache, MatrixStateCache, ConvTailCache), so
+their state in the sequence's decode slot (RecurrentStateCache, MatrixStateCache, ConvTailCache, MemoryStateCache), so
 slots and pages are handed from one sequence to the next with no clearing pass.  The decode step of each batch bucket
 is captured into a graph like ModelRunner's; prompt portions and mixed steps run eagerly.
 """
@@ -109,11 +122,12 @@ import numpy as np
 import torch
 
 from .. import ops
+from ..models.lobidra import MEMORY_EPS
 from ..models.muderax import LRU_DECAY_SCALE
-from ..models.surodra import UNIT_EPS, HalfRotarySpec
+from ..models.surodra import NO_WINDOW, UNIT_EPS, HalfRotarySpec
 from ..parallel.comm import TPComm
-from .kv_cache import (PAGE, ConvTailCache, LatentKVCache, MatrixStateCache, MixedKVCache, PagedKVCache,
-                       RecurrentStateCache)
+from .kv_cache import (PAGE, ConvTailCache, LatentKVCache, MatrixStateCache, MemoryStateCache, MixedKVCache,
+                       PagedKVCache, RecurrentStateCache)
 from .model_runner import RunnerBase, _capture, batch_buckets
 from .weights import LayeredWeights
 
@@ -146,10 +160,14 @@ class LayeredRunner(RunnerBase):
         self.num_blocks = num_blocks
         self.prenorm = getattr(cfg, "family", "") == "surodra"   # pre-norm blocks with matrix-state mixers
         self.multistream = getattr(cfg, "family", "") == "dironex"  # pre-norm blocks on several residual streams
-        self.bracket = getattr(cfg, "family", "") == "murulorn"    # a norm before and after each sublayer, token inputs
+        self.bracket = getattr(cfg, "family", "") in ("murulorn", "lobidra")  # a norm before and after each sublayer
+        self.memory = getattr(cfg, "family", "") == "lobidra"      # ... with matrix memories and table-routed experts
+        self.pair = self.bracket and not self.memory               # ... with token inputs and an embedding of token pairs
         self.joint = getattr(cfg, "family", "") == "kagorax"       # one norm feeds the mixer and the feed-forward
         if self.joint:
             self._setup_joint()
+        elif self.memory:
+            self._setup_memory()
         elif self.bracket:
             self._setup_bracket()
         elif self.multistream:
@@ -211,7 +229,7 @@ class LayeredRunner(RunnerBase):
             d.update(self._joint_buffers(M))
             return d
         if self.bracket:
-            d.update(self._bracket_buffers(M))
+            d.update(self._memory_buffers(M) if self.memory else self._bracket_buffers(M))
             return d
         if self.multistream:
             d.update(self._stream_buffers(M))
@@ -842,13 +860,17 @@ class LayeredRunner(RunnerBase):
 
         cfg, w, eps = self.cfg, self.w, self.cfg.eps
         W = cfg.width
-        bg = cfg.bigram
-        prev_rows, prev_out, keep = prev if prev is not None else (None, None, None)
-        if bg is not None and prev_rows is None:
-            raise ValueError(f"{cfg.name}: the embedding reads each row's previous token")
-        cat = d["cat"]
-        ops.embed_pair_rows(ids, prev_rows, pos, w.embed, w.bigram, bg.mul_prev if bg else 0, bg.mul_cur if bg else 0,
-                            bg.buckets if bg else 1, d["resid"], cat[:, W:] if cat is not None else None, prev_out, keep)
+        cat = d.get("cat")
+        if self.memory:
+            ops.embed_rows(ids, w.embed, d["resid"], None, cfg.embed_scale)
+            self._expert_lists(ids, M, d)
+        else:
+            bg = cfg.bigram
+            prev_rows, prev_out, keep = prev if prev is not None else (None, None, None)
+            if bg is not None and prev_rows is None:
+                raise ValueError(f"{cfg.name}: the embedding reads each row's previous token")
+            ops.embed_pair_rows(ids, prev_rows, pos, w.embed, w.bigram, bg.mul_prev if bg else 0, bg.mul_cur if bg else 0,
+                                bg.buckets if bg else 1, d["resid"], cat[:, W:] if cat is not None else None, prev_out, keep)
         pending = (None, 1, None)
         ready = False  # the next sublayer's input (xb, or the stream's half of cat) is already written
         fused_side = cfg.side_dim > 0 and ops.token_side_fits(M, W, cfg.side_dim)
@@ -869,6 +891,8 @@ class LayeredRunner(RunnerBase):
                 ops.add_norm_rows(*pending, d["resid"], Lw.norm2, eps, d["xb"], d["hn"] if routed else None)
                 if routed:
                     pending = self._softmax_routed_ff(L.mlp, Lw.mlp, M, d) + (Lw.norm2b,)
+                elif self.memory:
+                    pending = self._memory_ff(run.layer, L.mlp, Lw.mlp, M, d) + (Lw.norm2b,)
                 else:
                     self._relu2_ff(L.mlp, Lw.mlp, M, d)
                     pending = (d["y"], 1, Lw.norm2b)
@@ -980,6 +1004,154 @@ class LayeredRunner(RunnerBase):
         ops.moe_grouped(d["xb"], tki, tkw, None, Fw.up, Fw.down, None, None, None, d["mo_sorted"], d["mo_tile"],
                         d["mo_n"], d["mo_h"], o)
         return o, f.top
+
+    # ------------------------------------------------------------------ convolved attention, matrix memories, table routing
+    def _setup_memory(self) -> None:
+        """Caches and state keyed by layer RUN (a layer that uses another one's tensors is a run of its own): keys and
+        values of every run's attention, convolution tails of the convolved runs, matrix state of the memories; and the
+        tables that depend on the position (rotations, query factors)."""
+        cfg, dev = self.cfg, self.device
+        self.runs = cfg.runs()
+        kv, mem, convs, self._rope, self._temp = {}, {}, {}, {}, {}
+        for r in self.runs:
+            L, m = cfg.layers[r.layer], cfg.layers[r.layer].mixer
+            if L.kind == "conv_attention":
+                kv[r.index] = (m.kv_heads, m.dim, m.dim)
+                convs[r.index] = ((m.heads + m.kv_heads) * m.dim, m.conv)
+                if m.rot is not None and m.rot not in self._rope:
+                    self._rope[m.rot] = m.rot.table(self.max_model_len + 1, dev)
+            else:
+                a = m.left
+                kv[r.index] = (a.kv_heads, a.dim, a.vdim)
+                mem[r.index] = (m.right.heads, m.right.dim, m.right.vdim)
+                if a.temp is not None and a.temp not in self._temp:
+                    self._temp[a.temp] = a.temp.table(self.max_model_len + 1, dev)
+        flash = [r for r, (_, dm, v) in kv.items() if ops.sink_flash_ok(self.dtype, dm, v) and
+                 ops.sink_flash_lds(dm) <= LDS_BYTES]
+        self.kv = PagedKVCache(kv, self.num_blocks, dev, self.dtype, transposed=flash)
+        self.state = MemoryStateCache(mem, convs, self.max_batch, dev)
+        self._moe_layers = [i for i, L in enumerate(cfg.layers) if hasattr(L.mlp, "experts") and L.weights_of == i]
+
+    def _memory_buffers(self, M: int) -> dict:
+        """Scratch of a step of M rows, each sized for the widest layer: `big` the fused projection's fp32 output, `qa`
+        the attention's queries, `ao` a mixer's gated heads in the element type (both halves of a twin layer side by
+        side), `mm` the matrix memory's work area (prompt-sized steps), `up` / `h` the dense feed-forward's hidden row,
+        and the experts' lists: one set per table-routed layer, all made when the step starts."""
+        cfg, dev = self.cfg, self.device
+        f32 = dict(device=dev, dtype=torch.float32)
+        el = dict(device=dev, dtype=self.dtype)
+        i32 = dict(device=dev, dtype=torch.int32)
+        W = cfg.width
+        big = max(Lw.mix.n_big for Lw in self.w.layers)
+        qa = ao = mm = ff = 1
+        for i, L in enumerate(cfg.layers):
+            m = L.mixer
+            a = m if L.kind == "conv_attention" else m.left
+            qa, ao = max(qa, a.heads * a.dim), max(ao, a.heads * a.vdim)
+            if L.kind == "twin":
+                ao = max(ao, -(-(a.heads * a.vdim + m.right.heads * m.right.vdim) // 8) * 8)
+                mm = max(mm, ops.memory_work_floats(M, m.right.heads, m.right.vdim))
+            if L.mlp is not None and not hasattr(L.mlp, "experts"):
+                ff = max(ff, L.mlp.ff)
+        d = {"big": torch.zeros(M * big, **f32), "qa": torch.zeros(M * qa, **f32), "ao": torch.zeros(M * ao, **el),
+             "mm": torch.zeros(mm, **f32), "up": torch.zeros(M * ff, **f32), "h": torch.zeros(M * ff, **el)}
+        moe = [cfg.layers[i].mlp for i in self._moe_layers]
+        if moe:
+            slots = [f.top + (f.shared_ff > 0) for f in moe]
+            tiles = [-(-M * S // 64) + f.experts + 2 for f, S in zip(moe, slots)]
+            ldh = -(-max(max(f.ff, f.shared_ff) for f in moe) // 8) * 8
+            d.update({"tki": [torch.zeros(M * f.top, **i32) for f in moe],
+                      "tkw": {f.top: torch.full((M * f.top,), 1.0 / f.top, **f32) for f in moe},
+                      "mo_sorted": [torch.zeros(t * 64, **i32) for t in tiles],
+                      "mo_tile": [torch.zeros(t, **i32) for t in tiles], "mo_n": [torch.zeros(1, **i32) for _ in moe],
+                      "mo_h": torch.zeros(M * max(slots), ldh, **el), "mo_o": torch.zeros(M * max(slots) * W, **f32)})
+        return d
+
+    def _expert_lists(self, ids, M: int, d: dict) -> None:
+        """Choices and work lists of all table-routed layers of the step."""
+        own = self._moe_layers
+        if own:
+            fs, tables = [self.cfg.layers[i].mlp for i in own], [self.w.layers[i].mlp.table for i in own]
+            tki = [t[:M * f.top].view(M, f.top) for t, f in zip(d["tki"], fs)]
+            ops.moe_table_lists(ids, tables, [f.experts for f in fs], [f.shared_ff > 0 for f in fs], tki, d["mo_sorted"],
+                                d["mo_tile"], d["mo_n"])
+
+    def _memory_ff(self, layer: int, f, Fw, M: int, d: dict):
+        """Dense: up GEMM (fp32) -> gelu -> down GEMM.  Experts: grouped gated-SiLU experts on the work list that the
+        step's start made, the shared expert as one more slot of every row.  Returns (output rows, parts per row)."""
+        if not hasattr(f, "experts"):
+            up, h = d["up"][:M * f.ff].view(M, f.ff), d["h"][:M * f.ff].view(M, f.ff)
+            self._lin(d["xb"], Fw.up, Fw.up_t, up)
+            ops.act_rows(up, h, 3)
+            self._lin(h, Fw.down, Fw.down_t, d["y"])
+            return d["y"], 1
+        n = self._moe_layers.index(layer)
+        S, W = f.top + (f.shared_ff > 0), self.cfg.width
+        tki, tkw = d["tki"][n][:M * f.top].view(M, f.top), d["tkw"][f.top][:M * f.top].view(M, f.top)
+        o = d["mo_o"][:M * S * W].view(M * S, W)
+        ops.moe_grouped(d["xb"], tki, tkw, Fw.gate, Fw.up, Fw.down, Fw.sgate, Fw.sup, Fw.sdown, d["mo_sorted"][n],
+                        d["mo_tile"][n], d["mo_n"][n], d["mo_h"], o, False, True)
+        return o, S
+
+    def _sink_rows(self, ri: int, a, qa, sink, gate, out, groups: list, out_scale: float = 1.0) -> None:
+        """Causal sink attention of every sequence group over this run's pages: the MFMA form for prompt portions, its
+        decode form for decode rows, the row form for head widths that neither covers."""
+        kc, vc, vt = self.kv.k[ri], self.kv.v[ri], self.kv.vt.get(ri)
+        for g in groups:
+            if vt is not None and g["qt"] > 1:
+                work, form = (g["hs"], g["ht"]), (SINK_ROWS_TILE, vt, False)
+            elif vt is not None and ops.sink_decode_ok(self.dtype, a.heads, a.kv_heads, a.dim, a.vdim):
+                work, form = (g["ws"], g["wt"]), (1, vt, False)
+            else:
+                work, form = (g["ws"], g["wt"]), (g["qt"], None, False)
+            ops.sink_attention(qa, kc, vc, g["bt"], g["qs"], g["ql"], g["ctx"], *work, sink, gate, out, NO_WINDOW, a.scale,
+                               *form, out_scale=out_scale)
+
+    def _qkv_rows(self, ri: int, a, big, taps, vdim: int, rope, temp, slots, qa, groups: list) -> None:
+        """q to a buffer, k and v into this run's pages, per sequence group (prompt portions in tiles of rows)."""
+        for g in groups:
+            ws, wt, qt = (g["ws"], g["wt"], 1) if g["qt"] == 1 else (g["hs"], g["ht"], SINK_ROWS_TILE)
+            ops.conv_qkv_rows(big, taps, self.state.tail.get(ri), g["qs"], g["ql"], g["ctx"], g["ss"], ws, wt, qt, a.heads,
+                              a.kv_heads, a.dim, vdim, rope, temp, slots, qa, self.kv.k[ri], self.kv.v[ri],
+                              self.kv.vt.get(ri))
+
+    def _conv_attention_bracket(self, ri: int, m, Lw, M: int, d: dict, pos, slots, groups: list) -> None:
+        """Attention whose q and k pass a convolution over time and whose values are the keys before their rotation."""
+        H, G, D = m.heads, m.kv_heads, m.dim
+        big = d["big"][:M * Lw.n_big].view(M, Lw.n_big)
+        self._lin(d["xb"], Lw.big, Lw.big_t, big)
+        qa = d["qa"][:M * H * D].view(M, H, D)
+        self._qkv_rows(ri, m, big, Lw.conv, 0, self._rope.get(m.rot), None, slots, qa, groups)
+        ao = d["ao"][:M * H * D].view(M, H, D)
+        self._sink_rows(ri, m, qa, Lw.sink, big[:, (H + G) * D:(H + G) * D + H], ao, groups)
+        self._lin(ao.view(M, H * D), Lw.o, Lw.o_t, d["y"])
+
+    def _twin_bracket(self, ri: int, m, Lw, M: int, d: dict, pos, slots, groups: list) -> None:
+        """Attention and matrix memory on the same rows; their gated heads, times the layer's two scales, are the two
+        column ranges of one row, and one output projection sums both halves."""
+        a, r = m.left, m.right
+        H, G, D, V = a.heads, a.kv_heads, a.dim, a.vdim
+        Hr, Dr, Vr = r.heads, r.dim, r.vdim
+        big = d["big"][:M * Lw.n_big].view(M, Lw.n_big)
+        self._lin(d["xb"], Lw.big, Lw.big_t, big)
+        K = -(-(H * V + Hr * Vr) // 8) * 8
+        ao = d["ao"][:M * K].view(M, K)
+        if K > H * V + Hr * Vr:
+            ao[:, H * V + Hr * Vr:].zero_()
+        qa = d["qa"][:M * H * D].view(M, H, D)
+        c = (H + G) * D + G * V
+        self._qkv_rows(ri, a, big, None, V, None, self._temp.get(a.temp), slots, qa, groups)
+        self._sink_rows(ri, a, qa, Lw.sink, big[:, c:c + H * V], ao[:, :H * V].unflatten(1, (H, V)), groups, m.left_scale)
+        c += H * V
+        q, k = self._cols(big, c, Hr, Dr), self._cols(big, c + Hr * Dr, Hr, Dr)
+        c += 2 * Hr * Dr
+        v, gate, zg = self._cols(big, c, Hr, Vr), big[:, c + Hr * Vr:c + 2 * Hr * Vr], big[:, c + 2 * Hr * Vr:]
+        for g in groups:
+            chunked = g["qt"] > 1 and self.device.type == "cuda" and ops.memory_chunk_ok(self.dtype, Dr, Vr)
+            ops.matrix_memory(q, k, v, zg[:, :2 * Hr], Lw.gate_b, r.gate_cap, self.state.state[ri], self.state.norm[ri],
+                              g["qs"], g["ql"], g["ctx"], g["ss"], gate, Lw.norm, self.cfg.eps, MEMORY_EPS, Dr ** -0.5,
+                              m.right_scale, ao[:, H * V:H * V + Hr * Vr], d["mm"] if chunked else None)
+        self._lin(ao, Lw.o, Lw.o_t, d["y"])
 
     # ------------------------------------------------------------------ mixer and feed-forward side by side
     def _setup_joint(self) -> None:
@@ -1103,7 +1275,7 @@ class LayeredRunner(RunnerBase):
 
     def _remember_last(self, seqs: list, g: dict) -> None:
         """After prompt portions: every portion's last token becomes its slot's previous token."""
-        if not self.bracket:
+        if not self.pair:
             return
         self.prev_ids.index_copy_(0, g["ss"].long(), g["last"])
         for s in seqs:
@@ -1123,7 +1295,7 @@ class LayeredRunner(RunnerBase):
                         self.q_len[r], self.kv.num_blocks)
         rows = ("resid", "xb", "y", "y2", "streams", "hn", "hc", "cat")
         d = {k: (v[:B] if k in rows and v is not None else v) for k, v in self._dec.items()}
-        prev = (self.prev_ids[r], self.prev_ids[r], self.q_len[r]) if self.bracket else None
+        prev = (self.prev_ids[r], self.prev_ids[r], self.q_len[r]) if self.pair else None
         self._layers(B, d, self.ids[r], self.positions[r], self.slots[r], [self._decode_group(B)], prev=prev)
         self._head(d["resid"], self._dec["xb"][:B], self.logits[r])
         self._sample_commit(B)
@@ -1162,7 +1334,7 @@ class LayeredRunner(RunnerBase):
         if self.device.type == "cuda":
             idx = idx.pin_memory().to(self.device, non_blocking=True)
         self.state.move(idx[0], idx[1])
-        if self.bracket:
+        if self.pair:
             self.prev_ids.index_copy_(0, idx[1], self.prev_ids.index_select(0, idx[0]))
             moved = {b: self._host_prev.get(a) for a, b in zip(src, dst)}
             self._host_prev.update({b: t for b, t in moved.items() if t is not None})
@@ -1185,7 +1357,7 @@ class LayeredRunner(RunnerBase):
             p = s.start_pos + np.arange(m, dtype=np.int64)
             table = np.asarray(s.block_table, dtype=np.int64)
             ids_l.append(np.asarray(s.tokens, dtype=np.int64))
-            if self.bracket:  # each row's previous token: the caller's (or the slot's remembered one), then the portion's own
+            if self.pair:  # each row's previous token: the caller's (or the slot's remembered one), then the portion's own
                 first = -1
                 if s.start_pos > 0:
                     first = s.prev_token if s.prev_token >= 0 else self._host_prev.get(s.slot, -1)
@@ -1218,7 +1390,7 @@ class LayeredRunner(RunnerBase):
             meta = meta.pin_memory().to(self.device, non_blocking=True)
             bt = bt.pin_memory().to(self.device, non_blocking=True)
         d, o = {}, 0
-        for name, k in (("ids", T), ("pos", T), ("slots", T), ("prev", T if self.bracket else 0), ("qs", n), ("ql", n),
+        for name, k in (("ids", T), ("pos", T), ("slots", T), ("prev", T if self.pair else 0), ("qs", n), ("ql", n),
                         ("ctx", n), ("ss", n), ("ws", len(ws)), ("wt", len(ws)), ("fs", len(fs)), ("ft", len(fs)),
                         ("hs", len(hs)), ("ht", len(hs)), ("last", len(last))):
             d[name], o = meta[o:o + k], o + k
@@ -1259,7 +1431,7 @@ class LayeredRunner(RunnerBase):
         pos = torch.cat([self.positions[r], g["pos"]])
         slots = torch.cat([self.slots[r], g["slots"]])
         d = self._buffers(M)
-        prev = (torch.cat([self.prev_ids[r], g["prev"]]), self.prev_ids[r], self.q_len[r]) if self.bracket else None
+        prev = (torch.cat([self.prev_ids[r], g["prev"]]), self.prev_ids[r], self.q_len[r]) if self.pair else None
         self._layers(M, d, ids, pos, slots, [self._decode_group(B), g], prev=prev)
         self._remember_last(seqs, g)
         self._lm_head(d["resid"][r], self.logits[r])

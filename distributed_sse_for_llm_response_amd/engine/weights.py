@@ -950,3 +950,135 @@ def load_kagorax_dir(cfg, path: str, device="cpu", dtype=torch.bfloat16) -> Laye
     for f in sorted(Path(path).glob("*.safetensors")):
         tensors.update(load_file(str(f)))
     return convert_kagorax(cfg, tensors, device=device, dtype=dtype)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Designs with convolved attention, attention beside a matrix memory, and experts chosen by token id (models/lobidra.py).
+# Projections of a mixer that read the same input are ONE weight; the two halves of a parallel layer also share their
+# output projection: their gated heads lie side by side in one row, so one product sums both.  Gains, convolution taps,
+# sinks and the recurrence's biases are fp32 in both element types.
+@dataclass
+class ConvAttentionWeights:
+    big: torch.Tensor        # rows [q (H D) | k (G D) | g (H) | zero rows] x W
+    n_big: int
+    conv: torch.Tensor       # [(H + G) D, taps] fp32, or None
+    sink: torch.Tensor       # [H] fp32 zeros: the constant sink's logit
+    o: torch.Tensor          # [W, H D]
+    big_t: torch.Tensor = None
+    o_t: torch.Tensor = None
+
+
+@dataclass
+class TwinWeights:
+    big: torch.Tensor        # rows [q | k | v | g of the attention | q | k | v | g | i | f of the memory | zero rows] x W
+    n_big: int
+    sink: torch.Tensor       # [H] fp32
+    gate_b: torch.Tensor     # [2 Hr] fp32: biases of the memory's input and forget gates
+    norm: torch.Tensor       # [Hr Vr] fp32
+    o: torch.Tensor          # [W, H V + Hr Vr (+ zero columns)]
+    big_t: torch.Tensor = None
+    o_t: torch.Tensor = None
+
+
+@dataclass
+class DenseGeluWeights:
+    up: torch.Tensor         # [F, W]
+    down: torch.Tensor       # [W, F]
+    up_t: torch.Tensor = None
+    down_t: torch.Tensor = None
+
+
+@dataclass
+class TableMoeWeights:
+    table: torch.Tensor      # [vocab, top] int32: every token id's experts
+    gate: torch.Tensor       # [E, F, W]
+    up: torch.Tensor         # [E, F, W]
+    down: torch.Tensor       # [E, W, F]
+    sgate: torch.Tensor = None   # shared expert [Fs, W] (None: the design has none)
+    sup: torch.Tensor = None
+    sdown: torch.Tensor = None   # [W, Fs]
+
+
+@torch.no_grad()
+def convert_lobidra(cfg, tensors: dict, device="cpu", dtype=torch.bfloat16) -> LayeredWeights:
+    """Checkpoint tensors {name: tensor} (models/lobidra.py tensor_shapes) -> the engine's grouped layout in `dtype`."""
+    from ..models.lobidra import DenseGeluSpec, tensor_shapes
+
+    for name, shape in tensor_shapes(cfg).items():
+        if name not in tensors:
+            raise KeyError(f"checkpoint lacks tensor {name!r}")
+        if tuple(tensors[name].shape) != tuple(shape):
+            raise ValueError(f"tensor {name!r} has shape {tuple(tensors[name].shape)}, the configuration says {shape}")
+
+    def t(name):
+        return tensors[name].to(device=device, dtype=dtype).contiguous()
+
+    def f(name):
+        return tensors[name].to(device=device, dtype=torch.float32).contiguous()
+
+    def gain(name):
+        return (1.0 + tensors[name].to(device=device, dtype=torch.float32)).contiguous()
+
+    def pad(w, dim: int, to: int):
+        """Zero rows (columns) up to a multiple of `to`."""
+        n = -w.shape[dim] % to
+        if n:
+            shape = list(w.shape)
+            shape[dim] = n
+            w = torch.cat([w, w.new_zeros(shape)], dim=dim)
+        return w.contiguous()
+
+    def cat(*parts):
+        w = torch.cat(parts, dim=0)
+        return pad(w, 0, 128 if w.shape[0] >= TILED_MIN else 8)
+
+    own = {}
+    for i, L in enumerate(cfg.layers):
+        if L.weights_of != i:
+            continue
+        p, m, fs = f"l{i}.", L.mixer, L.mlp
+        if L.kind == "conv_attention":
+            big = cat(*(t(f"{p}mix.{n}") for n in ("q", "k", "g")))
+            conv = torch.cat([f(p + "mix.q.conv"), f(p + "mix.k.conv")]).contiguous() if m.conv > 0 else None
+            mix = ConvAttentionWeights(big=big, n_big=big.shape[0], conv=conv,
+                                       sink=torch.zeros(m.heads, device=device), o=t(p + "mix.o"))
+        else:
+            a, r = p + "mix.left.", p + "mix.right."
+            big = cat(*(t(a + n) for n in ("q", "k", "v", "g")), *(t(r + n) for n in ("q", "k", "v", "g", "i", "f")))
+            mix = TwinWeights(big=big, n_big=big.shape[0], sink=f(a + "sink"),
+                              gate_b=torch.cat([f(r + "i.b"), f(r + "f.b")]).contiguous(), norm=f(r + "norm"),
+                              o=pad(torch.cat([t(a + "o"), t(r + "o")], dim=1), 1, 8))
+        _tile_fields(mix, ("big", "o"))
+        layer = BracketLayer(norm1=gain(p + "norm1"), norm1b=gain(p + "norm1b"), mix=mix)
+        if fs is not None:
+            layer.norm2, layer.norm2b = gain(p + "norm2"), gain(p + "norm2b")
+        if isinstance(fs, DenseGeluSpec):
+            layer.mlp = DenseGeluWeights(up=t(p + "mlp.up"), down=t(p + "mlp.down"))
+            _tile_fields(layer.mlp, ("up", "down"))
+        elif fs is not None:
+            table = tensors[p + "mlp.table"].to(torch.int32)
+            if int(table.min()) < 0 or int(table.max()) >= fs.experts:
+                raise ValueError(f"layer {i}: the expert table names experts outside 0..{fs.experts - 1}")
+            stack = lambda leaf: torch.stack([t(f"{p}mlp.e{e}.{leaf}") for e in range(fs.experts)]).contiguous()  # noqa: E731
+            layer.mlp = TableMoeWeights(table=table.to(device).contiguous(), gate=stack("gate"), up=stack("up"),
+                                        down=stack("down"))
+            if fs.shared_ff:
+                layer.mlp.sgate, layer.mlp.sup, layer.mlp.sdown = (t(f"{p}mlp.shared.{leaf}")
+                                                                   for leaf in ("gate", "up", "down"))
+        own[i] = layer
+    out = LayeredWeights(cfg=cfg, embed=t("embed"), layers=[own[L.weights_of] for L in cfg.layers],
+                         final_norm=gain("final.norm"), head=t("head"), dtype=dtype)
+    _tile_fields(out, ("head",))
+    return out
+
+
+def load_lobidra_dir(cfg, path: str, device="cpu", dtype=torch.bfloat16) -> LayeredWeights:
+    """``*.safetensors`` of a checkpoint directory -> the engine's layout (the loader executes nothing from them)."""
+    from pathlib import Path
+
+    from safetensors.torch import load_file
+
+    tensors = {}
+    for f in sorted(Path(path).glob("*.safetensors")):
+        tensors.update(load_file(str(f)))
+    return convert_lobidra(cfg, tensors, device=device, dtype=dtype)

@@ -216,7 +216,7 @@ def sink_flash_lds(dim: int) -> int:
 
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile, sink, gate, out,
                    window: int, scale: float, qt: int, vt=None, split: bool = False, softcap: float = 0.0, out_rope=None,
-                   rel=None, keep_first: int = 0):
+                   rel=None, keep_first: int = 0, out_scale: float = 1.0):
     """Causal softmax attention of q [T, H, D] over paged keys [pages, 32, G, D] and values [pages, 32, G, V] (grouped
     heads), scores and weights in fp32; sink [H] adds exp(sink) to each head's denominator, gate [T, H] multiplies the
     head's output by its sigmoid.  `qt` query rows per work item (work_seq, work_tile).  With vt (transposed value
@@ -229,13 +229,15 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, wor
     values that were rotated by THEIR positions when cached, a value enters the output rotated by the distance (the
     MFMA form then needs V % 32 == 0).  rel [H, N] (fp32): the entry of the key's distance to the query (the last one for
     distances from N - 1 on) is added to the score.  keep_first: the sequence's first keep_first keys stay visible when the
-    window has passed them.  A gate of H * V columns multiplies the heads element by element."""
+    window has passed them.  A gate of H * V columns multiplies the heads element by element.  out (rows may be a column
+    slice of a wider buffer) is multiplied by out_scale before it is rounded."""
     if _hip(q):
         torch.ops.dsse.sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile,
-                                      sink, gate, out, window, scale, qt, vt, split, softcap, out_rope, rel, keep_first)
+                                      sink, gate, out, window, scale, qt, vt, split, softcap, out_rope, rel, keep_first,
+                                      out_scale)
     else:
         lref.sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sink, gate, out, window, scale, vt,
-                            softcap, out_rope, rel, keep_first)
+                            softcap, out_rope, rel, keep_first, out_scale)
 
 
 def gate_math(x, kind: int, p1=None, p2=None, c: float = 1.0):
@@ -352,7 +354,7 @@ def stream_mix(y, nsum: int, mult: float, streams, ids=None, embed=None, embed_s
 def act_rows(x, out, kind: int, params=None, gate=None):
     """out [M, F] (fp32 or the element type) = act(x) * sigmoid(gate) for fp32 x and gate (column slices are fine; gate
     may be None).  kind 0: identity; 1: xIELU, a_p z^2 + z / 2 for z > 0 else a_n (e^z - 1 - z) + z / 2 with
-    params = fp32 (a_p, a_n); 2: relu(z)^2."""
+    params = fp32 (a_p, a_n); 2: relu(z)^2; 3: gelu (tanh form)."""
     if _hip(x):
         torch.ops.dsse.act_rows(x, out, kind, params, gate)
     else:
@@ -446,3 +448,65 @@ def qkv_rows(x, bias, heads: int, kv_heads: int, dim: int, vdim: int, eps: float
         torch.ops.dsse.qkv_rows(x, bias, heads, kv_heads, dim, vdim, eps, slots, q, kcache, vcache, vt)
     else:
         lref.qkv_rows(x, bias, heads, kv_heads, dim, vdim, eps, slots, q, kcache, vcache, vt)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Designs with convolved attention, attention beside a matrix memory, and experts chosen by token id.
+def conv_qkv_rows(x, taps, tail, q_start, q_len, ctx_len, state_slot, work_seq, work_tile, qt: int, heads: int,
+                  kv_heads: int, dim: int, vdim: int, rope, q_factor, slots, q, kcache, vcache, vt=None):
+    """The fused projection's rows x [T, ..] (fp32, columns [q | k | v | anything]) into the attention's operands in one
+    launch, per work item of `qt` rows of a sequence: with taps ([(H + G) D, K] fp32) q and k pass a causal convolution
+    over time per channel, continued from the slot's tail [slots, K - 1, (H + G) D] (which is moved); then the leading
+    2 * rope.shape[1] coordinates of every q and k head turn as interleaved pairs (rope [positions, dims / 2, 2] or
+    None); queries are multiplied by q_factor[position] (fp32, or None).  q [T, H, D] (fp32) receives the queries, the
+    pages [pages, 32, G, D] / [pages, 32, G, V] the keys and values at rows slots[t] (negative: skipped), vt the values
+    once more in transposed pages.  vdim = 0: there are no value columns, the values are the convolved keys before their
+    rotation.  qt = 1: every sequence has one row (a decode step)."""
+    if _hip(x):
+        torch.ops.dsse.conv_qkv_rows(x, taps, tail, q_start, q_len, ctx_len, state_slot, work_seq, work_tile, qt, heads,
+                                     kv_heads, dim, vdim, rope, q_factor, slots, q, kcache, vcache, vt)
+    else:
+        lref.conv_qkv_rows(x, taps, tail, q_start, q_len, ctx_len, state_slot, heads, kv_heads, dim, vdim, rope, q_factor,
+                           slots, q, kcache, vcache, vt)
+
+
+MEMORY_CHUNK = 32       # tokens per chunk of the MFMA form of matrix_memory
+
+
+def memory_chunk_ok(dtype, dim: int, vdim: int) -> bool:
+    """Shapes the MFMA form of matrix_memory covers (prompt portions; everything else takes the walk)."""
+    return dtype == torch.bfloat16 and dim <= 256 and dim % 4 == 0
+
+
+def memory_work_floats(rows: int, heads: int, vdim: int) -> int:
+    """fp32 words of the MFMA form's work area: read-outs, normaliser products, running maxima and two gate sums."""
+    return rows * heads * (vdim + 4)
+
+
+def matrix_memory(q, k, v, gates, gate_b, cap: float, state, norm, q_start, q_len, ctx_len, state_slot, out_gate, norm_w,
+                  eps: float, den_eps: float, q_scale: float, out_scale: float, out, work=None):
+    """Matrix memory with exponential gates per (sequence, head), continued from the slot's state [slots, H, D, V] and
+    norm [slots, H, D + 1] (the normaliser, then the running maximum; zeros at position 0), all fp32:
+    i = cap tanh((gates[:, :H] + b_i) / cap), f = logsigmoid(cap tanh((gates[:, H:] + b_f) / cap)), gate_b = [b_i | b_f];
+    m' = max(f + m, i); S = e^(f + m - m') S + e^(i - m') k v^T; n likewise with k alone;
+    o = S^T q / (max(|n . q|, e^-m') + den_eps) with q times q_scale.  Then out [T, H V] (element type, a column slice is
+    fine) = o / rms(o) per head * norm_w [H V] * sigmoid(out_gate) * out_scale.  q, k [T, H, D], v [T, H, V], gates and
+    out_gate are fp32 column slices.  work (fp32, memory_work_floats; memory_chunk_ok shapes): the MFMA form over chunks
+    of MEMORY_CHUNK tokens for prompt portions; None: the walk, a token at a time, any sizes, both element types."""
+    if _hip(v):
+        torch.ops.dsse.matrix_memory(q, k, v, gates, gate_b, cap, state, norm, q_start, q_len, ctx_len, state_slot, out_gate,
+                                     norm_w, eps, den_eps, q_scale, out_scale, out, work)
+    else:
+        lref.matrix_memory(q, k, v, gates, gate_b, cap, state, norm, q_start, q_len, ctx_len, state_slot, out_gate, norm_w,
+                           eps, den_eps, q_scale, out_scale, out)
+
+
+def moe_table_lists(ids, tables: list, experts: list, shared: list, topk_idx: list, sorted_ids: list, tile_expert: list,
+                    num_tiles: list):
+    """The choices and moe_grouped work lists of EVERY table-routed layer of a step in one launch: layer l's experts of
+    row r are tables[l][ids[r]] ([vocab, top] int32, distinct in a row); topk_idx[l] [M, top] receives them, the other
+    lists are moe_grouped's scratch, made for experts[l] experts and, with shared[l], the shared expert's slot."""
+    if _hip(ids):
+        torch.ops.dsse.moe_table_lists(ids, tables, experts, shared, topk_idx, sorted_ids, tile_expert, num_tiles)
+    else:
+        lref.moe_table_lists(ids, tables, topk_idx)

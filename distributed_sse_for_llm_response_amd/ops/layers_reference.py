@@ -291,14 +291,15 @@ def norm_rope_rows(x, norm_w, positions, rope, out, out_rows, norm_kind, eps, sc
 
 
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sink, gate, out, window, scale, vt=None,
-                   softcap=0.0, out_rope=None, rel=None, keep_first=0):
+                   softcap=0.0, out_rope=None, rel=None, keep_first=0, out_scale=1.0):
     """Softmax attention over paged keys [pages, PAGE, G, D] and values [pages, PAGE, G, V] with grouped heads; the
     denominator also holds exp(sink[h]) when sink is given; the head's output is multiplied by sigmoid(gate[row, h])
     when gate is given.  With vt the values come from the transposed pages [pages, G, V, PAGE].  softcap > 0: scores
     softcap * tanh(. / softcap).  out_rope [positions, V / 2, 2]: the head's output is turned BACK by the query's
     position (rotate-half pairs), undoing the rotation of a value rotated by that same position.  rel [H, N]: the entry of
     the key's distance (the last one for distances from N - 1 on) is added to the score.  keep_first: that many first keys
-    of the sequence stay visible outside the window.  A gate of H * V columns is applied element by element."""
+    of the sequence stay visible outside the window.  A gate of H * V columns is applied element by element.  out_scale
+    multiplies the output before it is rounded."""
     H = q.shape[1]
     G = kcache.shape[2]
     kf = kcache.view(-1, G, kcache.shape[3]).float()
@@ -337,7 +338,7 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sin
                 o = rotate_half_rows(o[None], cs[None], 2 * out_rope.shape[1])[0]
             if gate is not None:
                 o = o * torch.sigmoid(gate[r0 + i].float()).view(H, -1)
-            out[r0 + i] = o.to(out.dtype)
+            out[r0 + i] = (o * out_scale).to(out.dtype)
 
 
 def gate_math(x, kind, p1, p2, c):
@@ -428,13 +429,15 @@ def stream_mix(y, nsum, mult, streams, ids, embed, embed_scale, out_w, mix, in_w
 
 def act_rows(x, out, kind, params, gate):
     """out = act(x) * sigmoid(gate) (gate given).  kind 0: identity; 1: a_p z^2 + z / 2 for z > 0, else
-    a_n (e^z - 1 - z) + z / 2, with params = (a_p, a_n); 2: relu(z)^2."""
+    a_n (e^z - 1 - z) + z / 2, with params = (a_p, a_n); 2: relu(z)^2; 3: gelu (tanh form)."""
     z = x.float()
     if kind == 1:
         ap, an = params.float()[0], params.float()[1]
         z = torch.where(z > 0, ap * z * z + 0.5 * z, an * (torch.expm1(torch.clamp(z, max=0.0)) - z) + 0.5 * z)
     elif kind == 2:
         z = torch.relu(z).pow(2)
+    elif kind == 3:
+        z = gelu_tanh(z)
     if gate is not None:
         z = z * torch.sigmoid(gate.float())
     out.copy_(z.to(out.dtype))
@@ -552,3 +555,71 @@ def qkv_rows(x, bias, H, G, D, V, eps, slots, q, kcache, vcache, vt):
     if kcache is not None:
         norm_rope_rows(rms_heads(y[:, H * D:(H + G) * D].reshape(T, G, D)), None, None, None, kcache, slots, 0, 0.0, 1.0)
         norm_rope_rows(y[:, (H + G) * D:].reshape(T, G, V), None, None, None, vcache, slots, 0, 0.0, 1.0, vt)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Designs with convolved attention, attention beside a matrix memory, and experts chosen by token id (models/lobidra.py)
+def conv_qkv_rows(x, taps, tail, q_start, q_len, ctx_len, state_slot, H, G, D, V, rope, q_factor, slots, q, kcache, vcache,
+                  vt):
+    """x [T, ..] fp32, columns [q | k | v] (no v columns with V = 0: the values are the unrotated keys)."""
+    C = (H + G) * D
+    for s in range(q_len.numel()):
+        ql = int(q_len[s])
+        if ql <= 0:
+            continue
+        r0 = int(q_start[s])
+        rows = slice(r0, r0 + ql)
+        pos = torch.arange(int(ctx_len[s]) - ql, int(ctx_len[s]))
+        y = x[rows, :C].float()
+        if taps is not None:
+            y = torch.empty_like(y)
+            one = [t[s:s + 1] for t in (q_len, ctx_len, state_slot)]
+            conv_state(x[rows, :C], taps, None, tail, torch.zeros_like(one[0]), *one, y, None)
+        qh, kh = y[:, :H * D].reshape(ql, H, D), y[:, H * D:].reshape(ql, G, D)
+        vh = kh if V == 0 else x[rows, C:C + G * V].float().reshape(ql, G, V)
+        if rope is not None:
+            n = 2 * rope.shape[1]
+            cs = rope[pos.clamp(max=rope.shape[0] - 1)][:, None]
+            qh, kh = (torch.cat([_rotate(t[..., :n], cs), t[..., n:]], dim=-1) for t in (qh, kh))
+        if q_factor is not None:
+            qh = qh * q_factor[pos.clamp(max=q_factor.numel() - 1)][:, None, None]
+        q[rows] = qh
+        norm_rope_rows(kh, None, None, None, kcache, slots[rows], 0, 0.0, 1.0)
+        norm_rope_rows(vh, None, None, None, vcache, slots[rows], 0, 0.0, 1.0, vt)
+
+
+def matrix_memory(q, k, v, gates, gate_b, cap, state, norm, q_start, q_len, ctx_len, state_slot, out_gate, norm_w, eps,
+                  den_eps, q_scale, out_scale, out):
+    """One token at a time; norm [slots, H, D + 1] holds the normaliser and, last, the running maximum."""
+    T, H, V = v.shape
+    D = k.shape[2]
+    z = cap * torch.tanh((gates.float() + gate_b) / cap)
+    ig, fg = z[:, :H], torch.nn.functional.logsigmoid(z[:, H:])
+    for s in range(q_len.numel()):
+        ql = int(q_len[s])
+        if ql <= 0:
+            continue
+        r0, slot = int(q_start[s]), int(state_slot[s])
+        fresh = int(ctx_len[s]) - ql == 0
+        S = torch.zeros(H, D, V) if fresh else state[slot].clone()
+        n = torch.zeros(H, D) if fresh else norm[slot, :, :D].clone()
+        m = torch.zeros(H) if fresh else norm[slot, :, D].clone()
+        for t in range(r0, r0 + ql):
+            new = torch.maximum(fg[t] + m, ig[t])
+            keep, put = torch.exp(fg[t] + m - new), torch.exp(ig[t] - new)
+            m = new
+            kt, qt = k[t].float(), q[t].float() * q_scale
+            S = keep[:, None, None] * S + put[:, None, None] * kt[:, :, None] * v[t].float()[:, None, :]
+            n = keep[:, None] * n + put[:, None] * kt
+            den = torch.maximum((n * qt).sum(-1).abs(), torch.exp(-m)) + den_eps
+            o = torch.einsum("hdv,hd->hv", S, qt) / den[:, None]
+            o = o / torch.sqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w.view(H, V)
+            out[t] = (o.reshape(-1) * torch.sigmoid(out_gate[t].float()) * out_scale).to(out.dtype)
+        state[slot], norm[slot, :, :D], norm[slot, :, D] = S, n, m
+
+
+def moe_table_lists(ids, tables, topk_idx):
+    for table, idx in zip(tables, topk_idx):
+        row = ids[:idx.shape[0]].long()
+        row = torch.where((row >= 0) & (row < table.shape[0]), row, torch.zeros_like(row))
+        idx.copy_(table[row])

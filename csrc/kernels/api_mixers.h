@@ -67,6 +67,8 @@ struct SinkAttnParams {
   int rel_len;
   int keep_first;        // the sequence's first keys that stay visible outside the window
   int gate_wide;         // 1: the gate has H * V columns, one per element of the output
+  int ldo;               // row stride of out, H * V when contiguous (a multiple of 4 for the MFMA form)
+  float out_scale;       // multiplies the output before it is rounded (1: nothing)
 };
 
 // The fused projection's q | k | v columns into the attention's operands.
@@ -211,7 +213,7 @@ hipError_t dsse_add_norm_rows(const dsse::AddNormParams* p, hipStream_t st);
 hipError_t dsse_token_gate_rows(const float* x, int ldx, const int* ids, const void* table, int vocab, int ldt, int col0,
                                 void* out, int M, int F, int f32, hipStream_t st);
 hipError_t dsse_stream_mix(const dsse::StreamMixParams* p, hipStream_t st);
-// out [M, F] = act(x) * sigmoid(gate): kind 0 identity, 1 xIELU with params = (a_p, a_n), 2 relu^2; gate may be null
+// out [M, F] = act(x) * sigmoid(gate): kind 0 identity, 1 xIELU with params = (a_p, a_n), 2 relu^2, 3 gelu (tanh); gate may be null
 hipError_t dsse_act_rows(const float* x, int ldx, void* out, int M, int F, int kind, const float* params,
                          const float* gate, int ldg, int f32, hipStream_t st);
 // group-limited routing from fp32 logits [M, E] (E <= 256); kind 0: sigmoid scores + correction, groups by the sum of

@@ -177,11 +177,11 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
                     const Tensor& q_start, const Tensor& q_len, const Tensor& ctx_len, const Tensor& work_seq,
                     const Tensor& work_tile, const OptTensor& sink, const OptTensor& gate, Tensor& out, int64_t window,
                     double scale, int64_t qt, const OptTensor& vt, bool split, double softcap, const OptTensor& out_rope,
-                    const OptTensor& rel, int64_t keep_first) {
+                    const OptTensor& rel, int64_t keep_first, double out_scale) {
   f32t(q, "q");
   gpu(kcache, "kcache");
   gpu(vcache, "vcache");
-  gpu(out, "out");
+  gpu(out, "out", false);
   TORCH_CHECK(kcache.scalar_type() == vcache.scalar_type() && out.scalar_type() == kcache.scalar_type(),
               "kcache, vcache and out share the element type");
   i32(block_tables, "block_tables");
@@ -196,6 +196,11 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
               "caches must be [pages, 32, G, D] and [pages, 32, G, V]");
   TORCH_CHECK(p.G >= 1 && p.H % p.G == 0 && p.D <= 512 && p.V <= 512, "heads must be a multiple of kv heads, widths <= 512");
   TORCH_CHECK(out.size(0) == T && out.size(1) == p.H && out.size(2) == p.V, "out must be [T, H, V]");
+  TORCH_CHECK((p.V == 1 || out.stride(2) == 1) && (p.H == 1 || out.stride(1) == p.V) && out.stride(0) >= (int64_t)p.H * p.V &&
+                  out.stride(0) < INT_MAX,
+              "out rows must hold adjacent heads");
+  p.ldo = (int)out.stride(0);
+  p.out_scale = (float)out_scale;
   TORCH_CHECK(block_tables.dim() == 2, "block_tables must be [seqs, max_blocks]");
   const int ns = (int)block_tables.size(0);
   seq_meta(q_start, q_len, ctx_len, ns);
@@ -255,6 +260,7 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
       DSSE_CHECK_HIP(dsse_sink_decode((int)work_seq.numel(), &p, vt->data_ptr(), cur_stream()));
       return;
     }
+    TORCH_CHECK(p.ldo % 4 == 0 && reinterpret_cast<uintptr_t>(p.out) % 8 == 0, "the MFMA form stores 8-byte pieces of out");
     TORCH_CHECK(qt == 16 && p.D % 32 == 0 && p.V % 16 == 0, "the MFMA form needs qt = 16, D % 32 == 0, V % 16 == 0");
     TORCH_CHECK(!split || p.V <= 128, "the key split of the MFMA form needs V <= 128");
     DSSE_CHECK_HIP(dsse_sink_flash((int)work_seq.numel(), &p, vt->data_ptr(), split ? 1 : 0, cur_stream()));
@@ -522,7 +528,7 @@ void act_rows(const Tensor& x, Tensor& out, int64_t kind, const OptTensor& param
   col_view(x, "x");
   gpu(out, "out");
   TORCH_CHECK(out.dim() == 2 && out.sizes() == x.sizes(), "out must be [M, F] like x");
-  TORCH_CHECK(kind >= 0 && kind <= 2, "kind: 0 identity, 1 xIELU, 2 relu^2");
+  TORCH_CHECK(kind >= 0 && kind <= 3, "kind: 0 identity, 1 xIELU, 2 relu^2, 3 gelu");
   const float* pp = opt_f32(params, "params", 2);
   TORCH_CHECK(kind != 1 || pp, "xIELU needs its two constants");
   const float* g = nullptr;
@@ -783,7 +789,7 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
   m.def("sink_attention(Tensor q, Tensor kcache, Tensor vcache, Tensor block_tables, Tensor q_start, Tensor q_len, "
         "Tensor ctx_len, Tensor work_seq, Tensor work_tile, Tensor? sink, Tensor? gate, Tensor(a!) out, int window, "
         "float scale, int qt, Tensor? vt=None, bool split=False, float softcap=0.0, Tensor? out_rope=None, "
-        "Tensor? rel=None, int keep_first=0) -> ()");
+        "Tensor? rel=None, int keep_first=0, float out_scale=1.0) -> ()");
   m.def("gate_math(Tensor(a!) x, int kind, Tensor? p1=None, Tensor? p2=None, float c=1.0) -> ()");
   m.def("matrix_scan(Tensor q, Tensor k, Tensor v, Tensor? decay, Tensor? beta, Tensor(a!) state, Tensor q_start, "
         "Tensor q_len, Tensor ctx_len, Tensor state_slot, Tensor(b!) out, float q_scale=1.0) -> ()");

@@ -8,6 +8,7 @@
 //                fp32 (the residual norm follows).  Each expert's weights are read once per row that chose it: the
 //                decode-shaped path (few rows per expert), and correct for any row count.
 #include "api_layers.h"
+#include "api_memory.h"
 #include "frag.h"
 
 namespace dsse {
@@ -170,9 +171,9 @@ DEV float in_weight(const MoeGroupedParams& p, int id) {
 
 constexpr int kMoeRows = 64;  // rows of one expert per workgroup tile: four 16-row MFMA tiles share every weight fragment
 
-// The work list from the choices, by one workgroup; sm holds 3 NE + 1 ints.  The choices are read with agent scope: in the
-// one-launch form below other workgroups of the same launch have just written them.
-DEV void align_ids(int M, int S, int top, int E, const int* topk_idx, int* sorted, int* tile_expert, int* num_tiles,
+// The work list from the choices, by one workgroup; sm holds 3 NE + 1 ints.  choice(row, k): expert k of a row.
+template <typename Choice>
+DEV void align_ids(int M, int S, int top, int E, Choice choice, int* sorted, int* tile_expert, int* num_tiles,
                    int max_tiles, int* sm) {
   const int NE = E + (S > top ? 1 : 0);
   int* cnt = sm;            // [NE]
@@ -181,7 +182,7 @@ DEV void align_ids(int M, int S, int top, int E, const int* topk_idx, int* sorte
   const int n = M * S;
   auto expert_of = [&](int id) {
     const int row = id / S, k = id % S;
-    const int e = k < top ? __hip_atomic_load(topk_idx + row * top + k, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) : E;
+    const int e = k < top ? choice(row, k) : E;
     return (unsigned)e < (unsigned)NE ? e : 0;
   };
   const int mine = (int)threadIdx.x < n ? expert_of(threadIdx.x) : 0;  // a thread's first id: read once
@@ -223,7 +224,21 @@ DEV void align_ids(int M, int S, int top, int E, const int* topk_idx, int* sorte
 
 __global__ __launch_bounds__(256) void moe_align_kernel(MoeGroupedParams p) {
   extern __shared__ int sm[];
-  align_ids(p.M, p.S, p.top, p.E, p.topk_idx, p.sorted, p.tile_expert, p.num_tiles, p.max_tiles, sm);
+  align_ids(p.M, p.S, p.top, p.E, [&](int row, int k) { return p.topk_idx[row * p.top + k]; }, p.sorted, p.tile_expert,
+            p.num_tiles, p.max_tiles, sm);
+}
+
+// Experts by token id: a row's choice is a table row, so the lists of every such layer of a step come from ONE launch, a
+// workgroup per layer, before the first layer runs.
+__global__ __launch_bounds__(1024) void moe_table_lists_kernel(MoeTableListsParams p) {
+  extern __shared__ int sm[];
+  const MoeTableListsParams::Layer L = p.layer[blockIdx.x];
+  auto choice = [&](int row, int k) {
+    const int id = p.ids[row];
+    return L.table[(int64_t)((unsigned)id < (unsigned)p.vocab ? id : 0) * L.top + k];
+  };
+  for (int i = threadIdx.x; i < p.M * L.top; i += blockDim.x) L.topk_idx[i] = choice(i / L.top, i % L.top);
+  align_ids(p.M, L.S, L.top, L.E, choice, L.sorted, L.tile_expert, L.num_tiles, L.max_tiles, sm);
 }
 
 // Router, choice and work list of a decode-sized step in ONE launch (three latency-sized ones otherwise): a workgroup of
@@ -331,8 +346,11 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_rows_kernel(MoeRouteR
     }
   }
   __syncthreads();
-  if (!last) return;  // uniform for the workgroup; align_ids reads the choices with agent scope
-  align_ids(p.M, p.S, p.top, p.E, p.topk_idx, p.sorted, p.tile_expert, p.num_tiles, p.max_tiles, sm);
+  if (!last) return;  // uniform for the workgroup
+  // agent scope: other workgroups of this launch have just written the choices
+  align_ids(p.M, p.S, p.top, p.E, [&](int row, int k) {
+    return __hip_atomic_load(p.topk_idx + row * p.top + k, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }, p.sorted, p.tile_expert, p.num_tiles, p.max_tiles, sm);
 }
 
 // Both expert GEMMs: a workgroup owns 16 output columns of one 64-row tile; its four waves split the K axis and meet in
@@ -710,5 +728,16 @@ extern "C" hipError_t dsse_moe_route_rows(const dsse::MoeRouteRowsParams* p, hip
   if (p->E > 64 * dsse::kRouteLanes || p->top < 1 || p->top > p->E || p->S < p->top || p->S > p->top + 1)
     return hipErrorInvalidValue;
   hipLaunchKernelGGL(dsse::moe_route_rows_kernel, dim3(p->M), dim3(dsse::kRouteThreads), sizeof(int) * (4 * NE + 1), st, *p);
+  return hipGetLastError();
+}
+
+extern "C" hipError_t dsse_moe_table_lists(const dsse::MoeTableListsParams* p, hipStream_t st) {
+  if (p->M <= 0 || p->layers <= 0) return hipSuccess;
+  if (p->layers > dsse::kTableLayers) return hipErrorInvalidValue;
+  int ne = 0;
+  for (int i = 0; i < p->layers; ++i) ne = p->layer[i].E + 1 > ne ? p->layer[i].E + 1 : ne;
+  if (ne > 4096) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(dsse::moe_table_lists_kernel, dim3(p->layers), dim3(p->M > 64 ? 1024 : 256),
+                     sizeof(int) * (3 * ne + 1), st, *p);
   return hipGetLastError();
 }

@@ -178,6 +178,8 @@ __global__ __launch_bounds__(256) void act_rows_kernel(const float* x, int ldx, 
       z = z > 0.0f ? ap * z * z + 0.5f * z : an * (expm1f(z) - z) + 0.5f * z;
     } else if (kind == 2) {
       z = z > 0.0f ? z * z : 0.0f;
+    } else if (kind == 3) {
+      z = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
     }
     if (gate) z *= 1.0f / (1.0f + expf(-gate[r * ldg + c]));
     out[i] = (T)z;

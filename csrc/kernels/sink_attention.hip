@@ -11,7 +11,8 @@
 //
 // A gate may also have one column per element of the output instead of one per head.  Distance bias and kept keys: an
 // entry rel[h][min(pos - j, rel_len - 1)] joins the score (after the scale), and the sequence's first keep_first keys stay
-// visible when the window has passed them: the kernels then walk the kept keys first and jump to the window.
+// visible when the window has passed them: the kernels then walk the kept keys first and jump to the window.  The output
+// rows may be a column slice of a wider buffer (rows ldo apart) and are multiplied by out_scale before they are rounded.
 //
 // The sink is a learned logit with no key and no value: it only enlarges the denominator, so a head can attend to
 // "nothing".  Scores, the running maximum, the weights and the output sums are fp32 in both element types; queries
@@ -137,7 +138,7 @@ __global__ __launch_bounds__(256) void sink_attention_kernel(SinkAttnParams p) {
     }
     const float* gp = p.gate ? p.gate + (int64_t)row * p.ldg + (p.gate_wide ? h * p.V : h) : nullptr;
     const float gate = gp && !p.gate_wide ? 1.0f / (1.0f + expf(-gp[0])) : 1.0f;
-    T* out = reinterpret_cast<T*>(p.out) + ((int64_t)row * p.H + h) * V;
+    T* out = reinterpret_cast<T*>(p.out) + (int64_t)row * p.ldo + h * V;
     const int half = V >> 1;
     const float2* orp = p.out_rope ? p.out_rope + (int64_t)(pos < p.out_rope_len ? pos : p.out_rope_len - 1) * half : nullptr;
     for (int d = threadIdx.x; d < V; d += blockDim.x) {
@@ -153,7 +154,7 @@ __global__ __launch_bounds__(256) void sink_attention_kernel(SinkAttnParams p) {
       }
       o = o / den * gate;
       if (p.gate_wide) o *= 1.0f / (1.0f + expf(-gp[d]));
-      out[d] = (T)o;
+      out[d] = (T)(o * p.out_scale);
     }
   }
 }
@@ -426,7 +427,7 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
       }
       float o = den > 0.f ? num / den : 0.f;
       if (p.gate) o *= 1.0f / (1.0f + expf(-p.gate[row * p.ldg + (p.gate_wide ? h * V + d : h)]));
-      reinterpret_cast<bf16*>(p.out)[(row * p.H + h) * V + d] = (bf16)o;
+      reinterpret_cast<bf16*>(p.out)[row * p.ldo + h * V + d] = (bf16)(o * p.out_scale);
     }
     return;
   }
@@ -438,7 +439,7 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
       f = expf(m - mm);
       den = l * f + expf(sk - mm);
     }
-    float inv = den > 0.f ? f / den : 0.0f;
+    float inv = den > 0.f ? f / den * p.out_scale : 0.0f;
     if (p.gate && !p.gate_wide) inv *= 1.0f / (1.0f + expf(-p.gate[c_row * p.ldg + h]));
     if (p.out_rope) {  // NT is even (the host checks V % 32 == 0): dimension m = 16 n + 4 g + i pairs with tile n + NT / 2
       const float2* orp = p.out_rope + (int64_t)(c_pos < p.out_rope_len ? c_pos : p.out_rope_len - 1) * (V >> 1);
@@ -452,7 +453,7 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
           O[n + NT / 2][i] = b * c.x - a * c.y;
         }
     }
-    bf16* out = reinterpret_cast<bf16*>(p.out) + (c_row * p.H + h) * V;
+    bf16* out = reinterpret_cast<bf16*>(p.out) + c_row * p.ldo + h * V;
     const float* gw = p.gate_wide ? p.gate + c_row * p.ldg + h * V + 4 * g : nullptr;
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
@@ -656,7 +657,7 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
     }
     float o = den > 0.f ? num / den : 0.f;
     if (p.gate) o *= 1.0f / (1.0f + expf(-p.gate[row * p.ldg + (p.gate_wide ? h * V + d : h)]));
-    reinterpret_cast<bf16*>(p.out)[(row * p.H + h) * V + d] = (bf16)o;
+    reinterpret_cast<bf16*>(p.out)[row * p.ldo + h * V + d] = (bf16)(o * p.out_scale);
   }
 }
 

@@ -1150,7 +1150,8 @@ class LayeredRunner(RunnerBase):
             chunked = g["qt"] > 1 and self.device.type == "cuda" and ops.memory_chunk_ok(self.dtype, Dr, Vr)
             ops.matrix_memory(q, k, v, zg[:, :2 * Hr], Lw.gate_b, r.gate_cap, self.state.state[ri], self.state.norm[ri],
                               g["qs"], g["ql"], g["ctx"], g["ss"], gate, Lw.norm, self.cfg.eps, MEMORY_EPS, Dr ** -0.5,
-                              m.right_scale, ao[:, H * V:H * V + Hr * Vr], d["mm"] if chunked else None)
+                              m.right_scale, ao[:, H * V:H * V + Hr * Vr], d["mm"] if chunked else None,
+                              *(g["rows"] if chunked else ()))
         self._lin(ao, Lw.o, Lw.o_t, d["y"])
 
     # ------------------------------------------------------------------ mixer and feed-forward side by side
@@ -1396,6 +1397,7 @@ class LayeredRunner(RunnerBase):
             d[name], o = meta[o:o + k], o + k
         d["bt"] = bt
         d["qt"] = ATTN_ROWS_TILE
+        d["rows"] = (row0, T)   # the packed rows of these portions
         if self.prenorm and T >= ops.layers.SCAN_CHUNKED_FROM:  # long portions: the recurrences' two-level walk
             s_first, s_count, rows = ops.layers.scan_chunks(qs, ql, ss)
             ck = torch.tensor([s_first, s_count], dtype=torch.int32)

@@ -484,7 +484,8 @@ def memory_work_floats(rows: int, heads: int, vdim: int) -> int:
 
 
 def matrix_memory(q, k, v, gates, gate_b, cap: float, state, norm, q_start, q_len, ctx_len, state_slot, out_gate, norm_w,
-                  eps: float, den_eps: float, q_scale: float, out_scale: float, out, work=None):
+                  eps: float, den_eps: float, q_scale: float, out_scale: float, out, work=None, row0: int = 0,
+                  rows: int = 0):
     """Matrix memory with exponential gates per (sequence, head), continued from the slot's state [slots, H, D, V] and
     norm [slots, H, D + 1] (the normaliser, then the running maximum; zeros at position 0), all fp32:
     i = cap tanh((gates[:, :H] + b_i) / cap), f = logsigmoid(cap tanh((gates[:, H:] + b_f) / cap)), gate_b = [b_i | b_f];
@@ -492,10 +493,11 @@ def matrix_memory(q, k, v, gates, gate_b, cap: float, state, norm, q_start, q_le
     o = S^T q / (max(|n . q|, e^-m') + den_eps) with q times q_scale.  Then out [T, H V] (element type, a column slice is
     fine) = o / rms(o) per head * norm_w [H V] * sigmoid(out_gate) * out_scale.  q, k [T, H, D], v [T, H, V], gates and
     out_gate are fp32 column slices.  work (fp32, memory_work_floats; memory_chunk_ok shapes): the MFMA form over chunks
-    of MEMORY_CHUNK tokens for prompt portions; None: the walk, a token at a time, any sizes, both element types."""
+    of MEMORY_CHUNK tokens for prompt portions, whose sequences are the `rows` rows from row0 on; None: the walk, a token at
+    a time, any sizes, both element types."""
     if _hip(v):
         torch.ops.dsse.matrix_memory(q, k, v, gates, gate_b, cap, state, norm, q_start, q_len, ctx_len, state_slot, out_gate,
-                                     norm_w, eps, den_eps, q_scale, out_scale, out, work)
+                                     norm_w, eps, den_eps, q_scale, out_scale, out, work, row0, rows)
     else:
         lref.matrix_memory(q, k, v, gates, gate_b, cap, state, norm, q_start, q_len, ctx_len, state_slot, out_gate, norm_w,
                            eps, den_eps, q_scale, out_scale, out)
@@ -507,6 +509,6 @@ def moe_table_lists(ids, tables: list, experts: list, shared: list, topk_idx: li
     row r are tables[l][ids[r]] ([vocab, top] int32, distinct in a row); topk_idx[l] [M, top] receives them, the other
     lists are moe_grouped's scratch, made for experts[l] experts and, with shared[l], the shared expert's slot."""
     if _hip(ids):
-        torch.ops.dsse.moe_table_lists(ids, tables, experts, shared, topk_idx, sorted_ids, tile_expert, num_tiles)
+        torch.ops.dsse.moe_table_lists(ids, tables, experts, [int(x) for x in shared], topk_idx, sorted_ids, tile_expert, num_tiles)
     else:
         lref.moe_table_lists(ids, tables, topk_idx)

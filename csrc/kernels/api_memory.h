@@ -50,8 +50,9 @@ struct MatrixMemoryParams {
   float* num;            // [T, H, V] read-outs before the division
   float* nq;             // [T, H] normaliser products
   float* m;              // [T, H] running maxima
-  float* acum;           // [H, T] log-decay sums inside a chunk
-  float* u;              // [H, T] log write strength minus that sum
+  float* acum;           // [H, ldsum] log2-decay sums inside a chunk, sequences at multiples of four
+  float* u;              // [H, ldsum] log2 write strength minus that sum
+  int ldsum;             // at least T + 4 nseq + 4, a multiple of 4
   int row0, rows;
   int vec;               // 16-byte loads of q and k rows allowed
 };

@@ -199,10 +199,13 @@ void matrix_memory(const Tensor& q, const Tensor& k, const Tensor& v, const Tens
   f32t(*work, "work");
   const int64_t n = T * H;
   TORCH_CHECK(!p.f32 && D <= 256 && D % 4 == 0, "the MFMA form is bf16, D <= 256, D % 4 == 0");
-  TORCH_CHECK(work->numel() >= n * (V + 4) && aligned16(work->data_ptr()), "work area too small");
+  const int64_t ldsum = ((T + 3) & ~(int64_t)3) + 4 * p.nseq + 4, n4 = (n + 3) & ~(int64_t)3;
+  TORCH_CHECK(work->numel() >= 2 * H * ldsum + 2 * n4 + n * V && aligned16(work->data_ptr()), "work area too small");
+  TORCH_CHECK(p.ldk < (1 << 24) && p.ldq < (1 << 24) && p.ldv < (1 << 24), "q, k, v rows too far apart");
   TORCH_CHECK(row0 >= 0 && rows >= 0 && row0 + rows <= T && rows * H < INT_MAX, "the rows of the call");
   float* w = work->data_ptr<float>();
-  p.num = w, p.nq = w + n * V, p.m = p.nq + n, p.acum = p.m + n, p.u = p.acum + n;
+  p.acum = w, p.u = w + H * ldsum, p.nq = w + 2 * H * ldsum, p.m = p.nq + n4, p.num = p.m + n4;
+  p.ldsum = (int)ldsum;
   p.row0 = (int)row0, p.rows = (int)rows;
   p.vec = aligned16(p.q) && aligned16(p.k) && p.ldq % 4 == 0 && p.ldk % 4 == 0;
   DSSE_CHECK_HIP(dsse_matrix_memory_chunk(&p, cur_stream()));

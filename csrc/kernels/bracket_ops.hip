@@ -139,8 +139,13 @@ __global__ __launch_bounds__(256) void add_norm_rows_kernel(AddNormParams p) {
     });
   } else if (y) {
     float sy = 0.f;
+    FVec<VEC> held[REG ? kNormRegs : 1], gain[REG ? kNormRegs : 1];  // the stream and the gains, requested with y
     each([&](int i, int d) {
       const FVec<VEC> v = parts(d);
+      if (REG) {
+        held[i] = ld_f<VEC>(resid + d);
+        gain[i] = ld_f<VEC>(p.g_add + d);
+      }
 #pragma unroll
       for (int e = 0; e < VEC; ++e) sy += v.v[e] * v.v[e];
       if (REG) vals[i] = v;
@@ -149,8 +154,8 @@ __global__ __launch_bounds__(256) void add_norm_rows_kernel(AddNormParams p) {
     const float inv = 1.0f / sqrtf(sy / (float)W + p.eps);
     each([&](int i, int d) {
       const FVec<VEC> v = REG ? vals[i] : parts(d);
-      const FVec<VEC> g = ld_f<VEC>(p.g_add + d);
-      FVec<VEC> r = ld_f<VEC>(resid + d);
+      const FVec<VEC> g = REG ? gain[i] : ld_f<VEC>(p.g_add + d);
+      FVec<VEC> r = REG ? held[i] : ld_f<VEC>(resid + d);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
         r.v[e] += v.v[e] * inv * g.v[e];

@@ -140,7 +140,13 @@ __global__ __launch_bounds__(256) void conv_qkv_rows_kernel(ConvQkvParams p) {
       }
     }
   }
-  if (p.qt == 1 && Kt > 0)  // one row per sequence: this thread alone reads and writes its channels of the tail (ascending:
+  if (KT > 1 && p.qt == 1 && part != 2) {  // one row per sequence: the window in registers is the new tail
+#pragma unroll
+    for (int j = 0; j + 1 < KR; ++j) {
+      tail[(int64_t)j * C] = w0[j + 1];
+      if (both) tail[(int64_t)j * C + 1] = w1[j + 1];
+    }
+  } else if (p.qt == 1 && Kt > 0)  // one row per sequence: this thread alone reads and writes its channels of the tail (ascending:
     for (int j = 0; j < Kt; ++j) {  // entry j takes the old entry j + ql, not yet overwritten)
       tail[(int64_t)j * C] = input(ql - Kt + j, 0);
       if (both) tail[(int64_t)j * C + 1] = input(ql - Kt + j, 1);

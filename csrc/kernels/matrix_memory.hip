@@ -181,9 +181,9 @@ void launch_walk(const MatrixMemoryParams& p, hipStream_t st) {
 // ---------------------------------------------------------------------------------------------------------------------
 // Chunk form for prompt portions.  The running maximum only rescales, so it is settled first:
 //
-//   memory_gates   one wave per (sequence, head), 64 tokens per step: the maximum is a scan of the pairs
-//                  (sum of f, best i + later f's); log a_t = f_t + m_(t-1) - m_t and log b_t = i_t - m_t are both <= 0.  Left
-//                  behind: A_t = the sum of log a inside its 32-token chunk, u_t = log b_t - A_t, and m_t.
+//   memory_gates   the maximum is a scan of the pairs (sum of f, best i + later f's); log a_t = f_t + m_(t-1) - m_t and
+//                  log b_t = i_t - m_t are both <= 0.  Left behind: A_t = the sum of log a inside its 32-token chunk,
+//                  u_t = log b_t - A_t (both times log2 e), and m_t.
 //   memory_chunk   S_t = a_t S_(t-1) + b_t k v^T over chunks of 32 tokens.  For s <= t of one chunk the write of s weighs
 //                  e^(A_t + u_s) in t's read-out, the incoming state e^(A_t):
 //                      O = e^A (Q S_in) + (Q K^T * W) V,     S_out = e^(A_end) S_in + sum_s e^(A_end + u_s) k_s v_s^T
@@ -200,24 +200,37 @@ void launch_walk(const MatrixMemoryParams& p, hipStream_t st) {
 // weighted scores -- enters as two bf16 parts (value and remainder), so a product carries about 16 bits of it; sums and the
 // state itself are fp32.
 constexpr int kChunk = 32;
+constexpr float kLog2e = 1.4426950408889634f;
 
-__global__ __launch_bounds__(64) void memory_gates_kernel(MatrixMemoryParams p) {
-  const int h = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x;
+// Workgroup barrier that orders LDS traffic only: the next chunk's loads stay in flight across it (__syncthreads() would
+// wait for them); the compiler waits for them where their registers are used.
+DEV void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// Where a sequence's chunk sums start in acum / u: the rows keep their order, every start is a multiple of four floats.
+DEV int sums_at(int row0, int seq) { return ((row0 + 3) & ~3) + 4 * seq; }
+
+// Sixteen waves per (sequence, head) take 1024 tokens at a time: a wave scans its 64, the waves' totals meet in LDS, and
+// every wave folds those before it.
+constexpr int kGateWaves = 16;
+
+__global__ __launch_bounds__(64 * kGateWaves) void memory_gates_kernel(MatrixMemoryParams p) {
+  __shared__ float tot_f[2][kGateWaves], tot_m[2][kGateWaves];
+  const int h = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int ql = p.q_len[seq];
   if (ql <= 0) return;
-  const int64_t row0 = p.q_start[seq];
+  const int row0 = p.q_start[seq];
   float* nm = p.norm + ((int64_t)p.state_slot[seq] * p.H + h) * (p.D + 1);
   float m_in = p.ctx_len[seq] - ql == 0 ? 0.0f : nm[p.D];
   const float bi = p.gate_b[h], bf = p.gate_b[p.H + h];
-  auto z_at = [&](int t, int c) { return t < ql ? p.gates[(row0 + t) * p.ldz + c * p.H + h] : 0.0f; };
-  float zi = z_at(lane, 0), zf = z_at(lane, 1);
-  for (int b = 0; b < ql; b += 64) {
-    const int t = b + lane;
+  float* acum = p.acum + (int64_t)h * p.ldsum + sums_at(row0, seq);
+  float* us = p.u + (int64_t)h * p.ldsum + sums_at(row0, seq);
+  for (int b = 0, it = 0; b < ql; b += 64 * kGateWaves, ++it) {
+    const int t = b + threadIdx.x;
     const bool on = t < ql;
-    const float i = on ? softcap_f(zi + bi, p.cap) : -INFINITY;
-    const float f = on ? logsigmoid_f(softcap_f(zf + bf, p.cap)) : 0.0f;
-    zi = z_at(t + 64, 0), zf = z_at(t + 64, 1);  // the next step's, in flight over the scans
-    float F = f, M = i;
+    const float* z = p.gates + (int64_t)(row0 + (on ? t : 0)) * p.ldz + h;
+    const float i = on ? softcap_f(z[0] + bi, p.cap) : -INFINITY;
+    const float f = on ? logsigmoid_f(softcap_f(z[p.H] + bf, p.cap)) : 0.0f;
+    float F = f, M = i;  // sum of f; the largest i plus the f after it
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
       const float Fp = __shfl_up(F, o), Mp = __shfl_up(M, o);
@@ -226,9 +239,17 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(MatrixMemoryParams p) 
         F += Fp;
       }
     }
-    const float m = fmaxf(m_in + F, M);
+    float *tf = tot_f[it & 1], *tm = tot_m[it & 1];  // two strips: one barrier per round
+    if (lane == 63) tf[wave] = F, tm[wave] = M;
+    __syncthreads();
+    float mw = m_in;  // the maximum ahead of this wave's tokens, and after all of the round's
+    for (int w = 0; w < kGateWaves; ++w) {
+      if (w == wave) mw = m_in;
+      m_in = fmaxf(m_in + tf[w], tm[w]);
+    }
+    const float m = fmaxf(mw + F, M);
     float mp = __shfl_up(m, 1);
-    if (lane == 0) mp = m_in;
+    if (lane == 0) mp = mw;
     float A = on ? f + mp - m : 0.0f;
     const float lb = i - m;
 #pragma unroll
@@ -237,13 +258,12 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(MatrixMemoryParams p) 
       if ((lane & (kChunk - 1)) >= o) A += Ap;
     }
     if (on) {
-      p.acum[(int64_t)h * p.T + row0 + t] = A;
-      p.u[(int64_t)h * p.T + row0 + t] = lb - A;
-      p.m[(row0 + t) * p.H + h] = m;
+      acum[t] = A * kLog2e;
+      us[t] = (lb - A) * kLog2e;
+      p.m[(int64_t)(row0 + t) * p.H + h] = m;
     }
-    m_in = __shfl(m, 63);
   }
-  if (lane == 0) nm[p.D] = m_in;
+  if (threadIdx.x == 0) nm[p.D] = m_in;  // every thread has read the old one before the first barrier
 }
 
 // value and remainder of fp32 numbers as bf16 operands
@@ -254,9 +274,16 @@ DEV void split8(const float (&x)[8], bf16x8& hi, bf16x8& lo) {
     lo[j] = (bf16)(x[j] - (float)hi[j]);
   }
 }
+// 2^x (one instruction): arguments here are at most 0 up to rounding
+DEV float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
+// uniform base, 32-bit lane offset in floats
+template <typename V>
+DEV V ld_at(const float* base, unsigned off) {
+  return ld_global<V>(reinterpret_cast<const char*>(base) + 4u * off);
+}
 
-// NK: 32-row groups of S (D rounded up); NW: waves (16-column tiles) per workgroup
-template <int NK, int NW>
+// NK: 32-row groups of S (D rounded up); NW: waves (16-column tiles) per workgroup; VEC: 16-byte loads of q and k rows
+template <int NK, int NW, bool VEC>
 __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParams p) {
   constexpr int Dp = 32 * NK, ldr = Dp + 8, ldt = kChunk + 8;
   constexpr int Q4 = 8 * NK;                  // 4-coordinate pieces of a row
@@ -272,7 +299,7 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
   const bool live = ct <= vtiles, is_norm = ct == vtiles;
   const int col = ct * 16 + r;
   const bool col_on = live && !is_norm && col < V;
-  const int64_t row0 = p.q_start[seq];
+  const int row0 = p.q_start[seq];
   const bool fresh = p.ctx_len[seq] - ql == 0;
   const int64_t entry = (int64_t)p.state_slot[seq] * p.H + h;
   float* st = p.state + entry * D * V + col;
@@ -290,43 +317,81 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
       }
       S[dt][i] = s;
     }
-  // the next chunk's inputs, requested while the current one is in the MFMAs
-  f32x4 nk[NB][4], nq[NB][4];
-  float nv[8], nu[8], nA0, nA1, nAL;
-  const float* Ah = p.acum + (int64_t)h * p.T + row0;
-  const float* uh = p.u + (int64_t)h * p.T + row0;
-  auto token_of = [&](int j) { return j < 4 ? 4 * g + j : 16 + 4 * g + (j - 4); };  // of k-axis slot (g, j)
-  auto ld4 = [&](const float* q) {
-    if (p.vec) return ld_global<f32x4>(q);
-    return f32x4{q[0], q[1], q[2], q[3]};
+  // The next chunk's inputs, requested while the current one is in the MFMAs.  Lane offsets are 32-bit and the same for
+  // every chunk, the moving part of an address is uniform.
+  f32x4 nk[NB][4], nq[NB][4], nu[2];
+  float nv[8], nA0, nA1, nAL;
+  const int64_t sums = (int64_t)h * p.ldsum + sums_at(row0, seq);
+  unsigned koff[NB], qoff[NB];
+  bool piece[NB];
+#pragma unroll
+  for (int n = 0; n < NB; ++n) {
+    const int b = n * 64 * NW + tid, d = 4 * (b % Q4), tq = 4 * (b / Q4);
+    piece[n] = b < 64 * NK && d < D;
+    koff[n] = piece[n] ? (unsigned)(tq * p.ldk + d) : 0u;  // pieces that do not exist read the first one and are masked
+    qoff[n] = piece[n] ? (unsigned)(tq * p.ldq + d) : 0u;
+  }
+  const unsigned voff = col_on ? (unsigned)(4 * g * p.ldv + col) : 0u;
+  const f32x4 zero4 = f32x4{0.f, 0.f, 0.f, 0.f};
+  auto ld4 = [&](const float* base, unsigned off) {
+    if constexpr (VEC) return ld_at<f32x4>(base, off);
+    else return f32x4{ld_at<float>(base, off), ld_at<float>(base, off + 1), ld_at<float>(base, off + 2), ld_at<float>(base, off + 3)};
   };
-  auto request = [&](int t0) {
+  auto request = [&](int t0) {  // no branch around a load: all of them are in flight together
     const int nt = ql - t0 < kChunk ? ql - t0 : kChunk;
+    const int64_t row = row0 + t0;
+    const float* kb = p.k + row * p.ldk + h * D;
+    const float* qb = p.q + row * p.ldq + h * D;
+    const float* vb = p.v + row * p.ldv + h * V;
+    const float *Ab = p.acum + sums + t0, *ub = p.u + sums + t0;
+    if (nt == kChunk) {
 #pragma unroll
-    for (int n = 0; n < NB; ++n) {
-      const int b = n * 64 * NW + tid, d = 4 * (b % Q4), tq = 4 * (b / Q4);
+      for (int n = 0; n < NB; ++n)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const bool on = tq + j < nt && d < D;
-        const int64_t row = row0 + t0 + tq + j;
-        nk[n][j] = on ? ld4(p.k + row * p.ldk + h * D + d) : f32x4{0.f, 0.f, 0.f, 0.f};
-        nq[n][j] = on ? ld4(p.q + row * p.ldq + h * D + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j < 4; ++j) {
+          nk[n][j] = ld4(kb + j * p.ldk, koff[n]);
+          nq[n][j] = ld4(qb + j * p.ldq, qoff[n]);
+        }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) nv[j] = ld_at<float>(vb + ((j & 3) + 16 * (j >> 2)) * p.ldv, voff);
+      nu[0] = ld_at<f32x4>(ub, 4 * g);
+      nu[1] = ld_at<f32x4>(ub + 16, 4 * g);
+      nA0 = ld_at<float>(Ab, r);
+      nA1 = ld_at<float>(Ab + 16, r);
+      nAL = Ab[kChunk - 1];
+    } else {  // the last tokens: rows past the end read the first one (masked below), their sums are the last token's
+#pragma unroll
+      for (int n = 0; n < NB; ++n) {
+        const int tq = 4 * ((n * 64 * NW + tid) / Q4);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const bool on = piece[n] && tq + j < nt;
+          nk[n][j] = ld4(kb, on ? koff[n] + j * p.ldk : 0u);
+          nq[n][j] = ld4(qb, on ? qoff[n] + j * p.ldq : 0u);
+        }
       }
-    }
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int s = token_of(j);
-      nv[j] = s >= nt ? 0.0f : (is_norm ? (r == 0 ? 1.0f : 0.0f) : (col_on ? p.v[(row0 + t0 + s) * p.ldv + h * V + col] : 0.0f));
-      nu[j] = uh[t0 + (s < nt ? s : nt - 1)];
+      for (int j = 0; j < 8; ++j) {
+        const int c = (j & 3) + 16 * (j >> 2), s = 4 * g + c;
+        nv[j] = ld_at<float>(vb, s < nt ? voff + c * p.ldv : 0u);
+        nu[j >> 2][j & 3] = ld_at<float>(ub, s < nt ? s : nt - 1);
+      }
+      nA0 = ld_at<float>(Ab, r < nt ? r : nt - 1);
+      nA1 = ld_at<float>(Ab, 16 + r < nt ? 16 + r : nt - 1);
+      nAL = Ab[nt - 1];
     }
-    nA0 = Ah[t0 + (r < nt ? r : nt - 1)];
-    nA1 = Ah[t0 + (16 + r < nt ? 16 + r : nt - 1)];
-    nAL = Ah[t0 + nt - 1];
   };
   auto place = [](int x) { return (x & ~31) + ((x & 15) >> 2) * 8 + ((x >> 4) & 1) * 4 + (x & 3); };
   request(0);
   for (int t0 = 0; t0 < ql; t0 += kChunk) {
     const int nt = ql - t0 < kChunk ? ql - t0 : kChunk;
+    if (nt < kChunk || D < Dp) {  // uniform: rows and coordinates that do not exist are zeros
+#pragma unroll
+      for (int n = 0; n < NB; ++n)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (!piece[n] || 4 * ((n * 64 * NW + tid) / Q4) + j >= nt) nk[n][j] = nq[n][j] = zero4;
+    }
 #pragma unroll
     for (int n = 0; n < NB; ++n) {
       const int b = n * 64 * NW + tid;
@@ -349,12 +414,16 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
     }
     float v[8], u[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = nv[j], u[j] = nu[j];
+    for (int j = 0; j < 8; ++j) {
+      const bool in = nt == kChunk || 4 * g + (j & 3) + 16 * (j >> 2) < nt;
+      v[j] = is_norm ? (r == 0 && in ? 1.0f : 0.0f) : (col_on && in ? nv[j] : 0.0f);
+      u[j] = nu[j >> 2][j & 3];
+    }
     const float A0 = nA0, A1 = nA1, AL = nAL;
-    __syncthreads();
+    lds_barrier();
     if (t0 + kChunk < ql) request(t0 + kChunk);
     if (live) {
-      f32x4 O0 = f32x4{0.f, 0.f, 0.f, 0.f}, O1 = O0, s00 = O0, s01 = O0, s11 = O0;
+      f32x4 O0 = zero4, O1 = zero4, s00 = zero4, s01 = zero4, s11 = zero4;
 #pragma unroll
       for (int k = 0; k < NK; ++k) {
         const bf16x8 q0 = *reinterpret_cast<const bf16x8*>(qs + r * ldr + 32 * k + 8 * g);
@@ -374,23 +443,23 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
         O0 = mfma16x16x32(lo, q0, O0);
         O1 = mfma16x16x32(lo, q1, O1);
       }
-      const float e0 = expf(A0), e1 = expf(A1), eL = expf(AL);
+      const float e0 = exp2_hw(A0), e1 = exp2_hw(A1), eL = exp2_hw(AL);
       float P0[8], P1[8], vw[8];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         O0[i] *= e0;
         O1[i] *= e1;
         const bool seen = 4 * g + i <= r;
-        P0[i] = seen ? s00[i] * expf(A0 + u[i]) : 0.0f;
+        P0[i] = seen ? s00[i] * exp2_hw(A0 + u[i]) : 0.0f;
         P0[4 + i] = 0.0f;
-        P1[i] = s01[i] * expf(A1 + u[i]);
-        P1[4 + i] = seen ? s11[i] * expf(A1 + u[4 + i]) : 0.0f;
+        P1[i] = s01[i] * exp2_hw(A1 + u[i]);
+        P1[4 + i] = seen ? s11[i] * exp2_hw(A1 + u[4 + i]) : 0.0f;
       }
       bf16x8 vb, hi, lo;
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
         vb[j] = (bf16)v[j];
-        vw[j] = v[j] * expf(AL + u[j]);
+        vw[j] = v[j] * exp2_hw(AL + u[j]);
       }
       split8(P0, hi, lo);
       O0 = mfma16x16x32(vb, hi, O0);
@@ -414,7 +483,7 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
         const f32x4 o = b == 0 ? O0 : O1;
         const int t = 16 * b + r;
         if (t >= nt) continue;
-        const int64_t at = (row0 + t0 + t) * p.H + h;
+        const int64_t at = (int64_t)(row0 + t0 + t) * p.H + h;
         if (is_norm) {
           if (g == 0) p.nq[at] = o[0];
         } else if (V % 4 == 0) {
@@ -426,7 +495,7 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
         }
       }
     }
-    __syncthreads();  // the staged chunk has been read
+    lds_barrier();  // the staged chunk has been read
   }
 #pragma unroll
   for (int dt = 0; dt < 2 * NK; ++dt)
@@ -439,32 +508,63 @@ __global__ __launch_bounds__(64 * NW) void memory_chunk_kernel(MatrixMemoryParam
     }
 }
 
-// one wave per (row, head)
-template <typename T>
+// LP lanes per (row, head), VEC neighbouring coordinates per lane and step: the head stays in registers between the sum of
+// squares and the write
+template <typename T, int LP, int VEC, int STEPS>
 __global__ __launch_bounds__(256) void memory_out_kernel(MatrixMemoryParams p) {
-  const int lane = threadIdx.x & 63;
-  const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int lane = threadIdx.x % LP;
+  const int64_t item = (int64_t)blockIdx.x * (256 / LP) + threadIdx.x / LP;
   if (item >= (int64_t)p.rows * p.H) return;
   const int64_t row = p.row0 + item / p.H;
   const int h = (int)(item % p.H), V = p.V;
   const int64_t at = row * p.H + h;
   const float* o = p.num + at * V;
+  const float* gate = p.out_gate + row * p.ldg + h * V;
+  const float* w = p.norm_w + h * V;
+  float y[STEPS][VEC], gv[STEPS][VEC], wv[STEPS][VEC];
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const int c = (i * LP + lane) * VEC;
+    if (c < V) {
+      ld_vec<VEC>(o + c, y[i]);
+      ld_vec<VEC>(gate + c, gv[i]);
+      ld_vec<VEC>(w + c, wv[i]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) y[i][e] = 0.0f;
+    }
+  }
   const float inv_den = 1.0f / (fmaxf(fabsf(p.nq[at]), expf(-p.m[at])) + p.den_eps);
-  float y[8];
   float ss = 0.f;
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    y[i] = i * 64 + lane < V ? o[i * 64 + lane] * inv_den : 0.0f;
-    ss += y[i] * y[i];
-  }
-  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)V + p.eps) * p.out_scale;
-  const float* gate = p.out_gate + row * p.ldg + h * V;
+  for (int i = 0; i < STEPS; ++i)
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      y[i][e] *= inv_den;
+      ss += y[i][e] * y[i][e];
+    }
+#pragma unroll
+  for (int m = LP / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m);
+  const float inv = 1.0f / sqrtf(ss / (float)V + p.eps) * p.out_scale;
   T* out = reinterpret_cast<T*>(p.out) + row * p.ldo + h * V;
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    const int c = i * 64 + lane;
-    if (c < V) out[c] = (T)(y[i] * inv * p.norm_w[h * V + c] * sigmoid_f(gate[c]));
+  for (int i = 0; i < STEPS; ++i) {
+    const int c = (i * LP + lane) * VEC;
+    if (c >= V) continue;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) out[c + e] = (T)(y[i][e] * inv * wv[i][e] * sigmoid_f(gv[i][e]));
   }
+}
+
+template <typename T>
+void launch_out(const MatrixMemoryParams& p, hipStream_t st) {
+  const long long items = (long long)p.rows * p.H;
+  auto blocks = [&](int per) { return dim3((unsigned)((items + per - 1) / per)); };
+  const bool vec = p.V % 4 == 0 && p.ldg % 4 == 0 && reinterpret_cast<uintptr_t>(p.out_gate) % 16 == 0 &&
+                   reinterpret_cast<uintptr_t>(p.norm_w) % 16 == 0;
+  if (vec && p.V <= 128) hipLaunchKernelGGL((memory_out_kernel<T, 32, 4, 1>), blocks(8), dim3(256), 0, st, p);
+  else if (vec) hipLaunchKernelGGL((memory_out_kernel<T, 64, 4, 2>), blocks(4), dim3(256), 0, st, p);
+  else hipLaunchKernelGGL((memory_out_kernel<T, 64, 1, 8>), blocks(4), dim3(256), 0, st, p);
 }
 
 }  // namespace
@@ -488,18 +588,20 @@ extern "C" hipError_t dsse_matrix_memory_chunk(const dsse::MatrixMemoryParams* p
   if (p->nseq <= 0 || p->H <= 0 || p->rows <= 0) return hipSuccess;
   if (p->f32 || p->D < 1 || p->D > 256 || p->D % 4 || p->V < 1 || p->V > 512 || p->nseq > 65535 || p->H > 65535)
     return hipErrorInvalidValue;
-  hipLaunchKernelGGL(dsse::memory_gates_kernel, dim3(p->H, p->nseq), dim3(64), 0, st, *p);
+  hipLaunchKernelGGL(dsse::memory_gates_kernel, dim3(p->H, p->nseq), dim3(64 * dsse::kGateWaves), 0, st, *p);
   const int tiles = (p->V + 15) / 16 + 1;
   constexpr int NW = 4;
   const dim3 grid((tiles + NW - 1) / NW, p->H, p->nseq);
   switch ((p->D + 31) / 32) {
 #define DSSE_CHUNK_CASE(n) \
-  case n: hipLaunchKernelGGL((dsse::memory_chunk_kernel<n, NW>), grid, dim3(64 * NW), 0, st, *p); break;
+  case n:                                                                                                      \
+    if (p->vec) hipLaunchKernelGGL((dsse::memory_chunk_kernel<n, NW, true>), grid, dim3(64 * NW), 0, st, *p);  \
+    else hipLaunchKernelGGL((dsse::memory_chunk_kernel<n, NW, false>), grid, dim3(64 * NW), 0, st, *p);        \
+    break;
     DSSE_CHUNK_CASE(1) DSSE_CHUNK_CASE(2) DSSE_CHUNK_CASE(3) DSSE_CHUNK_CASE(4) DSSE_CHUNK_CASE(5) DSSE_CHUNK_CASE(6)
     DSSE_CHUNK_CASE(7) DSSE_CHUNK_CASE(8)
 #undef DSSE_CHUNK_CASE
   }
-  const long long items = (long long)p->rows * p->H;
-  hipLaunchKernelGGL(dsse::memory_out_kernel<bf16>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, *p);
+  dsse::launch_out<bf16>(*p, st);
   return hipGetLastError();
 }

@@ -452,6 +452,7 @@ def run_family_bench(model: str, device=None, streams: int = 16, prompt_len: int
     pf_s = pf[len(pf) // 2]
     r.active[:streams] = 1
     r.temperature[:streams] = 1.0
+    r.seeds[:streams, 0] = torch.arange(1, streams + 1, dtype=torch.int32)  # every stream draws its own tokens
     if cuda:
         r.capture([streams])
     for _ in range(warmup):

@@ -1050,7 +1050,7 @@ class LayeredRunner(RunnerBase):
             qa, ao = max(qa, a.heads * a.dim), max(ao, a.heads * a.vdim)
             if L.kind == "twin":
                 ao = max(ao, -(-(a.heads * a.vdim + m.right.heads * m.right.vdim) // 8) * 8)
-                mm = max(mm, ops.memory_work_floats(M, m.right.heads, m.right.vdim))
+                mm = max(mm, ops.memory_work_floats(M, m.right.heads, m.right.vdim, self.max_batch))
             if L.mlp is not None and not hasattr(L.mlp, "experts"):
                 ff = max(ff, L.mlp.ff)
         d = {"big": torch.zeros(M * big, **f32), "qa": torch.zeros(M * qa, **f32), "ao": torch.zeros(M * ao, **el),
@@ -1110,9 +1110,8 @@ class LayeredRunner(RunnerBase):
     def _qkv_rows(self, ri: int, a, big, taps, vdim: int, rope, temp, slots, qa, groups: list) -> None:
         """q to a buffer, k and v into this run's pages, per sequence group (prompt portions in tiles of rows)."""
         for g in groups:
-            ws, wt, qt = (g["ws"], g["wt"], 1) if g["qt"] == 1 else (g["hs"], g["ht"], SINK_ROWS_TILE)
-            ops.conv_qkv_rows(big, taps, self.state.tail.get(ri), g["qs"], g["ql"], g["ctx"], g["ss"], ws, wt, qt, a.heads,
-                              a.kv_heads, a.dim, vdim, rope, temp, slots, qa, self.kv.k[ri], self.kv.v[ri],
+            ops.conv_qkv_rows(big, taps, self.state.tail.get(ri), g["qs"], g["ql"], g["ctx"], g["ss"], g["ws"], g["wt"], g["qt"],
+                              a.heads, a.kv_heads, a.dim, vdim, rope, temp, slots, qa, self.kv.k[ri], self.kv.v[ri],
                               self.kv.vt.get(ri))
 
     def _conv_attention_bracket(self, ri: int, m, Lw, M: int, d: dict, pos, slots, groups: list) -> None:

@@ -478,9 +478,10 @@ def memory_chunk_ok(dtype, dim: int, vdim: int) -> bool:
     return dtype == torch.bfloat16 and dim <= 256 and dim % 4 == 0
 
 
-def memory_work_floats(rows: int, heads: int, vdim: int) -> int:
-    """fp32 words of the MFMA form's work area: read-outs, normaliser products, running maxima and two gate sums."""
-    return rows * heads * (vdim + 4)
+def memory_work_floats(rows: int, heads: int, vdim: int, seqs: int) -> int:
+    """fp32 words of the MFMA form's work area: read-outs, normaliser products, running maxima and two gate sums (whose
+    rows start every sequence at a multiple of four)."""
+    return rows * heads * (vdim + 2) + 8 + 2 * heads * (rows + 4 * seqs + 8)
 
 
 def matrix_memory(q, k, v, gates, gate_b, cap: float, state, norm, q_start, q_len, ctx_len, state_slot, out_gate, norm_w,

@@ -37,11 +37,10 @@ def short_conv(u, taps):
     """y[t] = sum_j taps[:, j] u[t - K + 1 + j] per channel; nothing before the start."""
     T, K = u.shape[0], taps.shape[1]
     y = torch.zeros_like(u)
-    for t in range(T):
-        for j in range(K):
-            s = t - K + 1 + j
-            if s >= 0:
-                y[t] = y[t] + taps[:, j] * u[s]
+    for j in range(K):
+        back = K - 1 - j
+        if back < T:
+            y[back:] = y[back:] + taps[:, j] * u[:T - back]
     return y
 
 
@@ -81,13 +80,13 @@ def sink_softmax(q, k, v, scale: float, sink):
     """Causal attention of q [T, H, D] over k [T, G, D], v [T, G, V]; exp(sink[h]) joins head h's denominator."""
     T, H, G = q.shape[0], q.shape[1], k.shape[1]
     o = torch.zeros(T, H, v.shape[2], dtype=q.dtype)
+    unseen = torch.arange(T)[None, :] > torch.arange(T)[:, None]
     for h in range(H):
         g = h // (H // G)
-        for t in range(T):
-            s = (k[:t + 1, g] @ q[t, h]) * scale
-            top = max(float(s.max()), float(sink[h]))
-            e = torch.exp(s - top)
-            o[t, h] = (e @ v[:t + 1, g]) / (e.sum() + torch.exp(sink[h] - top))
+        s = ((q[:, h] @ k[:, g].T) * scale).masked_fill(unseen, float("-inf"))
+        top = torch.maximum(s.max(-1, keepdim=True).values, sink[h])
+        e = torch.exp(s - top)
+        o[:, h] = (e @ v[:, g]) / (e.sum(-1, keepdim=True) + torch.exp(sink[h] - top))
     return o
 
 
@@ -117,18 +116,20 @@ def warm_attention(h, m: dict, w: dict):
 
 
 def matrix_memory(q, k, v, ig, fg):
-    """One head: q, k [T, D], v [T, V], log gates ig, fg [T] -> read-outs [T, V]; the running maximum starts at zero."""
-    T, D, V = k.shape[0], k.shape[1], v.shape[1]
-    S, n, m = torch.zeros(D, V, dtype=k.dtype), torch.zeros(D, dtype=k.dtype), torch.zeros((), dtype=k.dtype)
-    o = torch.zeros(T, V, dtype=k.dtype)
+    """q, k [T, H, D], v [T, H, V], log gates ig, fg [T, H] -> read-outs [T, H, V]; the running maximum starts at zero."""
+    T, H, D = k.shape
+    S = torch.zeros(H, D, v.shape[2], dtype=k.dtype)
+    n, m = torch.zeros(H, D, dtype=k.dtype), torch.zeros(H, dtype=k.dtype)
+    out = torch.zeros_like(v)
     for t in range(T):
         new = torch.maximum(fg[t] + m, ig[t])
         keep, put = torch.exp(fg[t] + m - new), torch.exp(ig[t] - new)
-        S = keep * S + put * torch.outer(k[t], v[t])
-        n = keep * n + put * k[t]
+        S = keep[:, None, None] * S + put[:, None, None] * (k[t][:, :, None] * v[t][:, None, :])
+        n = keep[:, None] * n + put[:, None] * k[t]
         m = new
-        o[t] = (S.T @ q[t]) / (torch.maximum((n @ q[t]).abs(), torch.exp(-m)) + 1e-6)
-    return o
+        den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+        out[t] = torch.einsum("hdv,hd->hv", S, q[t]) / den[:, None]
+    return out
 
 
 def memory_mixer(h, m: dict, w: dict, eps: float):
@@ -138,8 +139,7 @@ def memory_mixer(h, m: dict, w: dict, eps: float):
     k, v = (h @ w["k"].T).view(T, H, D), (h @ w["v"].T).view(T, H, V)
     ig = cap * torch.tanh((h @ w["i"].T + w["i.b"]) / cap)
     fg = torch.nn.functional.logsigmoid(cap * torch.tanh((h @ w["f"].T + w["f.b"]) / cap))
-    o = torch.stack([matrix_memory(q[:, n], k[:, n], v[:, n], ig[:, n], fg[:, n]) for n in range(H)], dim=1)
-    o = rms(o, eps).reshape(T, H * V) * w["norm"]
+    o = rms(matrix_memory(q, k, v, ig, fg), eps).reshape(T, H * V) * w["norm"]
     return (o * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
 
 
@@ -188,7 +188,9 @@ def forward(cfg: dict, weights: dict, tokens, trace: list | None = None):
     tokens = torch.as_tensor(tokens, dtype=torch.long)
     x = w["embed"][tokens] * float((cfg.get("embedding") or {}).get("scale", 1.0))
     for i, L in enumerate(cfg["layers"]):
-        owner = i if L.get("weights_of") is None else int(L["weights_of"])
+        owner = i
+        while cfg["layers"][owner].get("weights_of") is not None:  # the layer that has the tensors
+            owner = int(cfg["layers"][owner]["weights_of"])
         x = layer(x, L, sub(w, f"l{owner}."), eps, tokens)
         if trace is not None:
             trace.append(x.clone())

@@ -1,0 +1,911 @@
+"""Lobidra on the engine against the plain oracle (tests/lobidra_oracle.py).
+
+Every test builds its own small configuration and random weights, drives the engine through its own entry points
+(LLMEngine.force_step for given tokens, add_request + step for generation) and compares the logits with the oracle's
+whole-sequence forward in float64.  The same tests run on the CPU (PyTorch reference ops: scheduler, cache, state and
+batch plumbing) and, marked ``gpu``, on the HIP kernels in fp32 (every row, tight tolerance) and bf16.  Where a test
+asserts that something matters, the mistake is planted in the oracle.
+"""
+from __future__ import annotations
+
+import copy
+import json
+import math
+
+import pytest
+import torch
+
+import lobidra_oracle as oracle
+from distributed_sse_for_llm_response_amd import ops
+from distributed_sse_for_llm_response_amd.engine.engine import LLMEngine, SamplingParams
+from distributed_sse_for_llm_response_amd.engine.model_runner import PrefillSeq
+from distributed_sse_for_llm_response_amd.engine.weights import convert_lobidra
+from distributed_sse_for_llm_response_amd.models import registry
+from distributed_sse_for_llm_response_amd.models.lobidra import (BandScaling, LobidraConfig, PairRotarySpec, QueryTemperature,
+                                                                 init_weights, tensor_shapes)
+
+GPU = pytest.param("cuda", marks=pytest.mark.gpu)
+DEVICES = ["cpu", GPU]
+VOCAB = 53
+SCALED = {"base": 5000.0, "dims": 6, "scaling": {"factor": 4.0, "low": 1.0, "high": 4.0, "original": 64}}
+
+
+def moe(experts=5, top=2, ff=9, shared=7):
+    f = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    if shared:
+        f["shared"] = {"ff": shared}
+    return f
+
+
+def dense(ff=21):
+    return {"kind": "dense", "ff": ff}
+
+
+def att(heads=4, kv_heads=2, dim=10, conv=4, scale=0.4, rot=SCALED, mlp=None, weights_of=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": scale}
+    if conv:
+        m["conv"] = conv
+    if rot:
+        m["rot"] = dict(rot)
+    e = {"type": "attention", "mixer": m, "mlp": mlp}
+    if weights_of is not None:
+        e["weights_of"] = weights_of
+    return e
+
+
+def par(heads=4, kv_heads=2, dim=8, vdim=6, scale=0.4, temp=(0.5, 8), mheads=3, mdim=12, mvdim=10, cap=6.0, ls=0.8, rs=1.3,
+        mlp=None, weights_of=None):
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale}
+    if temp:
+        left["q_temp"] = {"coef": temp[0], "every": temp[1]}
+    e = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": left, "right": {"heads": mheads, "dim": mdim, "vdim": mvdim, "gate_cap": cap}, "left_scale": ls,
+        "right_scale": rs}}
+    if weights_of is not None:
+        e["weights_of"] = weights_of
+    return e
+
+
+def config(layers, width=26, vocab=VOCAB, eps=3e-6, scale=3.0):
+    return {"architecture": "Lobidra", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "embedding": {"scale": scale}, "layers": copy.deepcopy(layers)}
+
+
+STACK = config([att(mlp=dense()), par(mlp=moe()), att(heads=3, kv_heads=3, dim=8, conv=2, rot=None, mlp=moe(top=1, shared=0)),
+                par(heads=3, kv_heads=1, dim=9, vdim=7, temp=None, mheads=2, mdim=10, mvdim=16, mlp=None),
+                par(mlp=moe(), weights_of=1), att(mlp=dense(), weights_of=0)], width=40)
+
+
+class Model:
+    """Configuration + random weights + an engine on `device` in `dtype`."""
+
+    def __init__(self, cfg_dict, device, dtype=torch.float32, seed=0, max_tokens=256, max_seqs=4, tweak=None):
+        self.cfg_dict = cfg_dict
+        self.cfg = LobidraConfig.from_dict(cfg_dict)
+        self.weights = init_weights(self.cfg, seed=seed)
+        if tweak:
+            tweak(self.weights)
+        self.device, self.dtype = torch.device(device), dtype
+        w = convert_lobidra(self.cfg, self.weights, device=self.device, dtype=dtype)
+        fam = registry.family_of(self.cfg)
+        assert fam.name == "lobidra"
+        self.runner = registry.make_runner(fam, w, num_blocks=-(-max_tokens // 32), max_batch=max_seqs,
+                                           max_model_len=max_tokens, max_prefill_tokens=max_tokens, device=self.device,
+                                           use_graphs=False)
+        self.engine = LLMEngine(self.runner, eos_id=-1)
+        self.engine.watermark = 0
+
+    def expect(self, tokens, cfg_dict=None, weights=None):
+        return oracle.forward(cfg_dict or self.cfg_dict, weights or self.weights, tokens).float()
+
+    def check(self, got, want, what=""):
+        """Row-wise: rms of the difference (mean taken off) over the rms of the expected logits.  fp32 judges every row,
+        bf16 nine rows in ten (all but one of a few), the median and, loosely, every row."""
+        got, want = got.detach().float().cpu(), want.float()
+        assert got.shape == want.shape, (got.shape, want.shape)
+        assert torch.isfinite(got).all(), what
+        d = got - want
+        d = d - d.mean(-1, keepdim=True)
+        err = d.pow(2).mean(-1).sqrt() / (want - want.mean(-1, keepdim=True)).pow(2).mean(-1).sqrt().clamp_min(1e-6)
+        if self.dtype == torch.float32:
+            assert float(err.max()) < 2e-4, f"{what}: worst row {int(err.argmax())} error {float(err.max()):.3g}"
+        else:
+            off = int((err >= 4e-2).sum())
+            assert off <= max(1, err.numel() // 10) and float(err.max()) < 0.15 and float(err.median()) < 2e-2, \
+                f"{what}: median {float(err.median()):.3g}, {off} of {err.numel()} rows off, worst {float(err.max()):.3g}"
+
+    def run_cut(self, cid, tokens, cuts, end=True):
+        """Feed `tokens` in portions of the given sizes (the last size repeats), all logits wanted."""
+        out, at, k = [], 0, 0
+        while at < len(tokens):
+            n = min(cuts[min(k, len(cuts) - 1)], len(tokens) - at)
+            last = at + n == len(tokens)
+            out.append(self.engine.force_step([(cid, tokens[at:at + n], list(range(n)))], [cid] if last and end else []))
+            at, k = at + n, k + 1
+        return torch.cat(out)
+
+
+def toks(n, vocab=VOCAB, seed=0):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randint(0, vocab, (n,), generator=g).tolist()
+
+
+def modes(device):
+    return [torch.float32] if device == "cpu" else [torch.float32, torch.bfloat16]
+
+
+def rel_err(a, b, rows=slice(None)):
+    a, b = a[rows], b[rows]
+    return (a - b).pow(2).mean(-1).sqrt() / b.pow(2).mean(-1).sqrt().clamp_min(1e-6)
+
+
+def gap(a, b, rows=slice(None)):
+    """Median over rows: how far a variant of the design is from the design."""
+    return float(rel_err(a, b, rows).median())
+
+
+def gap_max(a, b, rows=slice(None)):
+    return float(rel_err(a, b, rows).max())
+
+
+def changed(weights, fn):
+    """A copy of the weights with fn(name, tensor) -> tensor or None (unchanged) applied."""
+    out = {}
+    for k, v in weights.items():
+        r = fn(k, v)
+        out[k] = v if r is None else r
+    return out
+
+
+def tweak_of(fn):
+    def tweak(w):
+        w.update(changed(w, fn))
+    return tweak
+
+
+# ---------------------------------------------------------------------------------------------- mechanisms alone
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name,cfgd", [
+    ("convolved attention, scaled rotation", config([att()])),
+    ("a key head per head, plain rotation of the whole head", config([att(heads=3, kv_heads=3, dim=8, rot={"base": 100.0, "dims": 8})])),
+    ("one key head, no rotation", config([att(heads=5, kv_heads=1, rot=None)])),
+    ("no convolution", config([att(conv=0)])),
+    ("one tap", config([att(conv=1)])),
+    ("two taps", config([att(conv=2)])),
+    ("three taps", config([att(conv=3)])),
+    ("more taps than the kernel keeps in registers", config([att(conv=7)])),
+    ("one-wide heads", config([att(heads=2, kv_heads=1, dim=1, rot=None)])),
+    ("odd head width", config([att(heads=2, kv_heads=2, dim=7, rot={"base": 50.0, "dims": 4})])),
+    ("attention beside a matrix memory", config([par()])),
+    ("no query temperature, other scales", config([par(temp=None, ls=-0.5, rs=0.25)])),
+    ("one-wide attention, one-wide memory", config([par(heads=2, kv_heads=1, dim=1, vdim=1, mheads=1, mdim=1, mvdim=1)])),
+    ("memory heads wider than the attention's", config([par(heads=2, kv_heads=2, mheads=2, mdim=24, mvdim=36)])),
+    ("dense feed-forward", config([att(heads=1, kv_heads=1, mlp=dense())])),
+    ("table-routed experts with a shared one", config([att(heads=1, kv_heads=1, mlp=moe())])),
+    ("one expert per token, no shared one", config([att(mlp=moe(top=1, shared=0))])),
+    ("every expert", config([att(mlp=moe(experts=4, top=4))])),
+    ("a single expert", config([att(mlp=moe(experts=1, top=1))])),
+    ("shared expert wider than the routed ones", config([att(mlp=moe(ff=3, shared=31))])),
+    ("another layer's tensors, both kinds", config([att(mlp=dense()), par(mlp=moe()), par(mlp=moe(), weights_of=1),
+                                                    att(mlp=dense(), weights_of=0)])),
+    ("a chain of borrowed tensors, and a lender behind its borrower", config(
+        [att(weights_of=2, mlp=moe()), par(), att(mlp=moe()), att(weights_of=0, mlp=moe())])),
+    ("embedding without a scale", {k: v for k, v in config([att(mlp=moe())]).items() if k != "embedding"}),
+])
+def test_mechanism_alone(device, name, cfgd):
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype)
+        t = toks(47, seed=1)
+        m.check(m.run_cut("a", t, [len(t)]), m.expect(t), name + ", whole")
+        m.check(m.run_cut("b", t, [9, 1]), m.expect(t), name + ", decoding")
+
+
+def test_each_op_against_its_oracle_function():
+    """The reference ops the CPU engine runs on, one mechanism at a time, against the oracle's functions."""
+    g = torch.Generator().manual_seed(5)
+    i32 = lambda *x: torch.tensor(x, dtype=torch.int32)  # noqa: E731
+    meta = (i32(0), i32(13), i32(13), i32(1))  # one sequence of 13 rows in slot 1
+    T, H, G, D = 13, 4, 2, 10
+    # convolution, rotation, pages: values are the keys before their rotation
+    x, taps = torch.randn(T, (H + G) * D + 5, generator=g), torch.randn((H + G) * D, 3, generator=g)
+    rot = PairRotarySpec.from_dict(SCALED)
+    q, kc, vc, vt = torch.zeros(T, H, D), torch.zeros(2, 32, G, D), torch.zeros(2, 32, G, D), torch.zeros(2, G, D, 32)
+    rows = torch.arange(30, 43, dtype=torch.int32)
+    tail = torch.zeros(2, 2, (H + G) * D)
+    ops.conv_qkv_rows(x, taps, tail, *meta, i32(0), i32(0), 16, H, G, D, 0, rot.table(20), None, rows, q, kc, vc, vt)
+    y = oracle.short_conv(x[:, :(H + G) * D].double(), taps.double())
+    want_q, k = oracle.rotate(y[:, :H * D].view(T, H, D), SCALED), y[:, H * D:].view(T, G, D)
+    assert torch.allclose(q, want_q.float(), atol=1e-4)
+    assert torch.allclose(kc.view(64, G, D)[30:43], oracle.rotate(k, SCALED).float(), atol=1e-4)
+    assert torch.allclose(vc.view(64, G, D)[30:43], k.float(), atol=1e-4)
+    assert torch.equal(tail[1], x[-2:, :(H + G) * D]) and not tail[0].any()
+    # queries times their position's factor, values of their own
+    x = torch.randn(T, H * D + G * (D + 6), generator=g)
+    vc, temp = torch.zeros(2, 32, G, 6), QueryTemperature(0.7, 3.0)
+    ops.conv_qkv_rows(x, None, None, *meta, i32(0), i32(0), 16, H, G, D, 6, None, temp.table(20), rows, q, kc, vc)
+    f = torch.tensor([oracle.temperature(p, {"coef": 0.7, "every": 3}) for p in range(T)])
+    assert torch.allclose(q, x[:, :H * D].view(T, H, D) * f[:, None, None], atol=1e-5)
+    assert torch.equal(vc.view(64, G, 6)[30:43], x[:, (H + G) * D:].view(T, G, 6))
+    # matrix memory with its output norm and gate
+    V, cap = 7, 3.0
+    q, k, v = (torch.randn(T, H, n, generator=g) for n in (D, D, V))
+    gates, gb = torch.randn(T, 2 * H, generator=g) * 4, torch.randn(2 * H, generator=g)
+    og, nw = torch.randn(T, H * V, generator=g), torch.randn(H * V, generator=g)
+    state, norm, out = torch.ones(2, H, D, V), torch.ones(2, H, D + 1), torch.zeros(T, H * V)
+    ops.matrix_memory(q, k, v, gates, gb, cap, state, norm, *meta, og, nw, 1e-5, 1e-6, 0.3, 1.7, out)
+    z = cap * torch.tanh((gates + gb).double() / cap)
+    o = oracle.matrix_memory(q.double() * 0.3, k.double(), v.double(), z[:, :H], torch.nn.functional.logsigmoid(z[:, H:]))
+    want = oracle.rms(o, 1e-5).reshape(T, H * V) * nw.double() * torch.sigmoid(og.double()) * 1.7
+    assert torch.allclose(out, want.float(), atol=1e-4)
+    # constant and learned sinks, scaled outputs in a wider row
+    kc, vc = torch.randn(1, 32, G, D, generator=g), torch.randn(1, 32, G, 6, generator=g)
+    wide, sink = torch.zeros(T, H * 6 + 3), torch.randn(H, generator=g)
+    ops.sink_attention(q, kc, vc, torch.zeros(1, 1, dtype=torch.int32), *meta[:3], i32(0), i32(0), sink, None,
+                       wide[:, :H * 6].unflatten(1, (H, 6)), 2 ** 31 - 1, 0.3, 4, out_scale=-2.0)
+    want = -2.0 * oracle.sink_softmax(q.double(), kc[0, :T].double(), vc[0, :T].double(), 0.3, sink.double()).reshape(T, -1)
+    assert torch.allclose(wide[:, :H * 6], want.float(), atol=1e-4) and not wide[:, H * 6:].any()
+    # gelu rows; the experts of a token id
+    up, act = torch.randn(5, 9, generator=g) * 3, torch.zeros(5, 9)
+    ops.act_rows(up, act, 3)
+    assert torch.allclose(act, oracle.gelu_tanh(up.double()).float(), atol=1e-5)
+    table = torch.randint(0, 9, (VOCAB, 2), generator=g, dtype=torch.int32)
+    idx = torch.zeros(4, 2, dtype=torch.int32)
+    ops.moe_table_lists(i32(3, 52, 0, 3), [table], [9], [True], [idx], [None], [None], [None])
+    assert torch.equal(idx, table[torch.tensor([3, 52, 0, 3])])
+
+
+def test_frequencies_and_factors():
+    """Every band of the frequency scaling, and the query factor's steps, against the oracle's functions."""
+    for rot in (SCALED, {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}},
+                {"base": 60.0, "dims": 12, "scaling": {"factor": 3.0, "low": 0.5, "high": 6.0, "original": 60}}, {"base": 7.0, "dims": 4}):
+        spec = PairRotarySpec.from_dict(rot)
+        f = oracle.frequencies(rot)
+        assert torch.allclose(spec.frequencies(), f, rtol=1e-12, atol=0)
+        if "scaling" in rot:
+            plain = oracle.frequencies({k: v for k, v in rot.items() if k != "scaling"})
+            kept, slowed = int((f == plain).sum()), int(torch.isclose(f, plain / rot["scaling"]["factor"]).sum())
+            assert kept >= 1 and slowed >= 1, rot
+        assert torch.allclose(spec.table(33)[32, :, 0], torch.cos(32 * f).float(), atol=1e-6)
+        assert PairRotarySpec.from_dict(spec.to_dict()) == spec
+    assert PairRotarySpec.from_dict({"base": 10.0, "dims": 0}) is None and PairRotarySpec.from_dict(None) is None
+    assert PairRotarySpec(8, 10.0, BandScaling(2.0, 1.0, 4.0, 30.0)) != PairRotarySpec(8, 10.0)
+    for every in (1, 3, 8, 100):
+        t = QueryTemperature(0.4, every).table(500)
+        assert torch.allclose(t, torch.tensor([oracle.temperature(p, {"coef": 0.4, "every": every}) for p in range(500)]), atol=1e-6)
+        if every > 1:
+            assert t[every - 2] == 1.0 and t[every - 1] > 1.0  # the step comes with position every - 1
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_layer_trace(device):
+    """The engine's layer trace (the stream after every layer) against the oracle's."""
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype)
+        t = toks(21, seed=2)
+        got, want = [], []
+        m.runner.prefill([PrefillSeq(slot=0, tokens=t, start_pos=0, block_table=[0], last_chunk=False)], 0, trace=got)
+        oracle.forward(m.cfg_dict, m.weights, t, want)
+        assert len(got) == len(want) == 6
+        for i, (a, b) in enumerate(zip(got, want)):
+            err = (a.cpu().double() - b).abs().amax(-1) / b.abs().max()
+            assert float(err.max()) < (1e-4 if dtype == torch.float32 else 4e-2), f"layer {i}"
+
+
+# ---------------------------------------------------------------------------------------------- cuts, batches, pools
+@pytest.mark.parametrize("device", DEVICES)
+def test_prefill_against_token_by_token(device):
+    t = toks(75, seed=3)
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype)
+        want = m.expect(t)
+        whole = m.run_cut("w", t, [len(t)])
+        single = m.run_cut("s", t, [1])
+        m.check(whole, want, "whole prompt")
+        m.check(single, want, "token by token")
+        if dtype == torch.float32:
+            m.check(single, whole.cpu(), "token by token against the whole prompt")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("cuts", [[2], [3, 2, 7], [5, 1, 1, 2, 11], [31, 2, 1], [33, 1], [64, 2], [32, 32, 6]])
+def test_portions(device, cuts):
+    """Portions cut inside pages, chunks and the convolutions' reach, down to two tokens (shorter than a tail)."""
+    t = toks(70, seed=4)
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype)
+        m.check(m.run_cut("p", t, cuts), m.expect(t), f"portions {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_unequal_batch_against_each_alone(device):
+    """Four requests of unequal length in one batch: portions of some beside single tokens of others, one sits out
+    steps, one ends early and its slot and pages go to a newcomer."""
+    seqs = {"a": toks(50, seed=5), "b": toks(9, seed=6), "c": toks(34, seed=7), "d": toks(1, seed=8), "e": toks(40, seed=9)}
+    plan = [{"a": 7, "b": 2, "c": 20}, {"a": 1, "b": 1, "d": 1}, {"a": 1, "c": 2, "b": 1}, {"a": 30, "b": 1, "e": 3},
+            {"a": 1, "b": 1, "c": 1, "e": 33}, {"a": 1, "b": 1, "c": 11, "e": 1}, {"a": 9, "b": 2, "e": 3}]
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype, max_tokens=256)
+        at = {k: 0 for k in seqs}
+        got = {k: [] for k in seqs}
+        for step in plan:
+            entries, end = [], []
+            for k, n in step.items():
+                n = min(n, len(seqs[k]) - at[k])
+                entries.append((k, seqs[k][at[k]:at[k] + n], list(range(n))))
+                at[k] += n
+                if at[k] == len(seqs[k]):
+                    end.append(k)
+            out = m.engine.force_step(entries, end)
+            o = 0
+            for k, tk, _ in entries:
+                got[k].append(out[o:o + len(tk)])
+                o += len(tk)
+        for k, t in seqs.items():
+            assert at[k] == len(t), k
+            m.check(torch.cat(got[k]), m.expect(t), f"request {k} in the batch")
+        assert m.engine.alloc.num_free == m.engine.alloc.num_blocks
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_pages_and_slots_used_again(device):
+    """A pool of three pages and two slots: every later request runs in pages and slots that held another one, in
+    prompts and in decoding; nothing of the old state, tail or pages shows."""
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype, max_tokens=96, max_seqs=2)
+        for i, (n, cuts) in enumerate([(60, [60]), (64, [33, 1]), (40, [2, 30, 1]), (64, [64]), (5, [1])]):
+            t = toks(n, seed=30 + i)
+            keep = toks(20, seed=40 + i)
+            first = m.engine.force_step([(f"k{i}", keep[:10], list(range(10)))])
+            got = m.run_cut(f"r{i}", t, cuts)
+            rest = m.engine.force_step([(f"k{i}", keep[10:], list(range(10)))], [f"k{i}"])
+            m.check(got, m.expect(t), f"request {i}")
+            m.check(torch.cat([first, rest]), m.expect(keep), f"neighbour of request {i}")
+        assert m.engine.alloc.num_free == m.engine.alloc.num_blocks
+    m.engine.force_step([("held", toks(64, seed=1), [])])
+    with pytest.raises(MemoryError):
+        m.engine.force_step([("late", toks(64, seed=2), [])])
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_state_follows_a_moved_slot(device):
+    """Slot compaction moves the matrix, the normaliser, its maximum and the convolution tails of a live sequence."""
+    t = toks(30, seed=31)
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype, max_seqs=3)
+        first = m.engine.force_step([("x", toks(12, seed=32), []), ("a", t[:20], list(range(20)))])
+        r = m.runner
+        for group in (r.state.state, r.state.norm, r.state.tail):
+            for v in group.values():
+                v[2] = 7.0
+        src = m.engine.slots.index(next(s for s in m.engine.slots if s is not None and s.conversation_id == "a"))
+        before = {k: v[src].clone() for k, v in r.state.norm.items()}
+        r.move_slots([src], [2])
+        for k, v in r.state.norm.items():
+            assert torch.equal(v[2], before[k]), k
+        r.move_slots([2], [src])
+        rest = m.engine.force_step([("a", t[20:], list(range(10)))], ["a"])
+        m.check(torch.cat([first, rest]), m.expect(t), "after the slot was moved and moved back")
+
+
+# ---------------------------------------------------------------------------------------------- far keys and edges
+def marked(w, cols, token, scale=30.0):
+    """Embedding rows whose first coordinate is a constant and whose second one only `token` has."""
+    e = w["embed"].float()
+    e[:, 0], e[:, 1] = 4.0, 0.0
+    e[token] *= 0.3
+    e[token, 1] = scale
+    w["embed"] = e.to(torch.bfloat16)
+    for k in list(w):
+        if k.endswith("norm1"):
+            w[k] = torch.zeros_like(w[k])
+
+
+WIDTHS = [10, 32]  # head widths of the row form and of the MFMA form
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dim", WIDTHS)
+def test_far_key_among_hundreds(device, dim):
+    """Every query points at the key of one token that occurs once, as the sequence's second: one far key carries the
+    weight.  Another token in its place moves the logits 250 tokens later in the oracle, and the engine agrees with it in
+    prompts cut at page borders and in decoding; in both kinds of attention."""
+    for kind in ("attention", "parallel"):
+        if kind == "attention":
+            cfgd = config([att(heads=2, kv_heads=1, dim=dim, conv=3, scale=1.0, rot={"base": 100.0, "dims": 4})], width=40)
+            q, k, o = "l0.mix.q", "l0.mix.k", "l0.mix.o"
+        else:
+            cfgd = config([par(heads=2, kv_heads=1, dim=dim, vdim=16, scale=1.0, temp=(0.1, 50), ls=2.0, rs=0.3)], width=40)
+            q, k, o = "l0.mix.left.q", "l0.mix.left.k", "l0.mix.left.o"
+
+        def planted(w):
+            marked(w, 40, VOCAB - 1)
+            wq, wk = torch.zeros_like(w[q]).float(), w[k].float() * 0.05
+            wq.view(2, dim, 40)[:, dim - 3:, 0] = 3.0        # a constant query in coordinates that do not turn
+            wk[:, 1] = 0.0
+            wk[dim - 3:, 1] = 3.0
+            w[q], w[k], w[o] = wq.to(torch.bfloat16), wk.to(torch.bfloat16), (w[o].float() * 3).to(torch.bfloat16)
+            for n in ("q", "k"):
+                if f"l0.mix.{n}.conv" in w:
+                    c = torch.zeros_like(w[f"l0.mix.{n}.conv"])
+                    c[:, -1] = 1.0
+                    w[f"l0.mix.{n}.conv"] = c
+
+        t = toks(300, vocab=VOCAB - 1, seed=10)
+        t[1] = VOCAB - 1
+        for dtype in modes(device):
+            m = Model(cfgd, device, dtype, max_tokens=320, tweak=planted)
+            want = m.expect(t)
+            moved = list(t)
+            moved[1] = 7
+            assert gap(m.expect(moved), want, slice(250, None)) > 5e-2, "the far key does not matter in this construction"
+            m.check(m.run_cut("a", t, [256, 1]), want, kind + ": prompt to a page border, then decoding")
+            m.check(m.run_cut("b", t, [32, 64, 33, 2, 97, 1]), want, kind + ": portions on and off page borders")
+
+
+def sharp(k, v):
+    """Projections of q and k that make the scores stand out, and mixers that count three times as much in the stream."""
+    if k.endswith((".q", ".k")):
+        return (v.float() * 1.8).to(v.dtype)
+    return (v.float() * 3).to(v.dtype) if k.endswith(("mix.o", "left.o", "right.o")) else None
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dim", WIDTHS)
+def test_rotation_and_its_scaling(device, dim, monkeypatch):
+    """Sharp attention over 130 tokens, pages and decoding: the oracle without the frequency scaling, with another band
+    limit, with half the pairs, with positions that start at one on the keys, or with values that turn too, is far away."""
+    rot = {"base": 300.0, "dims": 8, "scaling": {"factor": 6.0, "low": 1.0, "high": 3.0, "original": 120}}
+
+    def cfg_r(r):
+        return config([att(heads=2, kv_heads=1, dim=dim, conv=2, scale=2.0 / math.sqrt(dim), rot=r)], width=40)
+
+    t = toks(130, seed=11)
+    for dtype in modes(device):
+        m = Model(cfg_r(rot), device, dtype, tweak=tweak_of(sharp))
+        want = m.expect(t)
+        for other in ({**rot, "scaling": None}, {**rot, "scaling": {**rot["scaling"], "high": 6.0}}, {**rot, "dims": 4},
+                      {**rot, "scaling": {**rot["scaling"], "factor": 3.0}}):
+            assert gap(m.expect(t, cfg_r(other)), want, slice(40, None)) > 1e-2, other
+        with monkeypatch.context() as mp:
+            plain, calls = oracle.sink_softmax, []
+            mp.setattr(oracle, "sink_softmax", lambda q, k, v, s, z: plain(q, k, k, s, z))
+            assert gap(m.expect(t), want) > 1e-2, "values that turn"
+        m.check(m.run_cut("w", t, [len(t)]), want, "prompt")
+        m.check(m.run_cut("d", t, [96, 1]), want, "decoding from a page's border")
+        m.check(m.run_cut("c", t, [2, 33, 31, 2, 1]), want, "portions")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_sinks(device, monkeypatch):
+    """Small scores and few keys: the constant sink takes much of the first rows' weight, a learned sink differs per head.
+    The oracle without a sink, with a sink that the score's scale touches, or with the heads' sinks exchanged is far
+    away; first rows as prompt, as portions and one by one."""
+    cfgd = config([att(heads=4, kv_heads=2, dim=8, scale=0.1), par(heads=4, kv_heads=2, dim=32, vdim=16, scale=0.1, ls=2.0)], width=40)
+
+    def heavy(k, v):
+        return (torch.tensor([4.0, -3.0, 1.5, 0.0])).to(v.dtype) if k.endswith("sink") else None
+
+    t = toks(40, seed=12)
+    plain = oracle.sink_softmax
+    variants = {
+        "none": lambda q, k, v, s, z: plain(q, k, v, s, torch.full_like(z, -1e30)),
+        "scaled": lambda q, k, v, s, z: plain(q, k, v, s, z * s),
+        "exchanged": lambda q, k, v, s, z: plain(q, k, v, s, z.flip(0)),
+        "constant left out": lambda q, k, v, s, z: plain(q, k, v, s, torch.where((z == 0).all(), torch.full_like(z, -1e30), z)),
+    }
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype, tweak=tweak_of(heavy))
+        want = m.expect(t)
+        for name, fn in variants.items():
+            with monkeypatch.context() as mp:
+                mp.setattr(oracle, "sink_softmax", fn)
+                assert gap_max(m.expect(t), want, slice(0, 6)) > 5e-3, name
+        m.check(m.run_cut("w", t, [len(t)]), want, "prompt")
+        m.check(m.run_cut("d", t, [1]), want, "one by one")
+        m.check(m.run_cut("c", t, [2]), want, "twos")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_query_temperature_steps(device, monkeypatch):
+    """A step at every eighth token: the oracle that counts from position 0, or leaves the factor out, is far away right at
+    the steps; the step comes inside portions, at their starts and in decoding."""
+    cfgd = config([par(heads=2, kv_heads=1, dim=32, vdim=16, scale=0.3, temp=(2.0, 8), ls=2.0, rs=0.3)], width=40)
+    t = toks(60, seed=13)
+    plain = oracle.temperature
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype, tweak=tweak_of(sharp))
+        want = m.expect(t)
+        with monkeypatch.context() as mp:
+            mp.setattr(oracle, "temperature", lambda p, c: plain(p - 1, c))
+            late = rel_err(m.expect(t), want)
+            assert float(late[15]) > 1e-2 and float(late[23]) > 1e-3, "one position late"
+            mp.setattr(oracle, "temperature", lambda p, c: 1.0)
+            assert gap(m.expect(t), want, slice(8, None)) > 1e-2
+        m.check(m.run_cut("w", t, [len(t)]), want, "prompt")
+        m.check(m.run_cut("d", t, [6, 1]), want, "decoding over the steps")
+        m.check(m.run_cut("c", t, [7, 8, 2, 7]), want, "portions at the steps")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("taps", [2, 4, 6])
+def test_convolution_reach(device, taps, monkeypatch):
+    """Taps that all count: the oracle with the taps turned round, with one tap less, or with a history that starts anew at
+    a portion's start is far away in the rows it touches."""
+    cfgd = config([att(heads=2, kv_heads=1, dim=10, conv=taps, scale=0.8)], width=40)
+    flat = tweak_of(lambda k, v: torch.linspace(0.3, 1.0, v.shape[-1])[None].expand_as(v).to(v.dtype).contiguous()
+                    if k.endswith("conv") else sharp(k, v))
+    t = toks(50, seed=14)
+    plain = oracle.short_conv
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype, tweak=flat)
+        want = m.expect(t)
+        for name, fn in (("turned round", lambda u, w: plain(u, w.flip(-1))), ("one less", lambda u, w: plain(u, w[:, 1:])),
+                         ("anew", lambda u, w: torch.cat([plain(u[:17], w), plain(u[17:], w)]))):
+            with monkeypatch.context() as mp:
+                mp.setattr(oracle, "short_conv", fn)
+                rows = slice(17, 17 + taps - 1) if name == "anew" else slice(taps, None)
+                assert gap_max(m.expect(t), want, rows) > 1e-2, name
+        m.check(m.run_cut("w", t, [len(t)]), want, "prompt")
+        m.check(m.run_cut("c", t, [17, 2, 2, 3, 1]), want, "portions shorter than the taps")
+        m.check(m.run_cut("d", t, [1]), want, "one by one")
+
+
+# ---------------------------------------------------------------------------------------------- matrix memory
+def memory_cfg(**kw):
+    return config([par(**{**dict(heads=1, kv_heads=1, dim=4, vdim=4, ls=0.2, rs=2.0), **kw})], width=40)
+
+
+MEMORIES = [dict(mheads=3, mdim=12, mvdim=20), dict(mheads=2, mdim=10, mvdim=9), dict(mheads=2, mdim=64, mvdim=48)]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("size", MEMORIES)
+def test_memory_formula(device, size, monkeypatch):
+    """Gates that move the running maximum up and down: the oracle whose maximum starts at minus infinity, whose
+    denominator has no lower bound or no absolute value, whose gates are not capped, or that forgets with a sigmoid of the
+    wrong sign is far away."""
+    cfgd = memory_cfg(cap=3.0, **size)
+    lively = tweak_of(lambda k, v: (v.float() * 4).to(v.dtype) if k.endswith(("right.i", "right.f"))
+                      else (v * 0 - 2.0 if k.endswith("i.b") else (v * 0 + 1.0 if k.endswith("f.b") else None)))
+
+    def variant(start=0.0, bound=True, absolute=True):
+        def mem(q, k, v, ig, fg):
+            T, H, D = k.shape
+            S, n = torch.zeros(H, D, v.shape[2], dtype=k.dtype), torch.zeros(H, D, dtype=k.dtype)
+            mx, out = torch.full((H,), start, dtype=k.dtype), torch.zeros_like(v)
+            for t in range(T):
+                new = torch.maximum(fg[t] + mx, ig[t])
+                keep, put = torch.exp(fg[t] + mx - new), torch.exp(ig[t] - new)
+                S = keep[:, None, None] * S + put[:, None, None] * (k[t][:, :, None] * v[t][:, None, :])
+                n, mx = keep[:, None] * n + put[:, None] * k[t], new
+                d = (n * q[t]).sum(-1)
+                d = d.abs() if absolute else d
+                d = torch.maximum(d, torch.exp(-mx)) if bound else d
+                out[t] = torch.einsum("hdv,hd->hv", S, q[t]) / (d + 1e-6)[:, None]
+            return out
+        return mem
+
+    t = toks(70, seed=15)
+    plain_mixer = oracle.memory_mixer
+    for dtype in modes(device):
+        # a large eps in the head norm keeps the read-outs' size visible behind it
+        cfgd["norm"]["eps"] = 0.05
+        m = Model(cfgd, device, dtype, tweak=lively)
+        want = m.expect(t)
+        for name, fn, bar in (("no bound", variant(bound=False), 5e-3), ("no absolute value", variant(absolute=False), 5e-3)):
+            with monkeypatch.context() as mp:
+                mp.setattr(oracle, "matrix_memory", fn)
+                assert gap_max(m.expect(t), want) > bar, name
+        with monkeypatch.context() as mp:
+            mp.setattr(oracle, "matrix_memory", variant())
+            assert gap_max(m.expect(t), want) < 1e-6, "the variants' base is the design"
+            mp.setattr(oracle, "memory_mixer", lambda h, c, w, e: plain_mixer(h, {**c, "gate_cap": 1e3}, w, e))
+            assert gap(m.expect(t), want) > 1e-2, "uncapped gates"
+        m.check(m.run_cut("w", t, [len(t)]), want, "prompt")
+        m.check(m.run_cut("d", t, [33, 1]), want, "decoding")
+        m.check(m.run_cut("c", t, [2, 31, 5, 2, 1]), want, "portions")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("size", MEMORIES)
+def test_running_maximum_starts_at_zero(device, size, monkeypatch):
+    """Input gates far below zero: with a maximum that starts at minus infinity the first tokens' denominators are bounded
+    by e^12 instead of 1 and the read-outs vanish behind the norm's eps (or do not)."""
+    cfgd = memory_cfg(cap=12.0, **size)
+    quiet = tweak_of(lambda k, v: v * 0 - 6.0 if k.endswith("i.b") else (v * 0 + 8.0 if k.endswith("f.b") else None))
+    cfgd["norm"]["eps"] = 1e-4
+    t = toks(40, seed=16)
+
+    def from_below(q, k, v, ig, fg):
+        T, H, D = k.shape
+        S, n = torch.zeros(H, D, v.shape[2], dtype=k.dtype), torch.zeros(H, D, dtype=k.dtype)
+        mx, out = torch.full((H,), -1e30, dtype=k.dtype), torch.zeros_like(v)
+        for i in range(T):
+            new = torch.maximum(fg[i] + mx, ig[i])
+            keep, put = torch.exp(fg[i] + mx - new), torch.exp(ig[i] - new)
+            S = keep[:, None, None] * S + put[:, None, None] * (k[i][:, :, None] * v[i][:, None, :])
+            n, mx = keep[:, None] * n + put[:, None] * k[i], new
+            den = torch.maximum((n * q[i]).sum(-1).abs(), torch.exp(-mx * 0)) + 1e-6  # the bound of an unscaled sum
+            out[i] = torch.einsum("hdv,hd->hv", S, q[i]) / den[:, None]
+        return out
+
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype, tweak=quiet)
+        want = m.expect(t)
+        with monkeypatch.context() as mp:
+            mp.setattr(oracle, "matrix_memory", from_below)
+            assert gap_max(m.expect(t), want, slice(0, 8)) > 1e-2
+        m.check(m.run_cut("w", t, [len(t)]), want, "prompt")
+        m.check(m.run_cut("d", t, [1]), want, "one by one")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("size", MEMORIES)
+def test_memory_keeps_a_far_write(device, size):
+    """One token writes with a wide open input gate, all others hardly write and nothing is forgotten: 250 tokens later
+    its value is still what is read.  Another token in its place moves the logits there; a state lost between portions, at
+    a chunk's edge or in decoding would too."""
+    cfgd = memory_cfg(cap=9.0, **size)
+
+    def planted(w):
+        marked(w, 40, VOCAB - 1, scale=12.0)
+        for n, v in (("i", 0.0), ("f", 0.0)):
+            w[f"l0.mix.right.{n}"] = torch.zeros_like(w[f"l0.mix.right.{n}"])
+        w["l0.mix.right.i"][:, 1] = 6.0
+        w["l0.mix.right.i.b"] = torch.full_like(w["l0.mix.right.i.b"], -8.0)
+        w["l0.mix.right.f.b"] = torch.full_like(w["l0.mix.right.f.b"], 40.0)
+
+    t = toks(300, vocab=VOCAB - 1, seed=17)
+    t[3] = VOCAB - 1
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype, max_tokens=320, tweak=planted)
+        want = m.expect(t)
+        moved = list(t)
+        moved[3] = 7
+        assert gap(m.expect(moved), want, slice(250, None)) > 5e-2, "the far write does not matter in this construction"
+        m.check(m.run_cut("a", t, [257, 1]), want, "prompt, then decoding")
+        m.check(m.run_cut("b", t, [31, 2, 64, 33, 2, 97, 1]), want, "portions on and off chunk borders")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_memory_forgets_and_overflows_nothing(device):
+    """Forget gates at their cap's floor and input gates at its ceiling, token by token at random: exponents of both signs
+    far beyond what a plain exponential could hold over a hundred tokens stay finite and right."""
+    cfgd = memory_cfg(cap=30.0, mheads=3, mdim=12, mvdim=20)
+    wild = tweak_of(lambda k, v: (v.float() * 40).to(v.dtype) if k.endswith(("right.i", "right.f")) else None)
+    t = toks(150, seed=18)
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype, tweak=wild)
+        want = m.expect(t)
+        assert torch.isfinite(want).all()
+        got = m.run_cut("w", t, [len(t)])
+        dec = m.run_cut("d", t, [60, 1])
+        assert torch.isfinite(got).all() and torch.isfinite(dec).all()
+        if dtype == torch.float32:  # a bf16 row moves a gate by whole units here
+            m.check(got, want, "prompt")
+            m.check(dec, want, "decoding")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_both_halves_and_their_scales(device):
+    """The oracle with the scales exchanged, or with one half left out, is far away."""
+    cfgd = config([par(ls=1.4, rs=0.5)], width=40)
+    t = toks(40, seed=19)
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype)
+        want = m.expect(t)
+        for ls, rs in ((0.5, 1.4), (1.4, 0.0), (0.0, 0.5), (1.4, 0.6)):
+            assert gap(m.expect(t, config([par(ls=ls, rs=rs)], width=40)), want) > 1e-2, (ls, rs)
+        m.check(m.run_cut("h", t, [17, 2, 1]), want, "both halves")
+
+
+# ---------------------------------------------------------------------------------------------- feed-forward, norms
+@pytest.mark.parametrize("device", DEVICES)
+def test_experts_by_token_id(device, monkeypatch):
+    """The oracle with the next id's experts, with the sequence's previous token's, with the chosen experts' sum instead
+    of their mean, or without the shared expert is far away; a request decoded in a batch uses its own tokens' rows."""
+    cfgd = config([att(mlp=moe(experts=7, top=2)), par(mlp=moe(experts=7, top=2)), att(mlp=moe(experts=4, top=3, shared=0))], width=40)
+    t, other = toks(40, seed=20), toks(40, seed=21)
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype)
+        want = m.expect(t)
+        shifted = changed(m.weights, lambda k, v: v.roll(1, 0) if k.endswith("table") else None)
+        assert gap(m.expect(t, weights=shifted), want) > 2e-2
+        swapped = dict(m.weights)
+        swapped["l0.mlp.table"], swapped["l1.mlp.table"] = m.weights["l1.mlp.table"], m.weights["l0.mlp.table"]
+        assert gap(m.expect(t, weights=swapped), want) > 2e-2
+        with monkeypatch.context() as mp:
+            plain = oracle.feed_forward
+            mp.setattr(oracle, "feed_forward", lambda h, f, w, tk: plain(h, {**f, "shared": None}, w, tk))
+            assert gap(m.expect(t), want) > 2e-2
+            mp.setattr(oracle, "feed_forward", lambda h, f, w, tk: plain(h, f, w, torch.cat([tk[:1], tk[:-1]])))
+            assert gap(m.expect(t), want) > 2e-2
+        out = [m.engine.force_step([("x", other[:9], []), ("y", t[:21], list(range(21)))])]
+        for i in range(21, 40):
+            step = m.engine.force_step([("x", other[i - 12:i - 11], [0]), ("y", t[i:i + 1], [0])], ["x", "y"] if i == 39 else [])
+            out.append(step[1:])
+        m.check(torch.cat(out), want, "beside another request")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_norms_on_both_sides(device, monkeypatch):
+    """The oracle whose gains are taken as they are stored, or that leaves the outer norms out, is far away."""
+    cfgd = config([att(mlp=dense()), par(mlp=moe())], width=40)
+    t = toks(30, seed=22)
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype)
+        want = m.expect(t)
+        with monkeypatch.context() as mp:
+            mp.setattr(oracle, "offset_norm", lambda v, g, e: oracle.rms(v, e) * g)
+            assert gap(m.expect(t), want) > 5e-2
+        ones = changed(m.weights, lambda k, v: torch.zeros_like(v) if k.endswith(("norm1b", "norm2b")) else None)
+        assert gap(m.expect(t, weights=ones), want) > 1e-2
+        m.check(m.run_cut("n", t, [len(t)]), want, "norms")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_first_tokens(device):
+    """Positions 0, 1, 2 as a one-token request, as single tokens from the start, and in a slot that held another
+    sequence."""
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype, max_seqs=1)
+        m.run_cut("warm", toks(40, seed=15), [40])
+        for n in (1, 2, 3):
+            t = toks(n, seed=16 + n)
+            m.check(m.run_cut(f"n{n}", t, [1]), m.expect(t), f"{n} first tokens, one by one")
+            m.check(m.run_cut(f"w{n}", t, [n]), m.expect(t), f"{n} first tokens, at once")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_long_decoding(device):
+    """Decoding runs over several pages."""
+    t = toks(150, seed=20)
+    for dtype in modes(device):
+        m = Model(STACK, device, dtype)
+        m.check(m.run_cut("l", t, [5, 1]), m.expect(t), "long decoding")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name,cfgd", [
+    ("all ones", config([att(heads=1, kv_heads=1, dim=1, conv=1, rot=None, mlp=moe(experts=1, top=1, ff=1, shared=1)),
+                         par(heads=1, kv_heads=1, dim=1, vdim=1, temp=(1.0, 1), mheads=1, mdim=1, mvdim=1, cap=1.0, ls=1.0, rs=1.0,
+                             mlp=dense(1))], width=2, vocab=7, scale=1.0)),
+    ("odd sizes", config([att(heads=6, kv_heads=3, dim=14, conv=5, rot={"base": 20.0, "dims": 14}, mlp=moe(experts=9, top=4, ff=7, shared=5)),
+                          par(heads=9, kv_heads=3, dim=13, vdim=11, mheads=5, mdim=9, mvdim=15, mlp=dense(17))], width=19, vocab=23)),
+    ("sizes that vector loads and the MFMA forms like", config(
+        [att(heads=8, kv_heads=2, dim=64, conv=4, scale=0.2, rot={"base": 900.0, "dims": 32}, mlp=moe(experts=8, top=2, ff=64, shared=32)),
+         par(heads=8, kv_heads=4, dim=64, vdim=32, scale=0.2, mheads=4, mdim=32, mvdim=64, mlp=moe(experts=4, top=1, ff=32, shared=0)),
+         par(heads=2, kv_heads=2, dim=32, vdim=80, mheads=3, mdim=96, mvdim=48, mlp=dense(64))], width=64, vocab=96)),
+    ("wide heads on the row form and on the walk", config(
+        [att(heads=2, kv_heads=1, dim=136, conv=3, scale=0.1, rot={"base": 900.0, "dims": 40}),
+         par(heads=2, kv_heads=1, dim=40, vdim=72, scale=0.1, mheads=2, mdim=270, mvdim=130)], width=48, vocab=50)),
+    ("wide heads on the MFMA forms", config(
+        [att(heads=3, kv_heads=3, dim=256, conv=4, scale=0.1, rot={"base": 900.0, "dims": 64}),
+         par(heads=4, kv_heads=1, dim=512, vdim=128, scale=0.05, mheads=2, mdim=256, mvdim=320),
+         par(heads=2, kv_heads=2, dim=96, vdim=16, scale=0.1, mheads=1, mdim=160, mvdim=512)], width=48, vocab=50)),
+    ("a memory whose state streams through memory", config([par(mheads=1, mdim=512, mvdim=512)], width=32, vocab=40)),
+    ("projections on the tiled-layout GEMMs", config(
+        [att(heads=8, kv_heads=4, dim=128, conv=4, scale=0.1, rot={"base": 900.0, "dims": 64}, mlp=dense(2048)),
+         par(heads=8, kv_heads=4, dim=128, vdim=64, scale=0.1, mheads=4, mdim=128, mvdim=128,
+             mlp=moe(experts=4, top=2, ff=256, shared=512))], width=1024, vocab=1024)),
+])
+def test_other_sizes(device, name, cfgd):
+    vocab = cfgd["vocab"]
+    t = toks(61, vocab=vocab, seed=21)
+    for dtype in modes(device):
+        m = Model(cfgd, device, dtype)
+        m.check(m.run_cut("x", t, [len(t)]), m.expect(t), name + ", whole")
+        m.check(m.run_cut("y", t, [7, 2, 1]), m.expect(t), name + ", portions and decoding")
+
+
+@pytest.mark.gpu
+def test_long_prompt_of_many_tiles():
+    """Six hundred tokens on the GPU: prompt-sized expert tiles, attention tiles over many pages, many memory chunks, more
+    than one round of the memory's gate scan."""
+    cfgd = config([att(heads=4, kv_heads=2, dim=32, conv=4, rot={"base": 900.0, "dims": 16}, mlp=moe(experts=8, top=2, ff=64, shared=128)),
+                   par(heads=4, kv_heads=2, dim=32, vdim=32, temp=(0.3, 64), mheads=4, mdim=32, mvdim=32,
+                       mlp=moe(experts=3, top=1, ff=64, shared=0))], width=64, vocab=200)
+    t = toks(1150, vocab=200, seed=22)
+    for dtype in (torch.float32, torch.bfloat16):
+        m = Model(cfgd, "cuda", dtype, max_tokens=1184)
+        want = m.expect(t)
+        m.check(m.run_cut("a", t, [1100, 1]), want, "prompt, then decoding")
+        m.check(m.run_cut("b", t, [300, 3, 797, 25, 1]), want, "portions")
+
+
+# ---------------------------------------------------------------------------------------------- generation
+@pytest.mark.parametrize("device", DEVICES)
+def test_greedy_generation_through_the_scheduler(device):
+    """add_request + step: admission, chunked prompt passes (a 16-token budget), mixed steps, decode with sampling at
+    temperature 0, slot release.  Each generated token is the oracle's argmax given the tokens before it (a step whose two
+    best logits are closer than the tolerance is not judged)."""
+    m = Model(STACK, device, torch.float32, max_tokens=512, max_seqs=3)
+    eng = LLMEngine(m.runner, eos_id=-1, prefill_budget=16, idle_prefill_budget=16)
+    prompts = {"g0": toks(19, seed=23), "g1": toks(40, seed=24), "g2": toks(3, seed=25), "g3": toks(33, seed=26)}
+    for cid, p in prompts.items():
+        eng.add_request(cid, p, SamplingParams(temperature=0.0, max_tokens=12, ignore_eos=True))
+    out = {cid: [] for cid in prompts}
+    for ev in eng.run_until_idle():
+        if not ev.done:
+            out[ev.conversation_id].append(ev.token_id)
+    for cid, p in prompts.items():
+        assert len(out[cid]) == 12, (cid, out[cid])
+        logits = m.expect(p + out[cid])
+        for i, tok in enumerate(out[cid]):
+            row = logits[len(p) + i - 1]
+            top = torch.topk(row, 2).values
+            if float(top[0] - top[1]) > 1e-3 * float(row.abs().max()):
+                assert tok == int(row.argmax()), f"{cid}: token {i} is {tok}, the oracle says {int(row.argmax())}"
+    assert eng.alloc.num_free == eng.alloc.num_blocks
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("cfgd", [STACK, config([att(heads=4, kv_heads=2, dim=32, rot={"base": 900.0, "dims": 16}, mlp=moe()),
+                                                 par(heads=4, kv_heads=2, dim=32, vdim=32, mheads=2, mdim=32, mvdim=32, mlp=moe())])])
+def test_decode_graphs_match_eager(cfgd):
+    """The captured decode step replayed over several steps (with eager work between the replays) gives the eager
+    step's logits."""
+    m = Model(cfgd, "cuda", torch.bfloat16)
+    t = toks(60, seed=27)
+    eager = m.run_cut("e", t, [20, 1])
+    m.runner.use_graphs = True
+    m.runner.capture()
+    assert m.runner.graphs
+    graphed = m.run_cut("g", t, [20, 1])
+    assert torch.allclose(eager, graphed, atol=1e-5, rtol=1e-5)
+    m.check(graphed, m.expect(t), "graph replays")
+
+
+def test_config_round_trip_and_registry(tmp_path):
+    cfg = LobidraConfig.from_dict(STACK)
+    again = LobidraConfig.from_dict(cfg.to_dict())
+    assert again.layers == cfg.layers and again == cfg
+    assert [(r.layer, r.index) for r in cfg.runs()] == [(0, 0), (1, 1), (2, 2), (3, 3), (1, 4), (0, 5)]
+    bare = LobidraConfig.from_dict(config([att(conv=0, rot=None)]))
+    assert LobidraConfig.from_dict(bare.to_dict()) == bare and set(tensor_shapes(bare)) == {
+        "embed", "head", "final.norm", "l0.norm1", "l0.norm1b", "l0.mix.q", "l0.mix.k", "l0.mix.g", "l0.mix.o"}
+    from safetensors.torch import save_file
+
+    (tmp_path / "config.json").write_text(json.dumps(STACK))
+    weights = init_weights(cfg, seed=3)
+    save_file({k: v.contiguous() for k, v in weights.items()}, str(tmp_path / "model.safetensors"))
+    fam, cfg2, path = registry.resolve(str(tmp_path))
+    assert fam.name == "lobidra" and cfg2.layers == cfg.layers and cfg2.width == cfg.width and path == str(tmp_path)
+    w = registry.load_weights(fam, cfg2, path, device="cpu", dtype=torch.float32)
+    assert w.layers[1].mlp.gate.shape == (5, 9, 40) and w.layers[1].mlp.table.dtype == torch.int32
+    assert w.layers[4] is w.layers[1] and w.layers[5] is w.layers[0] and w.layers[2].mlp.sgate is None and w.layers[3].mlp is None
+    assert torch.equal(w.layers[0].norm1, 1.0 + weights["l0.norm1"].float()) and not w.layers[0].mix.sink.any()
+    assert w.layers[0].mix.big.shape == (64, 40) and w.layers[1].mix.o.shape == (40, 56)
+    r = registry.make_runner(fam, w, num_blocks=4, max_batch=2, max_model_len=64, device=torch.device("cpu"))
+    assert sorted(r.kv.k) == list(range(6)) and sorted(r.state.state) == [1, 3, 4] and sorted(r.state.tail) == [0, 2, 5]
+    assert set(tensor_shapes(cfg)) == set(weights)
+    assert registry.resolve("lobidra-tiny")[0].name == "lobidra"
+    assert cfg.cache_bytes_per_token() == 2 * (2 * 20 + 2 * 14 + 3 * 16 + 1 * 16 + 2 * 14 + 2 * 20)
+    assert registry.cache_blocks_for_budget(cfg, cfg.cache_bytes_per_token() * 32 * 7) == 7
+    for name, cut in (("l0.mix.q", lambda v: v[:-1]), ("l1.mlp.table", lambda v: v + 5)):
+        bad = dict(weights)
+        bad[name] = cut(bad[name])
+        with pytest.raises(ValueError):
+            convert_lobidra(cfg, bad)
+    wrong_v = att()
+    wrong_v["mixer"]["vdim"] = 12
+    for layers in ([att(heads=3)], [wrong_v], [att(mlp=moe(experts=2, top=3))], [att(), att(dim=12, weights_of=0)],
+                   [att(), par(weights_of=0)], [att(rot={"base": 10.0, "dims": 12})], [att(weights_of=0), att(weights_of=5)],
+                   [par(cap=0.0)], [par(mdim=600)]):
+        with pytest.raises(ValueError):
+            LobidraConfig.from_dict(config(layers))
+    with pytest.raises(ValueError):
+        cfg.validate(tp=2)
+
+
+def test_serving_builds_the_family_by_name():
+    """The serving launcher's engine builder resolves the family through the registry and generates with it."""
+    from distributed_sse_for_llm_response_amd.serving.app import build_engine
+    from distributed_sse_for_llm_response_amd.serving.config import ServeConfig
+
+    eng, _ = build_engine(ServeConfig(model="lobidra-tiny", engine="cpu"))
+    eng.add_request("c1", [5, 6, 7, 8, 9, 10], SamplingParams(temperature=0.0, max_tokens=4, ignore_eos=True))
+    eng.add_request("c2", [11, 12], SamplingParams(temperature=0.8, max_tokens=3, ignore_eos=True))
+    ev = eng.run_until_idle()
+    assert sum(1 for e in ev if e.conversation_id == "c1" and not e.done) == 4
+    assert sum(1 for e in ev if e.conversation_id == "c2" and not e.done) == 3

@@ -100,7 +100,7 @@ class Model:
 
     def check(self, got, want, what=""):
         """Row-wise: rms of the difference (mean taken off) over the rms of the expected logits.  fp32 judges every row,
-        bf16 nine rows in ten (all but one of a few), the median and, loosely, every row."""
+        bf16 nine rows in ten and the median; of a few rows all but one, and that one loosely."""
         got, want = got.detach().float().cpu(), want.float()
         assert got.shape == want.shape, (got.shape, want.shape)
         assert torch.isfinite(got).all(), what
@@ -111,7 +111,8 @@ class Model:
             assert float(err.max()) < 2e-4, f"{what}: worst row {int(err.argmax())} error {float(err.max()):.3g}"
         else:
             off = int((err >= 4e-2).sum())
-            assert off <= max(1, err.numel() // 10) and float(err.max()) < 0.15 and float(err.median()) < 2e-2, \
+            few = off == 0 or err.numel() > 10 or float(err.max()) < 0.15
+            assert off <= max(1, err.numel() // 10) and few and float(err.median()) < 2e-2, \
                 f"{what}: median {float(err.median()):.3g}, {off} of {err.numel()} rows off, worst {float(err.max()):.3g}"
 
     def run_cut(self, cid, tokens, cuts, end=True):

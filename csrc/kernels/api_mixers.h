@@ -69,6 +69,8 @@ struct SinkAttnParams {
   int gate_wide;         // 1: the gate has H * V columns, one per element of the output
   int ldo;               // row stride of out, H * V when contiguous (a multiple of 4 for the MFMA form)
   float out_scale;       // multiplies the output before it is rounded (1: nothing)
+  int nparts;            // decode form: stretches the walk of a row is split into (<= 1: none, at most 16)
+  float* part;           // [work items, H, nparts, V + 2] when split
 };
 
 // The fused projection's q | k | v columns into the attention's operands.
@@ -230,6 +232,8 @@ hipError_t dsse_sink_attention(int num_work, const dsse::SinkAttnParams* p, hipS
 // transposed pages vt [pages, G, V, kBS] (keys permuted inside a page as the MFMA's k axis wants them)
 // split (V <= 128): the four waves of a workgroup share one (tile, head) and split its pages -- decode steps
 hipError_t dsse_sink_flash(int num_work, const dsse::SinkAttnParams* p, const void* vt, int split, hipStream_t st);
+// prompt portions with every page staged once for 8 / rt heads of a key/value group and rt tiles of 16 rows (rt 2, 4, 8)
+hipError_t dsse_sink_tile(int num_work, const dsse::SinkAttnParams* p, const void* vt, int rt, hipStream_t st);
 // decode form over the same pages: one row per item, the heads of a key/value group side by side, pages split over waves
 hipError_t dsse_sink_decode(int num_work, const dsse::SinkAttnParams* p, const void* vt, hipStream_t st);
 // p1 / p2 hold N / rep1 and N / rep2 numbers: entry j serves columns [j rep, (j + 1) rep)

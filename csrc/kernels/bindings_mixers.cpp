@@ -177,7 +177,7 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
                     const Tensor& q_start, const Tensor& q_len, const Tensor& ctx_len, const Tensor& work_seq,
                     const Tensor& work_tile, const OptTensor& sink, const OptTensor& gate, Tensor& out, int64_t window,
                     double scale, int64_t qt, const OptTensor& vt, bool split, double softcap, const OptTensor& out_rope,
-                    const OptTensor& rel, int64_t keep_first, double out_scale) {
+                    const OptTensor& rel, int64_t keep_first, double out_scale, const OptTensor& part, int64_t nparts) {
   f32t(q, "q");
   gpu(kcache, "kcache");
   gpu(vcache, "vcache");
@@ -256,11 +256,26 @@ void sink_attention(const Tensor& q, const Tensor& kcache, const Tensor& vcache,
                 "vt must be [pages, G, V, 32]");
     if (qt == 1) {  // decode form: one row per item
       TORCH_CHECK(p.D % 32 == 0 && p.V % 16 == 0 && !split, "the decode form needs D % 32 == 0, V % 16 == 0, no split");
-      TORCH_CHECK(p.G <= 65535 && p.H / p.G <= 16 * 65535, "too many heads");
+      TORCH_CHECK(p.G <= 65535 && p.H / p.G <= 16 * 1024, "too many heads");
+      if (part.has_value() && nparts > 1) {
+        f32t(*part, "part");
+        TORCH_CHECK(nparts <= 16 && part->numel() >= work_seq.numel() * p.H * nparts * (p.V + 2) &&
+                        work_seq.numel() * p.H < INT_MAX / 4,
+                    "part must hold [work items, H, nparts <= 16, V + 2]");
+        p.part = part->data_ptr<float>();
+        p.nparts = (int)nparts;
+      }
       DSSE_CHECK_HIP(dsse_sink_decode((int)work_seq.numel(), &p, vt->data_ptr(), cur_stream()));
       return;
     }
     TORCH_CHECK(p.ldo % 4 == 0 && reinterpret_cast<uintptr_t>(p.out) % 8 == 0, "the MFMA form stores 8-byte pieces of out");
+    if (qt > 16) {  // pages shared by 128 / qt heads of a group
+      TORCH_CHECK((qt == 32 || qt == 64 || qt == 128) && (p.H / p.G) % (128 / qt) == 0 && p.D % 32 == 0 && p.V % 16 == 0 &&
+                      p.D <= 128 && p.V <= 128 && !p.rel && !p.out_rope && !split && work_seq.numel() <= 65535,
+                  "the shared-page form: qt 32 / 64 / 128 for groups of 4 / 2 / 1 heads, widths up to 128, no bias, no rotation");
+      DSSE_CHECK_HIP(dsse_sink_tile((int)work_seq.numel(), &p, vt->data_ptr(), (int)qt / 16, cur_stream()));
+      return;
+    }
     TORCH_CHECK(qt == 16 && p.D % 32 == 0 && p.V % 16 == 0, "the MFMA form needs qt = 16, D % 32 == 0, V % 16 == 0");
     TORCH_CHECK(!split || p.V <= 128, "the key split of the MFMA form needs V <= 128");
     DSSE_CHECK_HIP(dsse_sink_flash((int)work_seq.numel(), &p, vt->data_ptr(), split ? 1 : 0, cur_stream()));
@@ -789,7 +804,7 @@ TORCH_LIBRARY_FRAGMENT(dsse, m) {
   m.def("sink_attention(Tensor q, Tensor kcache, Tensor vcache, Tensor block_tables, Tensor q_start, Tensor q_len, "
         "Tensor ctx_len, Tensor work_seq, Tensor work_tile, Tensor? sink, Tensor? gate, Tensor(a!) out, int window, "
         "float scale, int qt, Tensor? vt=None, bool split=False, float softcap=0.0, Tensor? out_rope=None, "
-        "Tensor? rel=None, int keep_first=0, float out_scale=1.0) -> ()");
+        "Tensor? rel=None, int keep_first=0, float out_scale=1.0, Tensor(b!)? part=None, int nparts=1) -> ()");
   m.def("gate_math(Tensor(a!) x, int kind, Tensor? p1=None, Tensor? p2=None, float c=1.0) -> ()");
   m.def("matrix_scan(Tensor q, Tensor k, Tensor v, Tensor? decay, Tensor? beta, Tensor(a!) state, Tensor q_start, "
         "Tensor q_len, Tensor ctx_len, Tensor state_slot, Tensor(b!) out, float q_scale=1.0) -> ()");

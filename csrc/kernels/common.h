@@ -63,6 +63,11 @@ DEV bf16x8 ld_buf_bf16x8(__amdgpu_buffer_rsrc_t r, uint32_t off) {
 }
 
 
+// Workgroup barrier that orders LDS traffic only.  __syncthreads() also waits for every outstanding global load, which
+// would land a prefetch at each barrier; here those loads stay in flight until their registers are used (the compiler's
+// own vmcnt wait).
+DEV void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // Non-temporal 16-byte load for once-read streams (weights, KV pages).
 DEV bf16x8 ld_nt_bf16x8(const bf16* p) {
   return __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(p));

@@ -202,10 +202,6 @@ void launch_walk(const MatrixMemoryParams& p, hipStream_t st) {
 constexpr int kChunk = 32;
 constexpr float kLog2e = 1.4426950408889634f;
 
-// Workgroup barrier that orders LDS traffic only: the next chunk's loads stay in flight across it (__syncthreads() would
-// wait for them); the compiler waits for them where their registers are used.
-DEV void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-
 // Where a sequence's chunk sums start in acum / u: the rows keep their order, every start is a multiple of four floats.
 DEV int sums_at(int row0, int seq) { return ((row0 + 3) & ~3) + 4 * seq; }
 

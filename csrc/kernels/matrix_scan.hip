@@ -31,11 +31,6 @@ namespace {
 
 constexpr int kScanCols = 16;
 
-// Workgroup barrier that orders LDS traffic only.  __syncthreads() also waits for every outstanding global load, which
-// would land the next block's prefetch at each barrier; here those loads stay in flight until stage() uses them (the
-// compiler's own vmcnt wait at the first use of their registers).
-DEV void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-
 template <int DPT, int TB, bool DELTA>
 __global__ __launch_bounds__(1024) void matrix_scan_kernel(MatrixScanParams p, int R) {
   constexpr int RW = 4 * DPT;        // rows of S per wave

@@ -28,6 +28,7 @@ namespace dsse {
 namespace {
 
 constexpr int kMaxV = 512;
+constexpr int kMaxParts = 16;  // stretches a decode walk may be split into
 constexpr int kAccs = kMaxV / 64;
 
 // q (LDS, fp32) . key row (global): 16-byte loads when the row width allows
@@ -186,6 +187,32 @@ DEV float tanh_fast(float x) {
   return (e - 1.0f) / (e + 1.0f);
 }
 
+// The MFMA forms keep scores and running maxima in units of log 2: a weight is then one instruction.
+constexpr float kLog2e = 1.4426950408889634f;
+DEV float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
+
+// One step of the online softmax over a page: a lane's eight scores (log2 units, -inf: not seen) become weights, the
+// MFMA operand pf; new maximum m and sum l; returned: the factor of the sums so far.  No branches: the next page's loads
+// stay in flight across it.
+DEV float softmax_step(const float (&sv)[8], float& m, float& l, bf16x8& pf) {
+  float mx = sv[0];
+#pragma unroll
+  for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
+  const float mn = fmaxf(m, rows4_max(mx));
+  const float at = mn == -INFINITY ? 0.0f : mn;  // nothing seen yet: exp2(-inf - 0) is 0
+  const float corr = exp2_hw(m - at);
+  float ps = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const float e = exp2_hw(sv[i] - at);
+    ps += e;
+    pf[i] = (bf16)e;
+  }
+  l = l * corr + rows4_sum(ps);
+  m = mn;
+  return corr;
+}
+
 // The distance biases of a lane's eight keys of a page: keys 0 .. 3 and 16 .. 19 from its first one, which is n0 away from
 // the query.  The branches are uniform: far pages share the last entry, a table that fits its LDS strip needs no memory.
 DEV void bias_entries(float (&bv)[8], bool far, float rel_far, const float* strip, const float* table, int strip_len,
@@ -266,7 +293,9 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
 #pragma unroll
   for (int n = 0; n < NT; ++n) O[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
-  const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f;
+  // scores in log2 units; a cap acts on the plain ones
+  const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f, cap2 = p.softcap * kLog2e;
+  const float scale2 = p.softcap > 0.f ? p.scale : p.scale * kLog2e;
   const int nks = D / 32;
   const int pg_lo = lo / kBS;
   int kept_pages = 0;  // whole pages of kept keys before the window's first page
@@ -349,7 +378,6 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
       if constexpr (AHEAD_V) load_values(nb, vn);
     }
     float sv[8];
-    float mx = -INFINITY;
     // uniform: every (row, key) pair of this tile and page is at least rel_len - 1 apart
     const bool far = EXT && p.rel && pos0 + tile * 16 - (pg * kBS + kBS - 1) >= p.rel_len - 1;
     float bv[8];
@@ -358,25 +386,13 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
     for (int i = 0; i < 8; ++i) {
       const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
       const bool seen = c_ok && key <= c_pos && (c_pos - key < p.window || (EXT && key < p.keep_first));
-      float sc = (i < 4 ? s0[i] : s1[i - 4]) * p.scale;
-      if (p.softcap > 0.f) sc = p.softcap * tanh_fast(sc * cap_inv);
-      if (EXT && p.rel) sc += bv[i];
+      float sc = (i < 4 ? s0[i] : s1[i - 4]) * scale2;
+      if (p.softcap > 0.f) sc = cap2 * tanh_fast(sc * cap_inv);
+      if (EXT && p.rel) sc += bv[i] * kLog2e;
       sv[i] = seen ? sc : -INFINITY;
-      mx = fmaxf(mx, sv[i]);
     }
-    mx = rows4_max(mx);
-    const float mn = fmaxf(m, mx);
-    const float corr = mn == -INFINITY ? 1.0f : expf(m - mn);
     bf16x8 pf;
-    float ps = 0.f;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float e = sv[i] == -INFINITY ? 0.0f : expf(sv[i] - mn);
-      ps += e;
-      pf[i] = (bf16)e;
-    }
-    l = l * corr + rows4_sum(ps);
-    m = mn;
+    const float corr = softmax_step(sv, m, l, pf);
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       f32x4 o = O[n];
@@ -407,15 +423,16 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
     for (int idx = threadIdx.x; idx < rows_on * V; idx += blockDim.x) {
       const int col = idx / V, d = idx - col * V;
       const int64_t row = q0 + tile * 16 + col;
-      float mm = p.sink ? p.sink[h] : -INFINITY;
+      const float sk = p.sink ? p.sink[h] * kLog2e : -INFINITY;
+      float mm = sk;
       for (int w = 0; w < 4; ++w) mm = fmaxf(mm, mg[(w * 16 + col) * ldm + V]);
-      float den = p.sink ? expf(p.sink[h] - mm) : 0.f, num = 0.f, nump = 0.f;
+      float den = p.sink ? exp2_hw(sk - mm) : 0.f, num = 0.f, nump = 0.f;
       const int half = V >> 1;
       const bool lo_half = d < half;
       const int dp = lo_half ? d + half : d - half;
       for (int w = 0; w < 4; ++w) {
         const float* src = mg + (w * 16 + col) * ldm;
-        const float f = src[V] == -INFINITY ? 0.f : expf(src[V] - mm);
+        const float f = src[V] == -INFINITY ? 0.f : exp2_hw(src[V] - mm);
         den += src[V + 1] * f;
         num += src[d] * f;
         nump += src[dp] * f;
@@ -434,10 +451,10 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
   if (c_ok) {
     float den = l, f = 1.0f;
     if (p.sink) {  // the sink joins the denominator under the common maximum
-      const float sk = p.sink[h];
+      const float sk = p.sink[h] * kLog2e;
       const float mm = fmaxf(m, sk);
-      f = expf(m - mm);
-      den = l * f + expf(sk - mm);
+      f = exp2_hw(m - mm);
+      den = l * f + exp2_hw(sk - mm);
     }
     float inv = den > 0.f ? f / den * p.out_scale : 0.0f;
     if (p.gate && !p.gate_wide) inv *= 1.0f / (1.0f + expf(-p.gate[c_row * p.ldg + h]));
@@ -470,12 +487,220 @@ __global__ __launch_bounds__(256) void sink_flash_kernel(SinkAttnParams p, const
 }
 
 // ---------------------------------------------------------------------------------------------------------------------
+// Shared-page form for prompt portions (bf16, head widths up to 128): a workgroup takes hb heads of ONE key/value group times
+// rt tiles of 16 query rows, hb rt = 8 column tiles, two per wave.  Each page's keys and transposed values are staged in LDS
+// once for all eight tiles, and a fragment read from LDS feeds both tiles of a wave; the next two pages are on their way
+// (in registers) while the current one is in the MFMAs, one barrier per page.  The query operands stay in registers.  Masks and
+// the rescaling of the sums are branches here: pages that every row sees whole and maxima that stay skip them.  The head
+// group is the fast grid dimension, so workgroups of one XCD keep to the same keys when the groups are a multiple of eight.
+constexpr int kTileWidth = 128;   // widest query and value heads
+constexpr int kTileLdv = kBS + 8;
+
+template <int NT>
+__global__ __launch_bounds__(256, 2) void sink_tile_kernel(SinkAttnParams p, const bf16* __restrict__ vt, int hb, int rt) {
+  extern __shared__ __align__(16) unsigned char smem_raw[];
+  constexpr int V = 16 * NT, KS = kTileWidth / 32, KC = kTileWidth * kBS / 8 / 256, VC = (V * kBS / 8 + 255) / 256;
+  const int D = p.D, nks = D / 32, ldk = D + 8;
+  const int buf_elems = kBS * ldk + V * kTileLdv;
+  bf16* smem = reinterpret_cast<bf16*>(smem_raw);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
+  const int seq = p.work_seq[blockIdx.y], tile = p.work_tile[blockIdx.y];
+  const int ql = p.q_len[seq], row_first = tile * 16 * rt;
+  if (row_first >= ql) return;  // uniform for the workgroup
+  const int h_first = blockIdx.x * hb, kvh = h_first / (p.H / p.G);
+  const int q0 = p.q_start[seq], pos0 = p.ctx_len[seq] - ql;
+  const int row_last = row_first + 16 * rt < ql ? row_first + 16 * rt - 1 : ql - 1;
+  const int hi = pos0 + row_last;
+  int lo = pos0 + row_first - p.window + 1;
+  lo = lo > 0 ? lo : 0;
+  const int pg_lo = lo / kBS;
+  int kept_pages = 0;
+  if (p.keep_first > 0) {
+    kept_pages = (p.keep_first + kBS - 1) / kBS;
+    kept_pages = kept_pages < pg_lo ? kept_pages : pg_lo;
+  }
+  const int walk = kept_pages + hi / kBS - pg_lo + 1;
+  const int* bt = p.block_tables + (int64_t)seq * p.max_blocks;
+  auto page_at = [&](int it) { return it < kept_pages ? it : pg_lo + it - kept_pages; };
+  auto ids_from = [&](int it0) {
+    const int b = it0 + lane < walk ? bt[page_at(it0 + lane)] : 0;
+    return (unsigned)b < (unsigned)p.num_blocks ? b : 0;
+  };
+  // this wave's two column tiles
+  int head[2], pos[2], tile_lo[2], tile_hi[2];
+  bool on[2];
+  int64_t row[2];
+  bf16x8 qf[2][KS];
+#pragma unroll
+  for (int c = 0; c < 2; ++c) {
+    const int ct = 2 * wave + c, off = row_first + 16 * (ct % rt) + r;
+    head[c] = h_first + ct / rt;
+    on[c] = off < ql;
+    row[c] = q0 + (on[c] ? off : 0);
+    pos[c] = on[c] ? pos0 + off : -1;
+    tile_lo[c] = pos0 + row_first + 16 * (ct % rt);
+    tile_hi[c] = tile_lo[c] + 15 < hi ? tile_lo[c] + 15 : hi;
+    const float* q = p.q + (row[c] * p.H + head[c]) * D + 8 * g;
+#pragma unroll
+    for (int u = 0; u < KS; ++u) {
+      qf[c][u] = zero_bf16x8();
+      if (u < nks && on[c]) {
+        const f32x4 a = ld_global<f32x4>(q + 32 * u), b = ld_global<f32x4>(q + 32 * u + 4);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) qf[c][u][j] = (bf16)a[j], qf[c][u][4 + j] = (bf16)b[j];
+      }
+    }
+  }
+  int blks = ids_from(0);
+  // staging: 16-byte pieces of the page's keys (rows G D apart) and of its transposed values (contiguous)
+  const bf16* kc = reinterpret_cast<const bf16*>(p.k);
+  const int k16 = D / 8;
+  bf16x8 nk[2][KC], nv[2][VC];  // two pages on their way
+  int koff[KC], kdst[KC], vdst[VC];
+#pragma unroll
+  for (int i = 0; i < KC; ++i) {
+    const int idx = tid + 256 * i, kr = idx / k16, c = idx - kr * k16;
+    const bool in = kr < kBS;
+    koff[i] = in ? kr * p.G * D + 8 * c : 0;
+    kdst[i] = in ? kr * ldk + 8 * c : -1;
+  }
+#pragma unroll
+  for (int i = 0; i < VC; ++i) {
+    const int idx = tid + 256 * i;
+    vdst[i] = idx < V * kBS / 8 ? kBS * ldk + (idx / (kBS / 8)) * kTileLdv + 8 * (idx % (kBS / 8)) : -1;
+  }
+  auto request = [&](int it, bf16x8(&rk)[KC], bf16x8(&rv)[VC]) {  // pages past the walk read its last one again
+    if (it < walk && (it & 63) == 0 && it > 0) blks = ids_from(it);
+    const int blk = __builtin_amdgcn_readlane(blks, it < walk ? it & 63 : (walk - 1) & 63);
+    const bf16* kp = kc + ((int64_t)blk * kBS * p.G + kvh) * D;
+    const bf16* vp = vt + ((int64_t)blk * p.G + kvh) * V * kBS;
+#pragma unroll
+    for (int i = 0; i < KC; ++i) rk[i] = ld_global<bf16x8>(kp + koff[i]);
+#pragma unroll
+    for (int i = 0; i < VC; ++i) rv[i] = ld_global<bf16x8>(vp + (vdst[i] >= 0 ? 8 * (tid + 256 * i) : 0));
+  };
+  auto stash = [&](int buf, const bf16x8(&rk)[KC], const bf16x8(&rv)[VC]) {
+    bf16* b = smem + buf * buf_elems;
+#pragma unroll
+    for (int i = 0; i < KC; ++i)
+      if (kdst[i] >= 0) *reinterpret_cast<bf16x8*>(b + kdst[i]) = rk[i];
+#pragma unroll
+    for (int i = 0; i < VC; ++i)
+      if (vdst[i] >= 0) *reinterpret_cast<bf16x8*>(b + vdst[i]) = rv[i];
+  };
+  f32x4 O[2][NT];
+#pragma unroll
+  for (int c = 0; c < 2; ++c)
+#pragma unroll
+    for (int n = 0; n < NT; ++n) O[c][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
+  const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f, cap2 = p.softcap * kLog2e;
+  const float scale2 = p.softcap > 0.f ? p.scale : p.scale * kLog2e;
+  const int wave_lo = tile_lo[0] < tile_lo[1] ? tile_lo[0] : tile_lo[1], wave_hi = tile_hi[0] > tile_hi[1] ? tile_hi[0] : tile_hi[1];
+  auto page_step = [&](int it, bf16x8(&rk)[KC], bf16x8(&rv)[VC], const bf16x8(&tk)[KC], const bf16x8(&tv)[VC]) {
+    const int pg = page_at(it);
+    request(it + 2, rk, rv);
+    if (pg * kBS <= wave_hi) {  // uniform for the wave: some row of it may see this page
+      const bf16* kb = smem + (it & 1) * buf_elems;
+      const bf16* vb = kb + kBS * ldk;
+      f32x4 s0[2], s1[2];
+#pragma unroll
+      for (int c = 0; c < 2; ++c) s0[c] = s1[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int u = 0; u < KS; ++u)
+        if (u < nks) {
+          const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(kb + r * ldk + 32 * u + 8 * g);
+          const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(kb + (16 + r) * ldk + 32 * u + 8 * g);
+#pragma unroll
+          for (int c = 0; c < 2; ++c) {
+            s0[c] = mfma16x16x32(k0, qf[c][u], s0[c]);
+            s1[c] = mfma16x16x32(k1, qf[c][u], s1[c]);
+          }
+        }
+      // uniform: every key of the page is at or before the wave's first row and inside the window of its last one
+      const bool full = pg * kBS + kBS - 1 <= wave_lo && wave_hi - pg * kBS < p.window;
+      bf16x8 pf[2];
+      float corr[2];
+#pragma unroll
+      for (int c = 0; c < 2; ++c) {
+        float sv[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          float sc = (i < 4 ? s0[c][i] : s1[c][i - 4]) * scale2;
+          if (p.softcap > 0.f) sc = cap2 * tanh_fast(sc * cap_inv);
+          sv[i] = sc;
+        }
+        if (!full) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
+            const bool seen = key <= pos[c] && (pos[c] - key < p.window || key < p.keep_first);
+            sv[i] = seen ? sv[i] : -INFINITY;
+          }
+        }
+        corr[c] = softmax_step(sv, m[c], l[c], pf[c]);
+      }
+      if (!__all(corr[0] == 1.0f && corr[1] == 1.0f)) {
+#pragma unroll
+        for (int n = 0; n < NT; ++n)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) O[0][n][i] *= corr[0], O[1][n][i] *= corr[1];
+      }
+#pragma unroll
+      for (int n = 0; n < NT; ++n) {
+        const bf16x8 v = *reinterpret_cast<const bf16x8*>(vb + (16 * n + r) * kTileLdv + 8 * g);
+#pragma unroll
+        for (int c = 0; c < 2; ++c) O[c][n] = mfma16x16x32(v, pf[c], O[c][n]);
+      }
+    }
+    stash((it + 1) & 1, tk, tv);  // page it + 1; that buffer was last read before the previous barrier
+    lds_barrier();
+  };
+  request(0, nk[0], nv[0]);
+  request(1, nk[1], nv[1]);
+  stash(0, nk[0], nv[0]);
+  lds_barrier();
+  for (int it = 0; it < walk; it += 2) {
+    page_step(it, nk[0], nv[0], nk[1], nv[1]);
+    if (it + 1 < walk) page_step(it + 1, nk[1], nv[1], nk[0], nv[0]);  // uniform for the workgroup
+  }
+#pragma unroll
+  for (int c = 0; c < 2; ++c) {
+    if (!on[c]) continue;
+    const int h = head[c];
+    float den = l[c], f = 1.0f;
+    if (p.sink) {
+      const float sk = p.sink[h] * kLog2e, mm = fmaxf(m[c], sk);
+      f = exp2_hw(m[c] - mm);
+      den = l[c] * f + exp2_hw(sk - mm);
+    }
+    float inv = den > 0.f ? f / den * p.out_scale : 0.0f;
+    if (p.gate && !p.gate_wide) inv *= 1.0f / (1.0f + expf(-p.gate[row[c] * p.ldg + h]));
+    bf16* out = reinterpret_cast<bf16*>(p.out) + row[c] * p.ldo + h * V + 4 * g;
+    const float* gw = p.gate_wide ? p.gate + row[c] * p.ldg + h * V + 4 * g : nullptr;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      bf16x4 v;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float o = O[c][n][i] * inv;
+        if (gw) o *= 1.0f / (1.0f + expf(-gw[16 * n + i]));
+        v[i] = (bf16)o;
+      }
+      *reinterpret_cast<bf16x4*>(out + 16 * n) = v;
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------
 // Decode form of the MFMA kernel: one query row per work item, and the heads of ONE key/value group side by side as the
 // 16 columns, so a page of keys and values is read once per group instead of once per head.  The NW waves of a workgroup
 // split the pages (wave, wave + NW, ...) and are merged through LDS.  A decode step has few workgroups and short walks,
 // so the walk is written against latency: a wave reads the ids of its next 64 pages in one load, requests the next
 // page's keys before it needs them (heads up to 128 wide: KB k-steps of both 16-key halves stay in registers), and the
-// values of a page while its scores are being made.  Same key order, masks, bias and epilogue as above.
+// values of a page while its scores are being made.  Same key order, masks, bias and epilogue as above.  Few sequences
+// with long walks: nparts workgroups per (item, group) take a stretch of the walk each, leave sum, maximum and weights in
+// `part`, and a second kernel joins the stretches.
 template <int NT, int KB, int NW, bool EXT>
 __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, const bf16* __restrict__ vt, int rel_lds) {
   extern __shared__ __align__(16) unsigned char smem_raw[];
@@ -483,8 +708,9 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
   const int ldq = D + 8;
   const int rep = p.H / p.G;
   const int kvh = blockIdx.y;
-  const int h0 = kvh * rep + blockIdx.z * 16;                       // first head of this column tile
-  const int cols = rep - (int)blockIdx.z * 16 < 16 ? rep - (int)blockIdx.z * 16 : 16;
+  const int parts = p.nparts > 1 ? p.nparts : 1, ctile = (int)blockIdx.z / parts, part = (int)blockIdx.z - ctile * parts;
+  const int h0 = kvh * rep + ctile * 16;                            // first head of this column tile
+  const int cols = rep - ctile * 16 < 16 ? rep - ctile * 16 : 16;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
   const int seq = p.work_seq[blockIdx.x], off = p.work_tile[blockIdx.x];
   const int ql = p.q_len[seq];
@@ -500,10 +726,12 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
     kept_pages = kept_pages < pg_lo ? kept_pages : pg_lo;
   }
   const int walk = kept_pages + pos / kBS - pg_lo + 1;
-  const int mine = walk > wave ? (walk - wave + NW - 1) / NW : 0;   // pages of this wave
+  const int per = (walk + parts - 1) / parts, start = part * per;   // this partition's stretch of the walk
+  const int stretch = walk - start < per ? walk - start : per;
+  const int mine = stretch > wave ? (stretch - wave + NW - 1) / NW : 0;   // pages of this wave
   const int* bt = p.block_tables + (int64_t)seq * p.max_blocks;
   auto page_at = [&](int it) {  // logical page of this wave's it-th step
-    const int pi = wave + it * NW;
+    const int pi = start + wave + it * NW;
     return pi < kept_pages ? pi : pg_lo + pi - kept_pages;
   };
   auto ids_from = [&](int it0) {  // the physical pages of this wave's steps it0 .. it0 + 63, one per lane
@@ -553,7 +781,9 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
 #pragma unroll
   for (int n = 0; n < NT; ++n) O[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
-  const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f;
+  // scores in log2 units; a cap acts on the plain ones
+  const float cap_inv = p.softcap > 0.f ? 1.0f / p.softcap : 0.f, cap2 = p.softcap * kLog2e;
+  const float scale2 = p.softcap > 0.f ? p.scale : p.scale * kLog2e;
   if (mine > 0) load_keys(__builtin_amdgcn_readlane(blks, 0));
   __syncthreads();
   for (int it = 0; it < mine; ++it) {
@@ -585,7 +815,6 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
       load_keys(__builtin_amdgcn_readlane(blks, (it + 1) & 63));
     }
     float sv[8];
-    float mx = -INFINITY;
     const bool far = EXT && p.rel && pos - (pg * kBS + kBS - 1) >= p.rel_len - 1;
     float bv[8];
     if (EXT && p.rel) bias_entries(bv, far, rel_far, relc, relg, rel_lds, p.rel_len, pos - pg * kBS - 4 * g);
@@ -593,25 +822,13 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
     for (int i = 0; i < 8; ++i) {
       const int key = pg * kBS + (i < 4 ? 4 * g + i : 16 + 4 * g + (i - 4));
       const bool seen = c_ok && key <= pos && (pos - key < p.window || (EXT && key < p.keep_first));
-      float sc = (i < 4 ? s0[i] : s1[i - 4]) * p.scale;
-      if (p.softcap > 0.f) sc = p.softcap * tanh_fast(sc * cap_inv);
-      if (EXT && p.rel) sc += bv[i];
+      float sc = (i < 4 ? s0[i] : s1[i - 4]) * scale2;
+      if (p.softcap > 0.f) sc = cap2 * tanh_fast(sc * cap_inv);
+      if (EXT && p.rel) sc += bv[i] * kLog2e;
       sv[i] = seen ? sc : -INFINITY;
-      mx = fmaxf(mx, sv[i]);
     }
-    mx = rows4_max(mx);
-    const float mn = fmaxf(m, mx);
-    const float corr = mn == -INFINITY ? 1.0f : expf(m - mn);
     bf16x8 pf;
-    float ps = 0.f;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float e = sv[i] == -INFINITY ? 0.0f : expf(sv[i] - mn);
-      ps += e;
-      pf[i] = (bf16)e;
-    }
-    l = l * corr + rows4_sum(ps);
-    m = mn;
+    const float corr = softmax_step(sv, m, l, pf);
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       f32x4 o = O[n];
@@ -637,21 +854,77 @@ __global__ __launch_bounds__(NW * 64) void sink_decode_kernel(SinkAttnParams p, 
   const float2* orp = p.out_rope ? p.out_rope + (int64_t)(pos < p.out_rope_len ? pos : p.out_rope_len - 1) * half : nullptr;
   for (int idx = threadIdx.x; idx < cols * V; idx += NW * 64) {
     const int col = idx / V, d = idx - col * V, h = h0 + col;
-    float mm = p.sink ? p.sink[h] : -INFINITY;
+    const float sk = p.sink && parts == 1 ? p.sink[h] * kLog2e : -INFINITY;
+    float mm = sk;
 #pragma unroll
     for (int w = 0; w < NW; ++w) mm = fmaxf(mm, mg[(w * cols + col) * ldm + V]);
-    float den = p.sink ? expf(p.sink[h] - mm) : 0.f, num = 0.f, nump = 0.f;
+    float den = sk > -INFINITY ? exp2_hw(sk - mm) : 0.f, num = 0.f, nump = 0.f;
     const bool lo_half = d < half;
     const int dp = orp ? (lo_half ? d + half : d - half) : d;
 #pragma unroll
     for (int w = 0; w < NW; ++w) {
       const float* src = mg + (w * cols + col) * ldm;
-      const float f = src[V] == -INFINITY ? 0.f : expf(src[V] - mm);
+      const float f = src[V] == -INFINITY ? 0.f : exp2_hw(src[V] - mm);
       den += src[V + 1] * f;
       num += src[d] * f;
       nump += src[dp] * f;
     }
+    if (parts > 1) {  // the combine kernel finishes: the stretch's sum, its maximum and its weights
+      float* dst = p.part + (((int64_t)blockIdx.x * p.H + h) * parts + part) * ldm;
+      dst[d] = num;
+      if (d == 0) {
+        dst[V] = mm;
+        dst[V + 1] = den;
+      }
+      continue;
+    }
     if (orp) {  // back by the row's position
+      const float2 cs = orp[lo_half ? d : dp];
+      num = lo_half ? num * cs.x + nump * cs.y : num * cs.x - nump * cs.y;
+    }
+    float o = den > 0.f ? num / den : 0.f;
+    if (p.gate) o *= 1.0f / (1.0f + expf(-p.gate[row * p.ldg + (p.gate_wide ? h * V + d : h)]));
+    reinterpret_cast<bf16*>(p.out)[row * p.ldo + h * V + d] = (bf16)(o * p.out_scale);
+  }
+}
+
+// The stretches of a split decode walk joined: one wave per (work item, head).
+__global__ __launch_bounds__(256) void sink_combine_kernel(SinkAttnParams p, int num_work) {
+  const int lane = threadIdx.x & 63;
+  const int item = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= num_work * p.H) return;
+  const int work = item / p.H, h = item - work * p.H, V = p.V, ldm = V + 2;
+  const int seq = p.work_seq[work], off = p.work_tile[work], ql = p.q_len[seq];
+  if (off >= ql) return;
+  const int64_t row = p.q_start[seq] + off;
+  const int pos = p.ctx_len[seq] - ql + off;
+  const float* src = p.part + (int64_t)item * p.nparts * ldm;
+  const float sk = p.sink ? p.sink[h] * kLog2e : -INFINITY;
+  float mm = sk;
+  for (int i = 0; i < p.nparts; ++i) mm = fmaxf(mm, src[i * ldm + V]);
+  float den = p.sink ? exp2_hw(sk - mm) : 0.f;
+  float f[kMaxParts];
+#pragma unroll
+  for (int i = 0; i < kMaxParts; ++i) {
+    f[i] = 0.f;
+    if (i < p.nparts && src[i * ldm + V] > -INFINITY) {
+      f[i] = exp2_hw(src[i * ldm + V] - mm);
+      den += src[i * ldm + V + 1] * f[i];
+    }
+  }
+  const int half = V >> 1;
+  const float2* orp = p.out_rope ? p.out_rope + (int64_t)(pos < p.out_rope_len ? pos : p.out_rope_len - 1) * half : nullptr;
+  for (int d = lane; d < V; d += 64) {
+    const bool lo_half = d < half;
+    const int dp = orp ? (lo_half ? d + half : d - half) : d;
+    float num = 0.f, nump = 0.f;
+#pragma unroll
+    for (int i = 0; i < kMaxParts; ++i)
+      if (i < p.nparts) {
+        num += src[i * ldm + d] * f[i];
+        nump += src[i * ldm + dp] * f[i];
+      }
+    if (orp) {
       const float2 cs = orp[lo_half ? d : dp];
       num = lo_half ? num * cs.x + nump * cs.y : num * cs.x - nump * cs.y;
     }
@@ -680,8 +953,11 @@ void launch_decode_waves(int num_work, const SinkAttnParams& p, const bf16* vt, 
     rel_lds = (int)(want < room ? want : room);
     lds += cols * rel_lds * sizeof(float);
   }
-  hipLaunchKernelGGL((sink_decode_kernel<NT, 4, NW, EXT>), dim3(num_work, p.G, (rep + 15) / 16), dim3(NW * 64), lds, st, p,
-                     vt, rel_lds);
+  const int parts = p.nparts > 1 ? p.nparts : 1;
+  hipLaunchKernelGGL((sink_decode_kernel<NT, 4, NW, EXT>), dim3(num_work, p.G, (rep + 15) / 16 * parts), dim3(NW * 64), lds,
+                     st, p, vt, rel_lds);
+  if (parts > 1)
+    hipLaunchKernelGGL(sink_combine_kernel, dim3((num_work * p.H + 3) / 4), dim3(256), 0, st, p, num_work);
 }
 
 template <int NT>
@@ -747,11 +1023,34 @@ extern "C" hipError_t dsse_sink_flash(int num_work, const dsse::SinkAttnParams* 
   return hipGetLastError();
 }
 
+// shared-page form: work_tile counts tiles of 16 rt rows, hb rt = 8; D and V up to 128, no bias and no output rotation
+extern "C" hipError_t dsse_sink_tile(int num_work, const dsse::SinkAttnParams* p, const void* vt, int rt, hipStream_t st) {
+  if (num_work <= 0 || p->H <= 0) return hipSuccess;
+  if ((rt != 2 && rt != 4 && rt != 8) || p->H % p->G || (p->H / p->G) % (8 / rt)) return hipErrorInvalidValue;
+  if (p->f32 || p->D % 32 || p->V % 16 || p->D > dsse::kTileWidth || p->V > dsse::kTileWidth || p->rel || p->out_rope ||
+      num_work > 65535)
+    return hipErrorInvalidValue;
+  const int hb = 8 / rt;
+  const dim3 grid(p->H / hb, num_work);
+  const size_t lds = 2 * sizeof(bf16) * (dsse::kBS * (size_t)(p->D + 8) + (size_t)p->V * dsse::kTileLdv);
+  const bf16* v = reinterpret_cast<const bf16*>(vt);
+  switch (p->V / 16) {
+#define DSSE_TILE_CASE(n) \
+  case n: hipLaunchKernelGGL(dsse::sink_tile_kernel<n>, grid, dim3(256), lds, st, *p, v, hb, rt); break;
+    DSSE_TILE_CASE(1) DSSE_TILE_CASE(2) DSSE_TILE_CASE(3) DSSE_TILE_CASE(4) DSSE_TILE_CASE(5) DSSE_TILE_CASE(6)
+    DSSE_TILE_CASE(7) DSSE_TILE_CASE(8)
+#undef DSSE_TILE_CASE
+    default: return hipErrorInvalidValue;
+  }
+  return hipGetLastError();
+}
+
 // decode form: work_tile counts single rows; V / 16 as above, LDS for at least four waves
 extern "C" hipError_t dsse_sink_decode(int num_work, const dsse::SinkAttnParams* p, const void* vt, hipStream_t st) {
   if (num_work <= 0 || p->H <= 0) return hipSuccess;
   if (p->f32 || p->D % 32 || p->V % 16 || p->V > 512 || p->D > 512 || p->H % p->G) return hipErrorInvalidValue;
   if (dsse::decode_lds(*p, 4) > dsse::kFlashLds) return hipErrorInvalidValue;
+  if (p->nparts > dsse::kMaxParts || (p->nparts > 1 && !p->part)) return hipErrorInvalidValue;
   const bf16* v = reinterpret_cast<const bf16*>(vt);
   switch (p->V / 16) {
 #define DSSE_DECODE_CASE(n) case n: dsse::launch_decode<n>(num_work, *p, v, st); break;

@@ -133,6 +133,9 @@ from .weights import LayeredWeights
 
 ATTN_ROWS_TILE = 4    # query rows per work item of the row-wise attention kernel (prompt portions)
 FLASH_DECODE_WAVES = 512  # waves a decode attention launch aims for (two per CU)
+SINK_DECODE_GROUPS = 512  # workgroups a decode launch of the sink attention aims for (two per CU)
+SINK_TILE_GROUPS = 256    # workgroups from which prompt portions take the shared-page form: below, one-tile items fill more
+SINK_DECODE_PAGES = 32    # fewest pages of a full cache that a workgroup's stretch of a split walk is worth
 SINK_ROWS_TILE = 16   # query rows per work item of the sink attention's MFMA form (one head per wave)
 FLASH_ROWS_TILE = 4   # query rows per work item of the MFMA attention form, x 4 heads = 16 columns: a page of keys is
                       # read once for four heads (16 rows x 1 head re-read it per head: 2-3x the time at 16 heads)
@@ -157,6 +160,7 @@ class LayeredRunner(RunnerBase):
         self.use_graphs = (self.device.type == "cuda") if use_graphs is None else use_graphs
         cfg, dev = self.cfg, self.device
         self._init_slots(max_batch, self.max_blocks, cfg.vocab_size, dev, self.comm)
+        self._tile_rows = []   # row counts of the shared-page attention's work items that this design's layers use
         self.num_blocks = num_blocks
         self.prenorm = getattr(cfg, "family", "") == "surodra"   # pre-norm blocks with matrix-state mixers
         self.multistream = getattr(cfg, "family", "") == "dironex"  # pre-norm blocks on several residual streams
@@ -1013,6 +1017,7 @@ class LayeredRunner(RunnerBase):
         cfg, dev = self.cfg, self.device
         self.runs = cfg.runs()
         kv, mem, convs, self._rope, self._temp = {}, {}, {}, {}, {}
+        atts = {L.mixer if L.kind == "conv_attention" else L.mixer.left for L in cfg.layers}
         for r in self.runs:
             L, m = cfg.layers[r.layer], cfg.layers[r.layer].mixer
             if L.kind == "conv_attention":
@@ -1030,6 +1035,10 @@ class LayeredRunner(RunnerBase):
                  ops.sink_flash_lds(dm) <= LDS_BYTES]
         self.kv = PagedKVCache(kv, self.num_blocks, dev, self.dtype, transposed=flash)
         self.state = MemoryStateCache(mem, convs, self.max_batch, dev)
+        self._tile_rows = sorted({ops.sink_tile_rows(self.dtype, a.heads, a.kv_heads, a.dim, a.vdim) for a in atts} - {0})
+        words = max((B * a.heads * self._walk_parts(B, a) * (a.vdim + 2) for B in range(1, self.max_batch + 1) for a in atts),
+                    default=0)
+        self._walk_part = torch.zeros(max(1, words), device=dev, dtype=torch.float32)
         self._moe_layers = [i for i, L in enumerate(cfg.layers) if hasattr(L.mlp, "experts") and L.weights_of == i]
 
     def _memory_buffers(self, M: int) -> dict:
@@ -1053,8 +1062,9 @@ class LayeredRunner(RunnerBase):
                 mm = max(mm, ops.memory_work_floats(M, m.right.heads, m.right.vdim, self.max_batch))
             if L.mlp is not None and not hasattr(L.mlp, "experts"):
                 ff = max(ff, L.mlp.ff)
-        d = {"big": torch.zeros(M * big, **f32), "qa": torch.zeros(M * qa, **f32), "ao": torch.zeros(M * ao, **el),
-             "mm": torch.zeros(mm, **f32), "up": torch.zeros(M * ff, **f32), "h": torch.zeros(M * ff, **el)}
+        # `empty`: written whole before they are read; rows of inactive decode slots in `qa` and `ao` never are
+        d = {"big": torch.empty(M * big, **f32), "qa": torch.zeros(M * qa, **f32), "ao": torch.zeros(M * ao, **el),
+             "mm": torch.empty(mm, **f32), "up": torch.empty(M * ff, **f32), "h": torch.empty(M * ff, **el)}
         moe = [cfg.layers[i].mlp for i in self._moe_layers]
         if moe:
             slots = [f.top + (f.shared_ff > 0) for f in moe]
@@ -1064,7 +1074,7 @@ class LayeredRunner(RunnerBase):
                       "tkw": {f.top: torch.full((M * f.top,), 1.0 / f.top, **f32) for f in moe},
                       "mo_sorted": [torch.zeros(t * 64, **i32) for t in tiles],
                       "mo_tile": [torch.zeros(t, **i32) for t in tiles], "mo_n": [torch.zeros(1, **i32) for _ in moe],
-                      "mo_h": torch.zeros(M * max(slots), ldh, **el), "mo_o": torch.zeros(M * max(slots) * W, **f32)})
+                      "mo_h": torch.empty(M * max(slots), ldh, **el), "mo_o": torch.empty(M * max(slots) * W, **f32)})
         return d
 
     def _expert_lists(self, ids, M: int, d: dict) -> None:
@@ -1094,18 +1104,29 @@ class LayeredRunner(RunnerBase):
         return o, S
 
     def _sink_rows(self, ri: int, a, qa, sink, gate, out, groups: list, out_scale: float = 1.0) -> None:
-        """Causal sink attention of every sequence group over this run's pages: the MFMA form for prompt portions, its
-        decode form for decode rows, the row form for head widths that neither covers."""
+        """Causal sink attention of every sequence group over this run's pages: the shared-page MFMA form (wide heads: the
+        one-tile form) for prompt portions, the decode form for decode rows, the row form for head widths that none covers."""
         kc, vc, vt = self.kv.k[ri], self.kv.v[ri], self.kv.vt.get(ri)
         for g in groups:
-            if vt is not None and g["qt"] > 1:
+            nparts = 1
+            rows = ops.sink_tile_rows(self.dtype, a.heads, a.kv_heads, a.dim, a.vdim)
+            if vt is not None and g["qt"] > 1 and rows and g["tiles"][rows][0].numel() * a.heads * rows >= 128 * SINK_TILE_GROUPS:
+                work, form = g["tiles"][rows], (rows, vt, False)
+            elif vt is not None and g["qt"] > 1:
                 work, form = (g["hs"], g["ht"]), (SINK_ROWS_TILE, vt, False)
             elif vt is not None and ops.sink_decode_ok(self.dtype, a.heads, a.kv_heads, a.dim, a.vdim):
                 work, form = (g["ws"], g["wt"]), (1, vt, False)
+                nparts = self._walk_parts(g["ws"].numel(), a)
             else:
                 work, form = (g["ws"], g["wt"]), (g["qt"], None, False)
             ops.sink_attention(qa, kc, vc, g["bt"], g["qs"], g["ql"], g["ctx"], *work, sink, gate, out, NO_WINDOW, a.scale,
-                               *form, out_scale=out_scale)
+                               *form, out_scale=out_scale, part=self._walk_part if nparts > 1 else None, nparts=nparts)
+
+    def _walk_parts(self, rows: int, a) -> int:
+        """Workgroups that share a decode row's walk over all of its pages: as many as fill the chip, as long as each has
+        pages enough when the sequence is as long as it may become (a captured step serves every length)."""
+        fill = SINK_DECODE_GROUPS // max(1, rows * a.kv_heads * -(-(a.heads // a.kv_heads) // 16))
+        return max(1, min(16, fill, self.max_blocks // SINK_DECODE_PAGES))
 
     def _qkv_rows(self, ri: int, a, big, taps, vdim: int, rope, temp, slots, qa, groups: list) -> None:
         """q to a buffer, k and v into this run's pages, per sequence group (prompt portions in tiles of rows)."""
@@ -1384,7 +1405,13 @@ class LayeredRunner(RunnerBase):
             ht += list(range(nh))
             row += m
         T = row
-        lists = np.asarray(qs + ql + ctx + ss + ws + wt + fs + ft + hs + ht + last, dtype=np.int64)
+        shared = []  # shared-page attention: the longest walks first
+        for R in self._tile_rows:
+            items = [(i, t) for i, s in enumerate(seqs) for t in range(math.ceil(len(s.tokens) / R))]
+            items.sort(key=lambda it: -(seqs[it[0]].start_pos + it[1] * R))
+            shared += [("tile_seq", R, [i for i, _ in items]), ("tile_no", R, [t for _, t in items])]
+        lists = np.asarray(qs + ql + ctx + ss + ws + wt + fs + ft + hs + ht + last + [x for _, _, xs in shared for x in xs],
+                           dtype=np.int64)
         meta = torch.from_numpy(np.concatenate(ids_l + pos_l + slots_l + prev_l + [lists]).astype(np.int32))
         if self.device.type == "cuda":
             meta = meta.pin_memory().to(self.device, non_blocking=True)
@@ -1394,6 +1421,9 @@ class LayeredRunner(RunnerBase):
                         ("ctx", n), ("ss", n), ("ws", len(ws)), ("wt", len(ws)), ("fs", len(fs)), ("ft", len(fs)),
                         ("hs", len(hs)), ("ht", len(hs)), ("last", len(last))):
             d[name], o = meta[o:o + k], o + k
+        for name, R, xs in shared:
+            d.setdefault(name, {})[R], o = meta[o:o + len(xs)], o + len(xs)
+        d["tiles"] = {R: (d["tile_seq"][R], d["tile_no"][R]) for R in self._tile_rows}
         d["bt"] = bt
         d["qt"] = ATTN_ROWS_TILE
         d["rows"] = (row0, T)   # the packed rows of these portions

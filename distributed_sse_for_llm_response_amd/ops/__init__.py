@@ -282,6 +282,6 @@ def kernel_checks(clear: bool = True, raise_on_error: bool = True) -> list:
 from .layers import (conv_state, embed_rows, gate_math, gated_act, gated_head_norm, gemm_rm, latent_attention,  # noqa: E402,F401
                      latent_flash_ok, latent_flash_part_floats, latent_kv_write, logit_cap, lru_scan, matrix_scan, matrix_scan_chunked,
                      moe_ffn, moe_grouped, moe_router, moe_topk, norm_rope_rows, rms_mix, scalar_norm, sink_attention,
-                     sink_flash_ok, sink_flash_lds, sink_decode_ok, moe_route_rows, stream_step, stream_mix, act_rows, moe_route, embed_pair_rows, add_norm_rows,
+                     sink_flash_ok, sink_flash_lds, sink_tile_rows, sink_decode_ok, moe_route_rows, stream_step, stream_mix, act_rows, moe_route, embed_pair_rows, add_norm_rows,
                      token_gate_rows, token_side_rows, token_side_fits, qkv_rows, conv_qkv_rows,
                      matrix_memory, memory_chunk_ok, memory_work_floats, moe_table_lists)

@@ -209,6 +209,15 @@ def sink_decode_ok(dtype, heads: int, kv_heads: int, dim: int, vdim: int) -> boo
         16 * (dim + 8) * 2 + 4 * min(16, heads // kv_heads) * (vdim + 2) * 4 <= 64 * 1024
 
 
+def sink_tile_rows(dtype, heads: int, kv_heads: int, dim: int, vdim: int) -> int:
+    """Query rows per work item of the shared-page form of sink_attention (32, 64 or 128: the heads of a key/value group
+    that fill the rest of eight 16-column tiles), 0 for shapes it does not cover."""
+    if not sink_flash_ok(dtype, dim, vdim) or dim > 128 or vdim > 128:
+        return 0
+    rep = heads // kv_heads
+    return 32 if rep % 4 == 0 else (64 if rep % 2 == 0 else 128)
+
+
 def sink_flash_lds(dim: int) -> int:
     """LDS bytes of the MFMA form before a distance bias: four waves' query tiles."""
     return 4 * 16 * (dim + 8) * 2
@@ -216,12 +225,13 @@ def sink_flash_lds(dim: int) -> int:
 
 def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile, sink, gate, out,
                    window: int, scale: float, qt: int, vt=None, split: bool = False, softcap: float = 0.0, out_rope=None,
-                   rel=None, keep_first: int = 0, out_scale: float = 1.0):
+                   rel=None, keep_first: int = 0, out_scale: float = 1.0, part=None, nparts: int = 1):
     """Causal softmax attention of q [T, H, D] over paged keys [pages, 32, G, D] and values [pages, 32, G, V] (grouped
     heads), scores and weights in fp32; sink [H] adds exp(sink) to each head's denominator, gate [T, H] multiplies the
     head's output by its sigmoid.  `qt` query rows per work item (work_seq, work_tile).  With vt (transposed value
     pages [pages, G, V, 32], sink_flash_ok shapes, qt = 16): the MFMA form; split (V <= 128) lets the four waves of a
-    workgroup share one (tile, head) and split its pages, for decode steps.  With vt and qt = 1: the decode form
+    workgroup share one (tile, head) and split its pages, for decode steps.  With vt and qt = sink_tile_rows: the shared-page
+    form (no rel, no out_rope), a page staged once for all rows and heads of an item.  With vt and qt = 1: the decode form
     (sink_decode_ok shapes), one row per item, the heads of a key/value group side by side, pages split over the waves of
     a workgroup.  softcap > 0: scores
     softcap * tanh(scale q.k / softcap).  out_rope ([positions, V / 2, 2] (cos, sin), rotate-half pairs over the whole
@@ -230,11 +240,12 @@ def sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, wor
     MFMA form then needs V % 32 == 0).  rel [H, N] (fp32): the entry of the key's distance to the query (the last one for
     distances from N - 1 on) is added to the score.  keep_first: the sequence's first keep_first keys stay visible when the
     window has passed them.  A gate of H * V columns multiplies the heads element by element.  out (rows may be a column
-    slice of a wider buffer) is multiplied by out_scale before it is rounded."""
+    slice of a wider buffer) is multiplied by out_scale before it is rounded.  part (fp32, [work items, H, nparts, V + 2]):
+    the decode form splits each row's walk over nparts (at most 16) workgroups and joins them in a second launch."""
     if _hip(q):
         torch.ops.dsse.sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, work_seq, work_tile,
                                       sink, gate, out, window, scale, qt, vt, split, softcap, out_rope, rel, keep_first,
-                                      out_scale)
+                                      out_scale, part, nparts)
     else:
         lref.sink_attention(q, kcache, vcache, block_tables, q_start, q_len, ctx_len, sink, gate, out, window, scale, vt,
                             softcap, out_rope, rel, keep_first, out_scale)

@@ -235,7 +235,7 @@ def test_gelu_rows(dtype):
 
 
 @pytest.mark.parametrize("wide_gate", [False, True])
-@pytest.mark.parametrize("form", ["row", "row fp32", "tiles", "split", "decode"])
+@pytest.mark.parametrize("form", ["row", "row fp32", "tiles", "split", "decode", "decode in 3 parts", "decode in 16 parts"])
 def test_attention_into_a_wider_row(form, wide_gate):
     """Every form of the paged attention with an output that is a column slice of a wider row, times a scale, with a
     sink."""
@@ -258,9 +258,41 @@ def test_attention_into_a_wider_row(form, wide_gate):
     want = torch.zeros(T, H * V + 16, dtype=dtype)
     lref.sink_attention(q, kc, vc, bt, *meta, sink, gate, want[:, 8:8 + H * V].unflatten(1, (H, V)), 10 ** 9, 0.2, out_scale=-1.5)
     qt, args = {"row": (4, (None, False)), "row fp32": (4, (None, False)), "tiles": (16, (c(vt), False)),
-                "split": (16, (c(vt), True)), "decode": (1, (c(vt), False))}[form]
+                "split": (16, (c(vt), True))}.get(form, (1, (c(vt), False)))
+    nparts = int(form.split()[2]) if "parts" in form else 1   # sixteen: more than the sequences have pages
     got = torch.zeros(T, H * V + 16, dtype=dtype, device=dev())
     ops.sink_attention(c(q), c(kc), c(vc), c(bt), *map(c, meta), *map(c, tiles(ql, qt)), c(sink), c(gate),
-                       got[:, 8:8 + H * V].unflatten(1, (H, V)), 10 ** 9, 0.2, qt, *args, out_scale=-1.5)
+                       got[:, 8:8 + H * V].unflatten(1, (H, V)), 10 ** 9, 0.2, qt, *args, out_scale=-1.5,
+                       part=torch.zeros(2 * H * nparts * (V + 2), device=dev()) if nparts > 1 else None, nparts=nparts)
     close(got, want, 1e-5 if dtype == torch.float32 else 2e-2)
     assert not got[:, :8].any() and not got[:, 8 + H * V:].any()
+
+
+@pytest.mark.parametrize("H,G,D,V", [(4, 2, 32, 48), (6, 6, 64, 16), (8, 2, 128, 128), (8, 1, 96, 112), (3, 1, 64, 64), (1, 1, 128, 80)])
+@pytest.mark.parametrize("window,keep,cap", [(10 ** 9, 0, 0.0), (40, 0, 0.0), (33, 5, 0.0), (70, 40, 3.0), (1, 0, 0.0)])
+def test_shared_page_attention(H, G, D, V, window, keep, cap):
+    """The shared-page form for prompt portions: sequences that start, continue in the middle of a page and are shorter
+    than a tile, one inactive; windows, kept keys, caps, sinks and both kinds of gate."""
+    g = torch.Generator().manual_seed(8)
+    ctx, ql = [150, 300, 9, 2], [150, 131, 0, 2]
+    T = sum(ql)
+    need = [math.ceil(n / PAGE) for n in ctx]
+    perm = torch.randperm(sum(need) + 2, generator=g).tolist()
+    bt, k = torch.zeros(4, max(need), dtype=torch.int32), 0
+    for s, n in enumerate(need):
+        bt[s, :n], k = i32(perm[k:k + n]), k + n
+    q = torch.randn(T, H, D, generator=g)
+    kc, vc = (torch.randn(sum(need) + 2, PAGE, G, n, generator=g).to(torch.bfloat16) for n in (D, V))
+    vt = torch.zeros(sum(need) + 2, G, V, PAGE, dtype=torch.bfloat16)
+    for off in range(PAGE):
+        vt[:, :, :, lref.vt_position(off)] = vc[:, off]
+    meta = (i32([0, ql[0], 281, 281]), i32(ql), i32(ctx))
+    rows = ops.sink_tile_rows(torch.bfloat16, H, G, D, V)
+    assert rows in (32, 64, 128)
+    for sink, cols in ((torch.randn(H, generator=g), H * V), (None, H), (torch.zeros(H), None)):
+        gate = torch.randn(T, cols, generator=g) if cols else None
+        want, got = torch.zeros(T, H, V, dtype=torch.bfloat16), torch.zeros(T, H, V, dtype=torch.bfloat16, device=dev())
+        lref.sink_attention(q, kc, vc, bt, *meta, sink, gate, want, window, 0.2, softcap=cap, keep_first=keep, out_scale=0.6)
+        ops.sink_attention(c(q), c(kc), c(vc), c(bt), *map(c, meta), *map(c, tiles(ql, rows)), c(sink), c(gate), got, window, 0.2,
+                           rows, c(vt), softcap=cap, keep_first=keep, out_scale=0.6)
+        close(got, want, 2e-2)

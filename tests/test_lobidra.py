@@ -774,7 +774,7 @@ def test_long_decoding(device):
     ("odd sizes", config([att(heads=6, kv_heads=3, dim=14, conv=5, rot={"base": 20.0, "dims": 14}, mlp=moe(experts=9, top=4, ff=7, shared=5)),
                           par(heads=9, kv_heads=3, dim=13, vdim=11, mheads=5, mdim=9, mvdim=15, mlp=dense(17))], width=19, vocab=23)),
     ("sizes that vector loads and the MFMA forms like", config(
-        [att(heads=8, kv_heads=2, dim=64, conv=4, scale=0.2, rot={"base": 900.0, "dims": 32}, mlp=moe(experts=8, top=2, ff=64, shared=32)),
+        [att(heads=12, kv_heads=4, dim=64, conv=4, scale=0.2, rot={"base": 900.0, "dims": 32}, mlp=moe(experts=9, top=2, ff=64, shared=32)),
          par(heads=8, kv_heads=4, dim=64, vdim=32, scale=0.2, mheads=4, mdim=32, mvdim=64, mlp=moe(experts=4, top=1, ff=32, shared=0)),
          par(heads=2, kv_heads=2, dim=32, vdim=80, mheads=3, mdim=96, mvdim=48, mlp=dense(64))], width=64, vocab=96)),
     ("wide heads on the row form and on the walk", config(
